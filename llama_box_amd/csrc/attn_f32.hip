@@ -42,9 +42,11 @@ __device__ __forceinline__ float mask_ld(const char * __restrict__ mrow, const i
     return mtype == GGML_TYPE_F16 ? h2f(((const uint16_t *) mrow)[j]) : ((const float *) mrow)[j];
 }
 
-// the additive term of a visible cell: the mask's value itself, or — with a per-head distance penalty (r1, r2) — the mask's value read as the distance
-// between query and cell: -r1 ln(1 + r2 distance)
-__device__ __forceinline__ float mask_term(const float mv, const bool pen, const float r1, const float r2) { return pen ? -r1 * logf(1.0f + r2 * mv) : mv; }
+// the additive term of a visible cell: the mask's value itself, or — with a per-head distance penalty — the mask's value read as the distance between query and cell:
+// -r1 ln(1 + r2 distance), or -r1 distance (kernels.h: ATTN_PEN_LOG, ATTN_PEN_LINEAR)
+__device__ __forceinline__ float mask_term(const float mv, const int pen, const float r1, const float r2) {
+    return pen == 0 ? mv : pen == ATTN_PEN_LINEAR ? -(r1 * mv) : -r1 * logf(1.0f + r2 * mv);
+}
 
 // the score of a visible cell before the mask's term: dot product x scale x a per-head factor, then optionally soft-capped (cap tanh(. / cap))
 __device__ __forceinline__ float attn_score(const float d, const float scale, const float temp, const float cap) {
@@ -116,7 +118,7 @@ __device__ __forceinline__ void attn_f32_pv8(const float p, const uint64_t live,
 
 template <int KT, int VT>
 __global__ void __launch_bounds__(256) k_attn_f32_rows(const tdesc q, const tdesc k, const tdesc v, const tdesc mask, const int has_mask, const float * __restrict__ sinks,
-                                                       const float * __restrict__ r12, const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap) {
+                                                       const float * __restrict__ r12, const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap, const int pen_kind) {
     __shared__ float qs[ATTN_F32_MAX_D];
     __shared__ float part_acc[4][ATTN_F32_MAX_D];
     __shared__ float part_m[4], part_l[4];
@@ -131,8 +133,8 @@ __global__ void __launch_bounds__(256) k_attn_f32_rows(const tdesc q, const tdes
     const char * mrow = has_mask ? mask.data + t * mask.nb[1] : nullptr;
     const char * kbase = k.data + g * k.nb[2];
     const char * vbase = v.data + g * v.nb[2];
-    const bool pen = r12 != nullptr;
-    const float r1 = pen ? r12[h] : 0.0f, r2 = pen ? r12[q.ne[2] + h] : 0.0f;
+    const int pen = r12 ? pen_kind : 0;
+    const float r1 = pen ? r12[h] : 0.0f, r2 = pen == ATTN_PEN_LOG ? r12[q.ne[2] + h] : 0.0f;
     // (value rows of 256 .. 512 two-byte entries: a lane owns eight neighbouring columns)
     const bool v_vec8 = VT != GGML_TYPE_F32 && DV > 256 && DV <= 512 && (DV % 8) == 0 && (v.nb[1] % 16) == 0 && (v.nb[2] % 16) == 0 && (((uintptr_t) v.data) & 15) == 0;
     const bool k_vec = KT != GGML_TYPE_F32 && (DK % 8) == 0 && (k.nb[1] % 16) == 0 && (k.nb[2] % 16) == 0 && (((uintptr_t) k.data) & 15) == 0;
@@ -225,7 +227,7 @@ __global__ void __launch_bounds__(256) k_attn_f32_rows(const tdesc q, const tdes
 // prompt batches: 64 query tokens x one head per workgroup; K / V blocks of 64 cells staged in LDS as f32
 template <int KT, int VT, int DKP, int DVP>   // DKP / DVP: head sizes rounded up to a multiple of 32 / 64 (LDS row lengths)
 __global__ void __launch_bounds__(256) k_attn_f32_tile(const tdesc q, const tdesc k, const tdesc v, const tdesc mask, const float * __restrict__ sinks,
-                                                       const float * __restrict__ r12, const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap) {
+                                                       const float * __restrict__ r12, const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap, const int pen_kind) {
     constexpr int QT = 64, KB = 64, QW = QT / 4;  // queries per workgroup, cells per block, queries per wave
     constexpr int KS = DKP + 1;                   // K row stride in LDS (odd: lanes that read column i of 64 different rows hit 64 different banks)
     extern __shared__ float lds[];
@@ -240,8 +242,8 @@ __global__ void __launch_bounds__(256) k_attn_f32_tile(const tdesc q, const tdes
     const int64_t g = h / (q.ne[2] / k.ne[2]);
     const char * kbase = k.data + g * k.nb[2];
     const char * vbase = v.data + g * v.nb[2];
-    const bool pen = r12 != nullptr;
-    const float r1 = pen ? r12[h] : 0.0f, r2 = pen ? r12[q.ne[2] + h] : 0.0f;
+    const int pen = r12 ? pen_kind : 0;
+    const float r1 = pen ? r12[h] : 0.0f, r2 = pen == ATTN_PEN_LOG ? r12[q.ne[2] + h] : 0.0f;
     for (int e = threadIdx.x; e < QT * DKP; e += 256) {
         const int qi = e / DKP, i = e % DKP;
         const int64_t t = t0 + qi;
@@ -352,7 +354,7 @@ __device__ __forceinline__ uint32_t att_bf16_bits(const float f) {
 }
 template <int DK16, int DVT>
 __global__ void __launch_bounds__(256) k_attn_mma_bf16(const tdesc q, const tdesc k, const tdesc v, const tdesc mask, const float * __restrict__ sinks, const float * __restrict__ r12, const tdesc dst,
-                                                       const float scale, const float * __restrict__ sig, const float softcap) {
+                                                       const float scale, const float * __restrict__ sig, const float softcap, const int pen_kind) {
     constexpr int VS = 36;  // V^T row stride in LDS (bf16 elements): 72 bytes keeps the 8-byte reads aligned and spreads the rows over the banks
     __shared__ __attribute__((aligned(16))) uint16_t Vt[DVT * 32 * VS];
     __shared__ int flag[2];
@@ -378,8 +380,8 @@ __global__ void __launch_bounds__(256) k_attn_mma_bf16(const tdesc q, const tdes
             qf[s] = make_uint4(b[0] | (b[1] << 16), b[2] | (b[3] << 16), b[4] | (b[5] << 16), b[6] | (b[7] << 16));
         }
     }
-    const bool pen = r12 != nullptr;
-    const float r1 = pen ? r12[h] : 0.0f, r2 = pen ? r12[q.ne[2] + h] : 0.0f;
+    const int pen = r12 ? pen_kind : 0;
+    const float r1 = pen ? r12[h] : 0.0f, r2 = pen == ATTN_PEN_LOG ? r12[q.ne[2] + h] : 0.0f;
     const bool sgm = sig != nullptr;
     const float s_temp = sgm ? sig[h] : 1.0f, s_bias = sgm ? sig[q.ne[2] + h] : 0.0f;
     float m = sgm ? 0.0f : (sinks ? sinks[h] : ATTN_F32_LOW), l = (sinks && !sgm) ? 1.0f : 0.0f;
@@ -518,7 +520,7 @@ __global__ void __launch_bounds__(256) k_attn_mma_bf16(const tdesc q, const tdes
 // 32-entry value tiles per wave.
 template <int DKQ, int DVQ>
 __global__ void __launch_bounds__(256) k_attn_mma_bf16_wide(const tdesc q, const tdesc k, const tdesc v, const tdesc mask, const float * __restrict__ sinks, const float * __restrict__ r12,
-                                                            const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap) {
+                                                            const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap, const int pen_kind) {
     constexpr int VS = 36;
     constexpr int DVT = 4 * DVQ;
     __shared__ __attribute__((aligned(16))) uint16_t Vt[DVT * 32 * VS];
@@ -545,8 +547,8 @@ __global__ void __launch_bounds__(256) k_attn_mma_bf16_wide(const tdesc q, const
             qf[s] = make_uint4(b[0] | (b[1] << 16), b[2] | (b[3] << 16), b[4] | (b[5] << 16), b[6] | (b[7] << 16));
         }
     }
-    const bool pen = r12 != nullptr;
-    const float r1 = pen ? r12[h] : 0.0f, r2 = pen ? r12[H + h] : 0.0f;
+    const int pen = r12 ? pen_kind : 0;
+    const float r1 = pen ? r12[h] : 0.0f, r2 = pen == ATTN_PEN_LOG ? r12[H + h] : 0.0f;
     const bool sgm = sig != nullptr;
     const float s_temp = sgm ? sig[h] : 1.0f, s_bias = sgm ? sig[q.ne[2] + h] : 0.0f;
     float m = sgm ? 0.0f : (sinks ? sinks[h] : ATTN_F32_LOW), l = (sinks && !sgm) ? 1.0f : 0.0f;
@@ -719,7 +721,7 @@ bool attn_f32_applies(const tdesc & q, const tdesc & k, const tdesc & v, const t
 
 template <int KT, int VT>
 static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const float * sinks, const float * r12, const tdesc & dst, float scale,
-                              const float * sig, float softcap) {
+                              const float * sig, float softcap, int pen_kind) {
     const int64_t n_q = q.ne[1], H = q.ne[2];
     const int DK = (int) q.ne[0], DV = (int) v.ne[0];
     if constexpr (KT == GGML_TYPE_BF16 && VT == GGML_TYPE_BF16) {
@@ -727,7 +729,7 @@ static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, c
         if (mma_on && attn_mma_bf16_wide_ok(q, k, v, mask, dst)) {  // one shared key/value head with wide rows (latent attention): four waves per 32 (token, head) pairs
             const dim3 grid((unsigned) ((n_q * H + 31) / 32));
             const int dkq = ((DK + 15) / 16 + 3) / 4, dvq = ((DV + 31) / 32 + 3) / 4;  // per wave: 16-entry key groups (<= 10), 32-entry value tiles (<= 4)
-#define MI_ATT_WIDE(A, B) hipLaunchKernelGGL((k_attn_mma_bf16_wide<A, B>), grid, dim3(256), 0, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap)
+#define MI_ATT_WIDE(A, B) hipLaunchKernelGGL((k_attn_mma_bf16_wide<A, B>), grid, dim3(256), 0, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap, pen_kind)
             const int a = dkq <= 3 ? 3 : (dkq <= 5 ? 5 : 10), b = dvq <= 1 ? 1 : (dvq <= 2 ? 2 : 4);
             if (a == 3 && b == 1) MI_ATT_WIDE(3, 1); else if (a == 3 && b == 2) MI_ATT_WIDE(3, 2); else if (a == 3) MI_ATT_WIDE(3, 4);
             else if (a == 5 && b == 1) MI_ATT_WIDE(5, 1); else if (a == 5 && b == 2) MI_ATT_WIDE(5, 2); else if (a == 5) MI_ATT_WIDE(5, 4);
@@ -745,7 +747,7 @@ static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, c
             const dim3 grid((unsigned) ((n_q + 32 * nw - 1) / (32 * nw)), (unsigned) H);
             const dim3 block((unsigned) (64 * nw));
             const int dk16 = (DK + 15) / 16, dvt = (DV + 31) / 32;
-#define MI_ATT_MMA(A, B) hipLaunchKernelGGL((k_attn_mma_bf16<A, B>), grid, block, 0, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap)
+#define MI_ATT_MMA(A, B) hipLaunchKernelGGL((k_attn_mma_bf16<A, B>), grid, block, 0, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap, pen_kind)
             const int a = dk16 <= 2 ? 2 : (dk16 <= 4 ? 4 : 8), b = dvt <= 1 ? 1 : (dvt <= 2 ? 2 : 4);
             if (a == 2 && b == 1) MI_ATT_MMA(2, 1); else if (a == 2 && b == 2) MI_ATT_MMA(2, 2); else if (a == 2) MI_ATT_MMA(2, 4);
             else if (a == 4 && b == 1) MI_ATT_MMA(4, 1); else if (a == 4 && b == 2) MI_ATT_MMA(4, 2); else if (a == 4) MI_ATT_MMA(4, 4);
@@ -761,7 +763,7 @@ static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, c
             const size_t lds = ((size_t) 64 * (dkp + 1) + (size_t) 64 * dvp + (size_t) 64 * dkp) * sizeof(float);
             // (more than the 64 KB a kernel gets by default: up to 97 KB of the CU's 160 KB; the attribute is per device and cheap to set again)
             if (lds > 48 * 1024) (void) hipFuncSetAttribute((const void *) kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int) lds);
-            hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap);
+            hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap, pen_kind);
         };
         const bool k64 = DK <= 64, v64 = DV <= 64;
         if (k64 && v64) go(k_attn_f32_tile<KT, VT, 64, 64>, 64, 64);
@@ -770,13 +772,13 @@ static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, c
         else go(k_attn_f32_tile<KT, VT, 128, 128>, 128, 128);
         return;
     }
-    hipLaunchKernelGGL((k_attn_f32_rows<KT, VT>), dim3((unsigned) n_q, (unsigned) H), dim3(256), 0, s, q, k, v, mask ? *mask : q, mask ? 1 : 0, sinks, r12, dst, scale, sig, softcap);
+    hipLaunchKernelGGL((k_attn_f32_rows<KT, VT>), dim3((unsigned) n_q, (unsigned) H), dim3(256), 0, s, q, k, v, mask ? *mask : q, mask ? 1 : 0, sinks, r12, dst, scale, sig, softcap, pen_kind);
 }
 
 void launch_attn_f32(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const float * sinks, const float * r12, const tdesc & dst, float scale,
-                     const float * sig, float softcap) {
+                     const float * sig, float softcap, int pen_kind) {
     if (q.ne[1] == 0 || q.ne[2] == 0) return;
-#define MI_ATTN_F32_CASE(KT, VT) if (k.type == KT && v.type == VT) { attn_f32_launch_t<KT, VT>(s, q, k, v, mask, sinks, r12, dst, scale, sig, softcap); return; }
+#define MI_ATTN_F32_CASE(KT, VT) if (k.type == KT && v.type == VT) { attn_f32_launch_t<KT, VT>(s, q, k, v, mask, sinks, r12, dst, scale, sig, softcap, pen_kind); return; }
     MI_ATTN_F32_CASE(GGML_TYPE_F32, GGML_TYPE_F32)
     MI_ATTN_F32_CASE(GGML_TYPE_BF16, GGML_TYPE_BF16)
     MI_ATTN_F32_CASE(GGML_TYPE_F16, GGML_TYPE_F16)

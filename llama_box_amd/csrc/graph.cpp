@@ -69,8 +69,9 @@ static bool fa_f32_route(const ggml_tensor * op) {
     // src[6]: per head a factor on the score and a bias — the weights are sigmoid(score + bias) instead of a soft-max (no sink then)
     if (op->src[6] && (op->src[6]->type != GGML_TYPE_F32 || !ggml_abi_is_contiguous(op->src[6]) || ggml_abi_nelements(op->src[6]) != 2 * a->ne[2] || op->src[4])) return false;
     if (op->src[4] && (op->src[4]->type != GGML_TYPE_F32 || ggml_abi_nelements(op->src[4]) < a->ne[2])) return false;
-    // src[5]: (r1, r2) per head of a logarithmic distance penalty; the F32 mask then holds distances
-    if (op->src[5] && (op->src[5]->type != GGML_TYPE_F32 || !ggml_abi_is_contiguous(op->src[5]) || ggml_abi_nelements(op->src[5]) != 2 * a->ne[2] || !m || m->type != GGML_TYPE_F32)) return false;
+    // src[5]: (r1, r2) per head of a logarithmic distance penalty, or r1 alone of a linear one; the F32 mask then holds distances
+    if (op->src[5] && (op->src[5]->type != GGML_TYPE_F32 || !ggml_abi_is_contiguous(op->src[5]) || !m || m->type != GGML_TYPE_F32 ||
+                       (ggml_abi_nelements(op->src[5]) != 2 * a->ne[2] && ggml_abi_nelements(op->src[5]) != a->ne[2]))) return false;
     const tdesc md = m ? TD(m) : TD(a);
     return attn_f32_applies(TD(a), TD(k), TD(v), m ? &md : nullptr, TD(op));
 }
@@ -173,6 +174,24 @@ static bool seq_op_ok(const ggml_tensor * op) {
     return op->ne[0] == DV && op->ne[1] == H && op->ne[2] == T && ggml_abi_is_contiguous(op);
 }
 
+// what lies between two sublayers of a residual stream kept as N streams (streams.hip), as a CUSTOM op in this backend's own operand layout: op_params[8] == MI_STREAM_OP_TAG
+// (words 0 .. 7 are where ggml's CUSTOM keeps its function pointer, so a host's own CUSTOM never carries the mark), [9] N, [10] 1 when the new streams are wanted, [11] eps, [12] mult.
+//   src (y [E, T_in], x [E, T_in, N] or null, mix [N (to), N (from)], out [N], in [N] or null, norm weight [E], ids [T] i32 or null)
+//   -> one block of memory: the normed rows [E, T], then the new streams [E, T, N]
+static constexpr int32_t MI_STREAM_OP_TAG = 0x57E;
+static bool stream_op_ok(const ggml_tensor * op) {
+    if (op->op_params[8] != MI_STREAM_OP_TAG || op->type != GGML_TYPE_F32) return false;
+    auto f32n = [](const ggml_tensor * t, int64_t n) { return t && t->type == GGML_TYPE_F32 && ggml_abi_is_contiguous(t) && ggml_abi_nelements(t) == n; };
+    const ggml_tensor * y = op->src[0], * x = op->src[1], * ids = op->src[6];
+    const int64_t N = op->op_params[9], keep = op->op_params[10];
+    if (N < 1 || N > STREAM_MAX_N || !y || y->type != GGML_TYPE_F32 || !ggml_abi_is_contiguous(y) || y->ne[2] != 1 || y->ne[3] != 1) return false;
+    const int64_t E = y->ne[0], T_in = y->ne[1], T = ids ? ids->ne[0] : T_in;
+    if (x && (!f32n(x, E * T_in * N) || !f32n(op->src[2], N * N) || !f32n(op->src[3], N))) return false;
+    if (op->src[4] && !f32n(op->src[4], N)) return false;
+    if (!f32n(op->src[5], E) || (ids && (ids->type != GGML_TYPE_I32 || !ggml_abi_is_contiguous(ids) || ggml_abi_nelements(ids) != T))) return false;
+    return ggml_abi_is_contiguous(op) && ggml_abi_nelements(op) == E * T * (keep ? N + 1 : 1);
+}
+
 bool supports_op(const ggml_tensor * op) {
     const ggml_tensor * a = op->src[0];
     const ggml_tensor * b = op->src[1];
@@ -226,8 +245,12 @@ bool supports_op(const ggml_tensor * op) {
             if (a->type != GGML_TYPE_F32 && a->type != GGML_TYPE_F16 && a->type != GGML_TYPE_BF16) return false;
             return a->nb[0] == ggml_abi_type_size(a->type) && b->nb[0] == 4 && a->ne[3] == 1 && b->ne[3] == 1 && (b->ne[1] == 1 || b->ne[1] == ids->ne[0]) && ids->ne[1] == b->ne[2];
         }
+        case GGML_OP_CUSTOM:
+            return stream_op_ok(op);
+        case GGML_OP_SUM_ROWS:
+            return a->type == GGML_TYPE_F32 && a->nb[0] == 4 && op->type == GGML_TYPE_F32 && op->ne[0] == 1 && op->ne[1] == a->ne[1] && op->ne[2] == a->ne[2] && op->ne[3] == a->ne[3];
         case GGML_OP_GLU:
-            return op->op_params[0] == GGML_GLU_OP_SWIGLU && a->type == GGML_TYPE_F32 && a->nb[0] == 4 && (!b || (b->type == GGML_TYPE_F32 && b->nb[0] == 4)) &&
+            return (op->op_params[0] == GGML_GLU_OP_SWIGLU || op->op_params[0] == GGML_GLU_OP_SWIGLU_OAI) && a->type == GGML_TYPE_F32 && a->nb[0] == 4 && (!b || (b->type == GGML_TYPE_F32 && b->nb[0] == 4)) &&
                    a->ne[2] == 1 && a->ne[3] == 1 && op->nb[0] == 4;
         case GGML_OP_CPY: case GGML_OP_DUP: case GGML_OP_CONT: {
             const int st = a->type, dt = op->type;
@@ -1960,6 +1983,93 @@ static int try_fuse_router_scores(exec_state & st, int i) {
     return 1;
 }
 
+// UNARY(SIGMOID, router logits) [-> ADD(., correction row)] -> ARGSORT (descending) -> VIEW (top k) -> GET_ROWS(scores as [1, n, T], view) -> SUM_ROWS -> SCALE(1, bias) -> DIV: a router
+// that chooses by corrected scores and weights by the normalised scores themselves, one launch (views between the nodes skipped).  Returns the nodes consumed (0: no match)
+static int try_fuse_router_sigmoid(exec_state & st, int i) {
+    ggml_cgraph * g = st.g;
+    const ggml_tensor * sg = g->nodes[i];
+    const ggml_tensor * a = sg->src[0];
+    if (a->ne[0] > 256 || a->ne[2] != 1 || a->ne[3] != 1 || !is_f32_contig(a) || !is_f32_contig(sg) || (sg->flags & GGML_TENSOR_FLAG_OUTPUT)) return 0;
+    const ggml_tensor * at[6] = {};
+    int found = 0, k = i + 1;
+    for (; k < g->n_nodes && k < i + 16 && found < 6; ++k) {
+        const ggml_tensor * t = g->nodes[k];
+        if (st.done[k]) return 0;
+        if (is_view_op(t)) continue;
+        if (found == 0 && t->op != GGML_OP_ADD) at[found++] = nullptr;  // (no correction)
+        at[found++] = t;
+    }
+    if (found < 6) return 0;
+    const ggml_tensor * ad = at[0], * as = at[1], * gr = at[2], * sm = at[3], * sc = at[4], * dv = at[5];
+    if (as->op != GGML_OP_ARGSORT || gr->op != GGML_OP_GET_ROWS || sm->op != GGML_OP_SUM_ROWS || sc->op != GGML_OP_SCALE || dv->op != GGML_OP_DIV) return 0;
+    if (ad && (ad->src[0] != sg || !is_row_of(ad->src[1], sg) || !same_shape(ad, sg) || !single_use(st, ad))) return 0;
+    if (as->src[0] != (ad ? ad : sg) || as->op_params[0] != 1 || as->op_params[1] > 1 || !ggml_abi_is_contiguous(as)) return 0;
+    const ggml_tensor * sel = gr->src[1];
+    if (!sel || sel->view_src != as || sel->view_offs != 0 || sel->ne[1] != a->ne[1] || sel->ne[0] > 256 || through_views(gr->src[0]) != sg || gr->src[0]->ne[0] != 1) return 0;
+    const int64_t top = sel->ne[0], T = a->ne[1];
+    if (through_views(sm->src[0]) != gr || sm->src[0]->ne[0] != top || sc->src[0] != sm || ggml_abi_op_param_f32(sc, 0) != 1.0f || !single_use(st, sm) || !single_use(st, sc)) return 0;
+    if (dv->src[1] != sc || through_views(dv->src[0]) != gr || dv->src[0]->ne[0] != top || !is_f32_contig(dv) || ggml_abi_nelements(dv) != top * T) return 0;
+    if (use_count(st, sg) != 2 || use_count(st, gr) != (dv->src[0] == sm->src[0] ? 1 : 2)) return 0;  // (the sort — or the sum it reads — and the pick; through one view, or one each)
+    if (ranges_overlap(as, a) || ranges_overlap(dv, a) || ranges_overlap(as, dv) || (ad && (ranges_overlap(as, ad->src[1]) || ranges_overlap(dv, ad->src[1])))) return 0;
+    timed_scope ts(st.c, "router", (double) ggml_abi_nbytes(a) * 2);
+    launch_router_sigmoid_topk(st.c->stream, TD(a), ad ? (const float *) ad->src[1]->data : nullptr, TD(as), (float *) dv->data, (int) top, ggml_abi_op_param_f32(sc, 1));
+    st.c->st.kernel_launches++;
+    st.c->st.fused_nodes += ad ? 6 : 5;
+    return k - i;
+}
+
+// RMS_NORM(q per head) -> MUL(w) [-> MUL(., one factor per token)], RMS_NORM(k per head) -> MUL(w), SET_ROWS(k), SET_ROWS(v) (views between the nodes skipped): the queries' and keys' norms
+// and both cache stores in one launch.  Returns the nodes consumed (0: no match)
+static int try_fuse_qk_norm_store(exec_state & st, int i) {
+    ggml_cgraph * g = st.g;
+    const ggml_tensor * nq = g->nodes[i];
+    const ggml_tensor * q = nq->src[0];
+    const ggml_tensor * at[6] = {};
+    int found = 0, k = i + 1;
+    for (; k < g->n_nodes && k < i + 20 && found < 6; ++k) {
+        const ggml_tensor * t = g->nodes[k];
+        if (st.done[k]) return 0;
+        if (is_view_op(t)) continue;
+        if (found == 1 && t->op != GGML_OP_MUL) at[found++] = nullptr;  // (no factor per token)
+        at[found++] = t;
+    }
+    if (found < 6) return 0;
+    const ggml_tensor * mq = at[0], * tq = at[1], * nk = at[2], * mk = at[3], * sk = at[4], * sv = at[5];
+    if (mq->op != GGML_OP_MUL || nk->op != GGML_OP_RMS_NORM || mk->op != GGML_OP_MUL || sk->op != GGML_OP_SET_ROWS || sv->op != GGML_OP_SET_ROWS) return 0;
+    const int64_t DK = q->ne[0], H = q->ne[1], T = q->ne[2];
+    const ggml_tensor * kx = nk->src[0];
+    if (q->ne[3] != 1 || !is_f32_contig(q) || !is_f32_contig(kx) || kx->ne[0] != DK || kx->ne[2] != T || kx->ne[3] != 1) return 0;
+    const ggml_tensor * qo = tq ? tq : mq;  // the queries as attention reads them
+    if (mq->src[0] != nq || mk->src[0] != nk || !single_use(st, nq) || !single_use(st, nk) || !is_row_of(mq->src[1], nq) || !is_row_of(mk->src[1], nk) || !is_f32_contig(qo) || !same_shape(qo, nq)) return 0;
+    if (tq && (tq->src[0] != mq || !single_use(st, mq) || !is_f32_contig(tq->src[1]) || tq->src[1]->ne[0] != 1 || tq->src[1]->ne[1] != 1 || tq->src[1]->ne[2] != T || tq->src[1]->ne[3] != 1)) return 0;
+    const ggml_tensor * v = through_views(sv->src[0]);
+    const int64_t G = kx->ne[1];
+    if (through_views(sk->src[0]) != mk || use_count(st, mk) != 1 || (mk->flags & GGML_TENSOR_FLAG_OUTPUT) || !is_f32_contig(v) || !is_f32_contig(sv->src[0]) || v == mk) return 0;
+    const ggml_tensor * idx = sk->src[1];
+    if (idx != sv->src[1] || idx->type != GGML_TYPE_I64 || !ggml_abi_is_contiguous(idx) || ggml_abi_nelements(idx) != T) return 0;
+    auto cache_ok = [](const ggml_tensor * t) {
+        return (t->type == GGML_TYPE_F32 || t->type == GGML_TYPE_BF16 || t->type == GGML_TYPE_F16) && t->nb[0] == ggml_abi_type_size(t->type) && t->ne[2] == 1 && t->ne[3] == 1;
+    };
+    const int64_t row_v = sv->src[0]->ne[0];
+    if (!cache_ok(sk) || !cache_ok(sv) || sk->ne[0] != DK * G || sk->src[0]->ne[0] != DK * G || sk->src[0]->ne[1] != T || sv->src[0]->ne[1] != T || sv->ne[0] != row_v || row_v % G != 0 ||
+        ggml_abi_nelements(v) != row_v * T) return 0;
+    // (every wave reads its own row before it writes: the queries' result may be the projection's own block, nothing else)
+    if (!elementwise_safe(qo, q) || ranges_overlap(qo, kx) || ranges_overlap(qo, v) || ranges_overlap(qo, mq->src[1]) || ranges_overlap(qo, mk->src[1]) || (tq && ranges_overlap(qo, tq->src[1]))) return 0;
+    qk_norm_store_args a{};
+    a.q = (const float *) q->data; a.qd = (float *) qo->data; a.k = (const float *) kx->data; a.v = (const float *) v->data;
+    a.qw = (const float *) mq->src[1]->data; a.kw = (const float *) mk->src[1]->data; a.temp = tq ? (const float *) tq->src[1]->data : nullptr;
+    a.k_cache = (char *) sk->data; a.v_cache = (char *) sv->data;
+    a.kc_nb1 = (int64_t) sk->nb[1]; a.vc_nb1 = (int64_t) sv->nb[1];
+    a.idx = (const int64_t *) idx->data;
+    a.eps_q = ggml_abi_op_param_f32(nq, 0); a.eps_k = ggml_abi_op_param_f32(nk, 0);
+    a.H = (int) H; a.G = (int) G; a.DK = (int) DK; a.DV = (int) (row_v / G); a.k_type = sk->type; a.v_type = sv->type;
+    timed_scope ts(st.c, "qk_norm_store", (double) (ggml_abi_nbytes(q) * 2 + ggml_abi_nbytes(kx) + ggml_abi_nbytes(v)));
+    launch_qk_norm_store(st.c->stream, a, T);
+    st.c->st.kernel_launches++;
+    st.c->st.fused_nodes += tq ? 6 : 5;
+    return k - i;
+}
+
 // ADD(x, y) -> RMS_NORM(.) -> MUL(., w row): a residual update and the norm of the sublayer that follows in one launch (pre-norm models whose norms are RMS norms).
 // The sum stays a tensor of its own: the stream goes on from it.  Returns the nodes consumed at position i (0: no match)
 static int try_fuse_add_rms_norm(exec_state & st, int i) {
@@ -2216,6 +2326,7 @@ static int run_node(exec_state & st, int i) {
         case GGML_OP_RMS_NORM: {
             if (fuse) { const int r = try_fuse_head_norm_gate(st, i); if (r) return r; }
             if (fuse) { const int r = try_fuse_norm2_blend(st, i); if (r) return r; }
+            if (fuse) { const int r = try_fuse_qk_norm_store(st, i); if (r) return r; }
             // RMS_NORM -> MUL(norm, w): one kernel writing the MUL's output
             ggml_tensor * m = next(1);
             if (fuse && m && m->op == GGML_OP_MUL && single_use(st, n) && m->type == GGML_TYPE_F32 && m->nb[0] == 4) {
@@ -2475,6 +2586,7 @@ static int run_node(exec_state & st, int i) {
             return 1;
         }
         case GGML_OP_UNARY: {
+            if (fuse && n->op_params[0] == GGML_UNARY_OP_SIGMOID) { const int r = try_fuse_router_sigmoid(st, i); if (r) return r; }
             // SIGMOID(g) -> RESHAPE -> MUL(x, .) with ONE gate per row of x (a number per head): one pass
             if (fuse && n->op_params[0] == GGML_UNARY_OP_SIGMOID && next(1) && next(2) && !st.done[i + 1] && !st.done[i + 2]) {
                 const ggml_tensor * rs = next(1), * gm2 = next(2);
@@ -2573,6 +2685,33 @@ static int run_node(exec_state & st, int i) {
             c->st.kernel_launches++;
             return 1;
         }
+        case GGML_OP_SUM_ROWS:
+            launch_sum_rows(s, TD(a), TD(n));
+            c->st.kernel_launches++;
+            return 1;
+        case GGML_OP_CUSTOM: {
+            if (!stream_op_ok(n)) { MI_ERR("graph_compute: node %d '%s': a CUSTOM op that is not this backend's", i, n->name); return -1; }
+            const int64_t N = n->op_params[9], E = a->ne[0], T_in = a->ne[1], T = n->src[6] ? n->src[6]->ne[0] : T_in;
+            stream_step_args sa{};
+            sa.y = (const float *) a->data;
+            sa.x = b ? (const float *) b->data : nullptr;
+            sa.mix = b ? (const float *) n->src[2]->data : nullptr;
+            sa.out = b ? (const float *) n->src[3]->data : nullptr;
+            sa.in = n->src[4] ? (const float *) n->src[4]->data : nullptr;
+            sa.w = (const float *) n->src[5]->data;
+            sa.ids = n->src[6] ? (const int32_t *) n->src[6]->data : nullptr;
+            sa.h = (float *) n->data;
+            sa.x_out = n->op_params[10] ? (float *) n->data + E * T : nullptr;
+            sa.E = E;
+            sa.x_plane = E * T_in;
+            sa.xo_plane = E * T;
+            sa.eps = ggml_abi_op_param_f32(n, 11);
+            sa.mult = ggml_abi_op_param_f32(n, 12);
+            timed_scope ts(c, "stream_step", (double) (E * T) * 4.0 * (double) (2 + (b ? N : 0) + (n->op_params[10] ? N : 0)));
+            launch_stream_step(s, sa, (int) N, T);
+            c->st.kernel_launches++;
+            return 1;
+        }
         case GGML_OP_SSM_CONV: {
             const int taps = n->op_params[0];
             if (n->op_params[2] == 1) {
@@ -2660,7 +2799,7 @@ static int run_node(exec_state & st, int i) {
             // the down projection of a mixture-of-experts block reads the same ids as its up projection: the per-expert column lists are made once
             // (valid only while nothing but element-wise nodes ran in between: they do not touch the scratch area)
             bool valid = st.moe_ids == ids && st.moe_node >= 0 && i - st.moe_node <= 6 && g->nodes[st.moe_node]->src[0]->ne[2] == a->ne[2];
-            for (int k = st.moe_node + 1; valid && k < i; ++k) valid = is_view_op(g->nodes[k]) || g->nodes[k]->op == GGML_OP_UNARY || g->nodes[k]->op == GGML_OP_SQR;
+            for (int k = st.moe_node + 1; valid && k < i; ++k) valid = is_view_op(g->nodes[k]) || g->nodes[k]->op == GGML_OP_UNARY || g->nodes[k]->op == GGML_OP_SQR || (g->nodes[k]->op == GGML_OP_GLU && !is_quant(a->type));
             const size_t need = mul_mat_id_workspace_bytes(TD(a), TD(ids));
             void * ws = (c->ws && st.aux_off + need <= c->ws_size) ? (char *) c->ws + st.aux_off : nullptr;
             timed_scope ts(c, "mul_mat_id", (double) ggml_abi_nbytes(a) / (double) std::max<int64_t>(1, a->ne[2]) * (double) std::min<int64_t>(a->ne[2], ggml_abi_nelements(ids)));
@@ -2672,6 +2811,12 @@ static int run_node(exec_state & st, int i) {
         }
         case GGML_OP_GLU: {
             const tdesc bd = b ? TD(b) : TD(a);
+            if (n->op_params[0] == GGML_GLU_OP_SWIGLU_OAI) {  // gate and up limited, gate's sigmoid at its own slope, up + 1
+                timed_scope ts(c, "swiglu_limited", (double) ggml_abi_nbytes(n) * 3);
+                launch_swiglu_limited(s, TD(a), b ? &bd : nullptr, TD(n), n->op_params[1], ggml_abi_op_param_f32(n, 2), ggml_abi_op_param_f32(n, 3));
+                c->st.kernel_launches++;
+                return 1;
+            }
             if (fuse && c->opt.prologue && ggml_abi_nrows(n) > 1 && (a->nb[1] % 16) == 0 && (!b || (b->nb[1] % 16) == 0) && !(((uintptr_t) a->data) & 15) &&
                 (!b || !(((uintptr_t) b->data) & 15)) && (b || ((n->ne[0] * 4) % 16) == 0) && quant_consumers_only(st, i, n)) {
                 timed_scope ts(c, "swiglu_quantize", (double) ggml_abi_nbytes(n) * 2);
@@ -2930,7 +3075,7 @@ static int run_node(exec_state & st, int i) {
                 const tdesc md4 = m ? TD(m) : qd;
                 timed_scope ts(c, "attn_f32", (double) ggml_abi_nbytes(k) + (double) ggml_abi_nbytes(v));
                 launch_attn_f32(s, qd, kd, vd, m ? &md4 : nullptr, n->src[4] ? (const float *) n->src[4]->data : nullptr, n->src[5] ? (const float *) n->src[5]->data : nullptr, TD(n), p.scale,
-                                n->src[6] ? (const float *) n->src[6]->data : nullptr, p.logit_softcap);
+                                n->src[6] ? (const float *) n->src[6]->data : nullptr, p.logit_softcap, n->src[5] && ggml_abi_nelements(n->src[5]) == a->ne[2] ? ATTN_PEN_LINEAR : ATTN_PEN_LOG);
                 c->st.kernel_launches++;
                 c->st.attn_f32_nodes++;
                 return 1;

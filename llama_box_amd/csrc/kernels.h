@@ -171,10 +171,11 @@ bool launch_mul_mat_id(hipStream_t s, const tdesc & as, const tdesc & b, const t
 // FLASH_ATTN_EXT in 32-bit arithmetic over f32 / bf16 / f16 K and V read in place, any head sizes up to 256, K and V sizes independent (attn_f32.hip)
 bool attn_f32_applies(const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const tdesc & dst);
 // r12 (optional: r1 of every head, then r2 of every head): the mask then holds the DISTANCE between query and cell for visible pairs (-inf for hidden ones) and the score is
-// q.k * scale - r1 ln(1 + r2 distance)
+// q.k * scale - r1 ln(1 + r2 distance); with pen_kind ATTN_PEN_LINEAR r12 holds r1 alone and the score is q.k * scale - r1 distance
+enum { ATTN_PEN_LOG = 1, ATTN_PEN_LINEAR = 2 };
 // sig: per head a factor on the score, then per head a bias ([heads, 2]) — the weights are then sigmoid(score + bias), not a soft-max; softcap > 0: score <- cap tanh(score / cap)
 void launch_attn_f32(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const float * sinks, const float * r12, const tdesc & dst, float scale,
-                     const float * sig = nullptr, float softcap = 0.0f);
+                     const float * sig = nullptr, float softcap = 0.0f, int pen_kind = ATTN_PEN_LOG);
 // ---- non-flash attention chain of a small batch over position lists (attn_nf.hip)
 size_t attn_nf_list_scratch_bytes(const tdesc & q, const tdesc & k, int * dq_out);
 bool launch_attn_nf_list(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc & mask, const tdesc & dst, const int * lists, int list_stride,
@@ -411,6 +412,40 @@ size_t seq_recurrence_scratch_bytes(int kind, int H, int DK, int64_t T);
 void launch_seq_recurrence(hipStream_t s, int kind, const seq_rec_args & a, int n_seqs, void * scratch = nullptr, size_t scratch_bytes = 0);
 // SOFT_MAX over a router's logits, the (group-limited) descending ARGSORT of the scores, GET_ROWS of the k first and SCALE in one launch (n <= 256 experts)
 void launch_router_softmax_topk(hipStream_t s, const tdesc & logits, const tdesc & probs, const tdesc & ids, const tdesc & wts /* [1, k, T] */, int k, int groups, int keep, float wscale);
+// UNARY(SIGMOID) over a router's logits, ADD of a correction, the descending ARGSORT of the sums, GET_ROWS of the k first SCORES, their SUM_ROWS, SCALE(1, bias) and DIV in one launch
+// (n <= 256 experts): ids gets the whole permutation, wts [1, k, T] the normalised scores
+void launch_router_sigmoid_topk(hipStream_t s, const tdesc & logits, const float * corr, const tdesc & ids, float * wts, int k, float sum_bias);
+// queries and keys behind their projections: RMS_NORM per head -> MUL(weight row) [-> MUL(one factor per token)] of q in place or to qd, RMS_NORM -> MUL of k and v as it is straight into
+// their cache rows (f32 / bf16 / f16) at idx[token]
+struct qk_norm_store_args {
+    const float * q; float * qd; const float * k; const float * v;  // q, qd [DK, H, T]; k [DK, G, T]; v [DV G, T], contiguous
+    const float * qw; const float * kw; const float * temp;          // temp: [T] or null
+    char * k_cache; char * v_cache;
+    int64_t kc_nb1, vc_nb1;
+    const int64_t * idx;
+    float eps_q, eps_k;
+    int H, G, DK, DV, k_type, v_type;
+};
+void launch_qk_norm_store(hipStream_t s, const qk_norm_store_args & a, int64_t n_tok);
+void launch_sum_rows(hipStream_t s, const tdesc & src, const tdesc & dst);
+void launch_swiglu_limited(hipStream_t s, const tdesc & a, const tdesc * b, const tdesc & dst, int swapped, float alpha, float limit);  // min(g, l) sigmoid(alpha min(g, l)) (clamp(u, -l, l) + 1)
+
+// ---- a residual stream kept as several streams (streams.hip)
+constexpr int STREAM_MAX_N = 8;
+struct stream_step_args {
+    const float * y;              // [E, T_in]: what joins the streams (or starts them)
+    const float * x;              // old streams, planes [E, T_in] x_plane floats apart; null: every stream starts as y
+    const float * mix;            // [N (from), N (to)]: mix[n * N + t]
+    const float * out;            // [N]: the sublayer's share per stream, times mult
+    const float * in;             // [N]: weights of the row that is normed; null: the plain sum
+    const float * w;              // [E]: the norm's weight
+    const int32_t * ids;          // row of (y, x) per output row, or null
+    float * h;                    // [E, T]: the normed rows
+    float * x_out;                // new streams, planes xo_plane floats apart; null: not wanted
+    int64_t E, x_plane, xo_plane;
+    float mult, eps;
+};
+void launch_stream_step(hipStream_t s, const stream_step_args & a, int n_streams, int64_t rows);
 // RMS_NORM per head -> MUL(weight: [DV] or [DV, H]) -> MUL(act(gate)), act SiLU (0) or sigmoid (1): o [DV, H, T] (rows contiguous), gate and d [DV H, T] contiguous
 void launch_head_norm_gate(hipStream_t s, const tdesc & o, const float * w, int w_per_head, const float * gate, int sigmoid_act, float * d, float eps);
 // ADD(x, y) -> RMS_NORM -> MUL(w): sum (may lie over x or y) and the normed rows d, all [n, rows] contiguous f32
@@ -440,6 +475,7 @@ void tu_touch_tp_p2p(hipStream_t s);
 void tu_touch_kv_types(hipStream_t s);
 void tu_touch_repack(hipStream_t s);
 void tu_touch_seq(hipStream_t s);
+void tu_touch_streams(hipStream_t s);
 inline void preload_kernel_files(hipStream_t s) {
     tu_touch_kv_types(s);
     tu_touch_repack(s);
@@ -458,6 +494,7 @@ inline void preload_kernel_files(hipStream_t s) {
     tu_touch_fattn_mma(s);
     tu_touch_tp_p2p(s);
     tu_touch_seq(s);
+    tu_touch_streams(s);
 }
 
 }  // namespace mi355x

@@ -336,6 +336,115 @@ void launch_router_softmax_topk(hipStream_t s, const tdesc & logits, const tdesc
     hipLaunchKernelGGL(k_router_softmax_topk, dim3((unsigned) logits.ne[1]), dim3(256), 0, s, logits, probs, ids, wts, k, groups, keep, wscale);
 }
 
+// ------------------------------------------------------------------------------------------------ router: sigmoid scores, corrected choice, normalised weights
+// one workgroup per token, a thread per expert (n <= 256): UNARY(SIGMOID), ADD(correction), the descending ARGSORT of the sums (ranks by counting: the stable order of
+// k_argsort), GET_ROWS of the k first scores, SUM_ROWS (f64, as k_sum_rows), SCALE(1, bias) and DIV — the nodes' own results
+__global__ void __launch_bounds__(256) k_router_sigmoid_topk(const tdesc a, const float * __restrict__ corr, const tdesc ids, float * __restrict__ wts, const int k, const float sum_bias) {
+    __shared__ float c[256], top[256];
+    __shared__ float sum_sh;
+    const int64_t t = blockIdx.x;
+    const int n = (int) a.ne[0], i = threadIdx.x;
+    float sc = 0.0f, v = 0.0f;
+    if (i < n) {
+        sc = 1.f / (1.f + expf(-((const float *) (a.data + t * a.nb[1]))[i]));
+        v = corr ? sc + corr[i] : sc;
+        c[i] = v;
+    }
+    __syncthreads();
+    if (i < n) {
+        int before = 0;
+        for (int j = 0; j < n; ++j) {
+            const float u = c[j];
+            before += (u > v || (u == v && j < i)) ? 1 : 0;
+        }
+        ((int32_t *) (ids.data + t * ids.nb[1]))[before] = i;
+        if (before < k) top[before] = sc;
+    }
+    __syncthreads();
+    if (i < 64) {
+        double s = 0.0;
+        for (int j = i; j < k; j += 64) s += (double) top[j];
+        s = wave_sum_d(s);
+        if (i == 0) { const float p = (float) s * 1.0f; sum_sh = p + sum_bias; }
+    }
+    __syncthreads();
+    if (i < k) wts[t * k + i] = top[i] / sum_sh;
+}
+void launch_router_sigmoid_topk(hipStream_t s, const tdesc & logits, const float * corr, const tdesc & ids, float * wts, int k, float sum_bias) {
+    if (logits.ne[1] == 0) return;
+    hipLaunchKernelGGL(k_router_sigmoid_topk, dim3((unsigned) logits.ne[1]), dim3(256), 0, s, logits, corr, ids, wts, k, sum_bias);
+}
+
+// ------------------------------------------------------------------------------------------------ SUM_ROWS
+// a wave per row, the sum in f64
+__global__ void __launch_bounds__(256) k_sum_rows(const tdesc a, const tdesc d) {
+    const int64_t row = (int64_t) blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (row >= a.ne[1] * a.ne[2] * a.ne[3]) return;
+    const int64_t i1 = row % a.ne[1], i2 = (row / a.ne[1]) % a.ne[2], i3 = row / (a.ne[1] * a.ne[2]);
+    const float * x = (const float *) (a.data + i1 * a.nb[1] + i2 * a.nb[2] + i3 * a.nb[3]);
+    double s = 0.0;
+    for (int64_t i = threadIdx.x & 63; i < a.ne[0]; i += 64) s += (double) x[i];
+    s = wave_sum_d(s);
+    if ((threadIdx.x & 63) == 0) *(float *) (d.data + i1 * d.nb[1] + i2 * d.nb[2] + i3 * d.nb[3]) = (float) s;
+}
+void launch_sum_rows(hipStream_t s, const tdesc & src, const tdesc & dst) {
+    const int64_t rows = src.ne[1] * src.ne[2] * src.ne[3];
+    if (rows == 0) return;
+    hipLaunchKernelGGL(k_sum_rows, dim3((unsigned) ((rows + 3) / 4)), dim3(256), 0, s, src, dst);
+}
+
+// ------------------------------------------------------------------------------------------------ per-head norms of queries and keys, straight into the cache rows
+// a wave per head row of one token: the query heads (norm, weight, optionally the token's factor), the key heads (norm, weight, stored), the value heads (stored).  The sum of
+// squares is f64 as in k_rms_norm, so the scale is the same f32 number; conversions are those of the row stores.  A wave has read its whole row before it writes any of it
+// (the query's result may lie over the projection).
+__device__ __forceinline__ void cache_put(char * row, const int type, const int64_t i, const float v) {
+    if (type == GGML_TYPE_F32) ((float *) row)[i] = v;
+    else if (type == GGML_TYPE_BF16) ((uint16_t *) row)[i] = f2bf(v);
+    else ((uint16_t *) row)[i] = f2h(v);
+}
+__global__ void __launch_bounds__(256) k_qk_norm_store(const qk_norm_store_args A, const int64_t rows) {
+    const int lane = threadIdx.x & 63, per = A.H + 2 * A.G;
+    const int64_t row = (int64_t) blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (row >= rows) return;
+    const int64_t t = row / per;
+    const int j = (int) (row % per), DK = A.DK;
+    if (j >= A.H + A.G) {
+        const int g = j - A.H - A.G, DV = A.DV;
+        const float * x = A.v + (t * A.G + g) * DV;
+        char * vrow = A.v_cache + A.idx[t] * A.vc_nb1;
+        for (int i = lane; i < DV; i += 64) cache_put(vrow, A.v_type, (int64_t) g * DV + i, x[i]);
+        return;
+    }
+    const bool is_q = j < A.H;
+    const float * x = is_q ? A.q + (t * A.H + j) * DK : A.k + (t * A.G + (j - A.H)) * DK;
+    double s = 0.0;
+    for (int i = lane; i < DK; i += 64) s += (double) (x[i] * x[i]);
+    for (int off = 32; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
+    const float mean = (float) (s / (double) DK);
+    const float scale = 1.0f / sqrtf(mean + (is_q ? A.eps_q : A.eps_k));
+    if (is_q) {
+        float * y = A.qd + (t * A.H + j) * DK;
+        const float f = A.temp ? A.temp[t] : 1.0f;
+        for (int i = lane; i < DK; i += 64) {
+            float v = x[i] * scale;
+            v = v * A.qw[i];
+            y[i] = A.temp ? v * f : v;
+        }
+    } else {
+        char * krow = A.k_cache + A.idx[t] * A.kc_nb1;
+        for (int i = lane; i < DK; i += 64) {
+            float v = x[i] * scale;
+            v = v * A.kw[i];
+            cache_put(krow, A.k_type, (int64_t) (j - A.H) * DK + i, v);
+        }
+    }
+}
+void launch_qk_norm_store(hipStream_t s, const qk_norm_store_args & a, int64_t n_tok) {
+    const int64_t rows = n_tok * (a.H + 2 * a.G);
+    if (rows == 0) return;
+    hipLaunchKernelGGL(k_qk_norm_store, dim3((unsigned) ((rows + 3) / 4)), dim3(256), 0, s, a, rows);
+}
+
 // ------------------------------------------------------------------------------------------------ residual sum and the RMS norm of the next sublayer
 // ADD(x, y) -> RMS_NORM -> MUL(., w): the stream's update and the norm that reads it in one launch; both results are written (the sum goes on as the residual).  The sum of
 // squares is f64 as in k_rms_norm.  A thread re-reads only entries of the sum it wrote itself, so the sum may lie over x or y.
@@ -708,6 +817,47 @@ void launch_swiglu(hipStream_t s, const tdesc & a, const tdesc * b, const tdesc 
     const dim3 grid((unsigned) rows, (unsigned) ((nc + 1023) / 1024));
     if (vec) hipLaunchKernelGGL(k_swiglu<true>, grid, dim3(256), 0, s, pa, pb, d.data, nc, a.nb[1], nbb1, d.nb[1]);
     else hipLaunchKernelGGL(k_swiglu<false>, grid, dim3(256), 0, s, pa, pb, d.data, nc, a.nb[1], nbb1, d.nb[1]);
+}
+
+// a gated activation with limits (ggml_swiglu_oai): g = min(a, limit), u = clamp(b, -limit, limit); y = g / (1 + exp(-alpha g)) * (u + 1)
+__device__ __forceinline__ float swiglu_limited_f(const float a, const float b, const float alpha, const float limit) {
+    const float g = fminf(a, limit), u = fminf(fmaxf(b, -limit), limit);
+    const float act = g / (1.0f + expf(alpha * -g));
+    return act * (u + 1.0f);
+}
+template <bool VEC>
+__global__ void __launch_bounds__(256) k_swiglu_limited(const char * __restrict__ pa, const char * __restrict__ pb, char * __restrict__ pd, const int64_t nc, const int64_t nba1, const int64_t nbb1,
+                                                        const int64_t nbd1, const float alpha, const float limit) {
+    const int64_t row = blockIdx.x;
+    const float * a = (const float *) (pa + row * nba1);
+    const float * b = (const float *) (pb + row * nbb1);
+    float * y = (float *) (pd + row * nbd1);
+    const int64_t i0 = ((int64_t) blockIdx.y * 256 + threadIdx.x) * 4;
+    if constexpr (VEC) {
+        if (i0 < nc) {  // (nc % 4 == 0)
+            const float4 av = *(const float4 *) (a + i0), bv = *(const float4 *) (b + i0);
+            *(float4 *) (y + i0) = make_float4(swiglu_limited_f(av.x, bv.x, alpha, limit), swiglu_limited_f(av.y, bv.y, alpha, limit), swiglu_limited_f(av.z, bv.z, alpha, limit),
+                                               swiglu_limited_f(av.w, bv.w, alpha, limit));
+        }
+    } else {
+        for (int64_t i = i0; i < i0 + 4 && i < nc; ++i) y[i] = swiglu_limited_f(a[i], b[i], alpha, limit);
+    }
+}
+void launch_swiglu_limited(hipStream_t s, const tdesc & a, const tdesc * b, const tdesc & d, int swapped, float alpha, float limit) {
+    const int64_t rows = a.ne[1] * a.ne[2] * a.ne[3];
+    const int64_t nc = d.ne[0];
+    if (rows == 0 || nc == 0) return;
+    const char * pa = a.data;
+    const char * pb = b ? b->data : a.data;
+    if (!b) {
+        pa += swapped ? nc * 4 : 0;
+        pb += swapped ? 0 : nc * 4;
+    }
+    const int64_t nbb1 = b ? b->nb[1] : a.nb[1];
+    const bool vec = (nc % 4) == 0 && (((uintptr_t) pa | (uintptr_t) pb | (uintptr_t) d.data | (uintptr_t) a.nb[1] | (uintptr_t) nbb1 | (uintptr_t) d.nb[1]) & 15) == 0;
+    const dim3 grid((unsigned) rows, (unsigned) ((nc + 1023) / 1024));
+    if (vec) hipLaunchKernelGGL(k_swiglu_limited<true>, grid, dim3(256), 0, s, pa, pb, d.data, nc, a.nb[1], nbb1, d.nb[1], alpha, limit);
+    else hipLaunchKernelGGL(k_swiglu_limited<false>, grid, dim3(256), 0, s, pa, pb, d.data, nc, a.nb[1], nbb1, d.nb[1], alpha, limit);
 }
 
 // ------------------------------------------------------------------------------------------------ CPY / DUP / CONT

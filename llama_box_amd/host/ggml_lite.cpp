@@ -465,6 +465,19 @@ static ggml_tensor * glu_impl(ggml_context * ctx, ggml_tensor * a, ggml_tensor *
 struct ggml_tensor * ggml_swiglu(struct ggml_context * ctx, struct ggml_tensor * a) { return glu_impl(ctx, a, nullptr, GGML_GLU_OP_SWIGLU, false); }
 struct ggml_tensor * ggml_swiglu_split(struct ggml_context * ctx, struct ggml_tensor * a, struct ggml_tensor * b) { return glu_impl(ctx, a, b, GGML_GLU_OP_SWIGLU, false); }
 
+struct ggml_tensor * ggml_swiglu_oai(struct ggml_context * ctx, struct ggml_tensor * a, struct ggml_tensor * b, float alpha, float limit) {
+    ggml_tensor * r = glu_impl(ctx, a, b, GGML_GLU_OP_SWIGLU_OAI, false);
+    set_f32(r, 2, alpha);
+    set_f32(r, 3, limit);
+    return r;
+}
+struct ggml_tensor * ggml_sum_rows(struct ggml_context * ctx, struct ggml_tensor * a) {
+    ggml_tensor * r = ggml_new_tensor_4d(ctx, a->type, 1, a->ne[1], a->ne[2], a->ne[3]);
+    r->op = GGML_OP_SUM_ROWS;
+    r->src[0] = a;
+    return r;
+}
+
 struct ggml_tensor * ggml_soft_max_ext(struct ggml_context * ctx, struct ggml_tensor * a, struct ggml_tensor * mask, float scale, float max_bias) {
     LITE_ASSERT(ggml_is_contiguous(a));
     if (mask) {
@@ -581,6 +594,11 @@ void ggml_flash_attn_ext_add_log_distance(struct ggml_tensor * a, struct ggml_te
     LITE_ASSERT(r12->type == GGML_TYPE_F32 && r12->ne[0] == a->src[0]->ne[2] && r12->ne[1] == 2 && ggml_is_contiguous(r12));
     a->src[5] = r12;
 }
+void ggml_flash_attn_ext_add_linear_distance(struct ggml_tensor * a, struct ggml_tensor * slopes) {
+    LITE_ASSERT(a->op == GGML_OP_FLASH_ATTN_EXT && a->src[3] != nullptr && a->src[3]->type == GGML_TYPE_F32);
+    LITE_ASSERT(slopes->type == GGML_TYPE_F32 && ggml_nelements(slopes) == a->src[0]->ne[2] && ggml_is_contiguous(slopes));
+    a->src[5] = slopes;
+}
 void ggml_flash_attn_ext_set_sigmoid(struct ggml_tensor * a, struct ggml_tensor * fb) {
     LITE_ASSERT(a->op == GGML_OP_FLASH_ATTN_EXT && a->src[3] != nullptr && a->src[3]->type == GGML_TYPE_F32 && a->src[4] == nullptr);
     LITE_ASSERT(fb->type == GGML_TYPE_F32 && fb->ne[0] == a->src[0]->ne[2] && fb->ne[1] == 2 && ggml_is_contiguous(fb));
@@ -592,6 +610,31 @@ struct ggml_tensor * ggml_argsort_grouped(struct ggml_context * ctx, struct ggml
     r->op_params[1] = groups;
     r->op_params[2] = keep;
     return r;
+}
+
+// ---- several residual streams: a CUSTOM op marked in op_params[8] (the words before it are where ggml keeps a CUSTOM's function pointer)
+static const int32_t STREAM_OP_TAG = 0x57E;
+struct ggml_tensor * ggml_stream_step(struct ggml_context * ctx, struct ggml_tensor * y, struct ggml_tensor * x, struct ggml_tensor * mix, struct ggml_tensor * out, struct ggml_tensor * in,
+                                      struct ggml_tensor * w, struct ggml_tensor * ids, int n_streams, int keep, float mult, float eps) {
+    const int64_t E = y->ne[0], T_in = y->ne[1], T = ids ? ids->ne[0] : T_in, N = n_streams;
+    LITE_ASSERT(N >= 1 && y->type == GGML_TYPE_F32 && ggml_is_contiguous(y) && y->ne[2] == 1 && y->ne[3] == 1 && ggml_nelements(w) == E);
+    LITE_ASSERT(!x || (ggml_is_contiguous(x) && x->ne[0] == E && x->ne[1] == T_in && x->ne[2] == N && mix && out && mix->ne[0] == N && mix->ne[1] == N && ggml_nelements(out) == N));
+    LITE_ASSERT(!in || ggml_nelements(in) == N);
+    ggml_tensor * r = ggml_new_tensor_3d(ctx, GGML_TYPE_F32, E, T, keep ? N + 1 : 1);  // plane 0: the normed rows; then the streams
+    r->op = GGML_OP_CUSTOM;
+    r->op_params[8] = STREAM_OP_TAG;
+    r->op_params[9] = n_streams;
+    r->op_params[10] = keep ? 1 : 0;
+    set_f32(r, 11, eps);
+    set_f32(r, 12, mult);
+    ggml_tensor * srcs[7] = {y, x, x ? mix : nullptr, x ? out : nullptr, in, w, ids};
+    for (int i = 0; i < 7; ++i) r->src[i] = srcs[i];
+    return r;
+}
+struct ggml_tensor * ggml_stream_step_rows(struct ggml_context * ctx, struct ggml_tensor * step) { return ggml_view_2d(ctx, step, step->ne[0], step->ne[1], step->nb[1], 0); }
+struct ggml_tensor * ggml_stream_step_streams(struct ggml_context * ctx, struct ggml_tensor * step) {
+    LITE_ASSERT(step->op == GGML_OP_CUSTOM && step->op_params[10]);
+    return ggml_view_3d(ctx, step, step->ne[0], step->ne[1], step->ne[2] - 1, step->nb[1], step->nb[2], step->nb[2]);
 }
 
 // ---- ops over sequence state: this harness's own operand layouts, marked by op_params[3] (the backend refuses the op numbers without the mark)

@@ -92,6 +92,9 @@ struct ggml_tensor * ggml_silu(struct ggml_context * ctx, struct ggml_tensor * a
 struct ggml_tensor * ggml_unary(struct ggml_context * ctx, struct ggml_tensor * a, enum ggml_unary_op op);
 struct ggml_tensor * ggml_swiglu(struct ggml_context * ctx, struct ggml_tensor * a);
 struct ggml_tensor * ggml_swiglu_split(struct ggml_context * ctx, struct ggml_tensor * a, struct ggml_tensor * b);
+/* g = min(a, limit), u = clamp(b, -limit, limit): g sigmoid(alpha g) (u + 1); b NULL: the two halves of a's rows */
+struct ggml_tensor * ggml_swiglu_oai(struct ggml_context * ctx, struct ggml_tensor * a, struct ggml_tensor * b, float alpha, float limit);
+struct ggml_tensor * ggml_sum_rows(struct ggml_context * ctx, struct ggml_tensor * a);
 struct ggml_tensor * ggml_soft_max(struct ggml_context * ctx, struct ggml_tensor * a);
 struct ggml_tensor * ggml_soft_max_ext(struct ggml_context * ctx, struct ggml_tensor * a, struct ggml_tensor * mask, float scale, float max_bias);
 void ggml_soft_max_add_sinks(struct ggml_tensor * a, struct ggml_tensor * sinks);
@@ -112,12 +115,25 @@ void ggml_flash_attn_ext_set_prec(struct ggml_tensor * a, enum ggml_prec prec);
 void ggml_flash_attn_ext_add_sinks(struct ggml_tensor * a, struct ggml_tensor * sinks);
 /* score -= r1[h] ln(1 + r2[h] distance): r12 is f32 [heads, 2] (all r1, then all r2); the F32 mask holds distances (>= 0) of visible pairs, -inf for hidden ones */
 void ggml_flash_attn_ext_add_log_distance(struct ggml_tensor * a, struct ggml_tensor * r12);
+/* score -= slope[h] distance: slopes is f32 [heads]; the mask as for the logarithmic form */
+void ggml_flash_attn_ext_add_linear_distance(struct ggml_tensor * a, struct ggml_tensor * slopes);
 /* weights that are no soft-max: every visible key gets sigmoid(score + bias[h]), nothing is normalised over the keys; the score is q.k * scale * factor[h], soft-capped when
    the op's logit_softcap > 0.  `fb` is f32 [heads, 2] (all factors, then all biases): src[6].  Served by the 32-bit attention route (F32 mask). */
 void ggml_flash_attn_ext_set_sigmoid(struct ggml_tensor * a, struct ggml_tensor * fb);
 /* descending argsort of a router's scores whose entries form `groups` equal groups of neighbours: entries outside the `keep` groups with the largest maxima sort last */
 struct ggml_tensor * ggml_argsort_grouped(struct ggml_context * ctx, struct ggml_tensor * a, int groups, int keep);
 struct ggml_tensor * ggml_argmax(struct ggml_context * ctx, struct ggml_tensor * a);
+
+/* ---- a residual stream kept as N parallel streams (hyper-connections).  What lies between two sublayers, as one op: every stream becomes a mixture of all old ones plus its share of
+   the sublayer's output y, and the streams weighted by `in` are RMS-normed for the next sublayer:
+     x_t <- sum_n mix[n, t] x_n + mult out[t] y;   h = rms_norm(sum_t in[t] x_t, eps) w
+   y [E, T]; x [E, T, N] contiguous planes, or NULL: every stream starts as y (mix, out unused); mix [N (to), N (from)]; out, in [N] (in NULL: the plain sum); w [E]; ids i32 [T'] or
+   NULL: only these rows go on.  keep 0: the new streams are not wanted.  The result is one block of memory: ggml_stream_step_rows gives the view of h [E, T'],
+   ggml_stream_step_streams the view of the new streams [E, T', N]. */
+struct ggml_tensor * ggml_stream_step(struct ggml_context * ctx, struct ggml_tensor * y, struct ggml_tensor * x, struct ggml_tensor * mix, struct ggml_tensor * out, struct ggml_tensor * in,
+                                      struct ggml_tensor * w, struct ggml_tensor * ids, int n_streams, int keep, float mult, float eps);
+struct ggml_tensor * ggml_stream_step_rows(struct ggml_context * ctx, struct ggml_tensor * step);
+struct ggml_tensor * ggml_stream_step_streams(struct ggml_context * ctx, struct ggml_tensor * step);
 
 /* ---- layers that carry state from token to token of a sequence, over batches that mix sequences freely.  The batch is described by four i32 inputs the
    scheduler fills: hist [hs, T] (where the d-th token before token t of the same sequence is found: a batch row, -1 = before the sequence's start, or

@@ -350,6 +350,10 @@ struct llm_layer {
     ggml_tensor *wbeta = nullptr, *wa1 = nullptr, *wa2 = nullptr, *wg1 = nullptr, *wg2 = nullptr, *wo_r = nullptr, *left_norm = nullptr, *right_norm = nullptr;
     // ... a state-space mixer: the input projection in three parts (gate z, convolved (x, B, C), step sizes), the convolution's bias
     ggml_tensor *ssm_in_z = nullptr, *ssm_in_xbc = nullptr, *ssm_in_dt = nullptr, *conv_b = nullptr;
+    // ... a residual stream kept as several streams: per sublayer (mixer, feed-forward) the weights of its input, its output's share and the mixture [to, from]
+    ggml_tensor *hc_in[2] = {nullptr, nullptr}, *hc_out[2] = {nullptr, nullptr}, *hc_mix[2] = {nullptr, nullptr};
+    // ... the slope per head of a linear distance penalty; a correction per expert that enters the choice of experts only
+    ggml_tensor *attn_slopes = nullptr, *ffn_corr = nullptr;
     // ... a per-layer token input: the layer's part of a second embedding table, a gate on the stream, the projection back and the norm weight
     ggml_tensor *side_embd = nullptr, *side_gate = nullptr, *side_proj = nullptr, *side_norm = nullptr;
 };
@@ -404,12 +408,26 @@ struct llm_layer_cfg {
     int ssm_state = 0, ssm_groups = 1, ssm_norm_groups = 1;  // state-space mixer (LLM_MIX_SSD): state size per head, groups of (B, C), parts of the gated norm; n_head x dv = inner
     int r_head = 0, r_head_kv = 0, r_dk = 0, r_dv = 0, r_rank = 0;  // the delta rule beside an attention (LLM_MIX_ATTN_DELTA): heads, key heads, sizes, inner size of decay / gate
     int side_dim = 0;                               // > 0: the per-layer token input of this many entries
+    bool dist_linear = false;                       // score -= slope_h (i - j) (attn_slopes)
+    int q_temp_id = -1;                             // >= 0: queries are multiplied by a factor that grows with their position (llm_model::q_temps)
+    bool ffn_gelu_tanh = false;                     // dense feed-forward W_down gelu_tanh(W_up h)
+    // mixture of experts: scores are sigmoids; the choice goes by score + correction (ffn_corr), the weights are the chosen scores divided by their sum (+ 1e-20); experts are
+    // W_down (g sigmoid(1.702 g) (u + 1)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit)
+    bool moe_sigmoid = false;
+    float moe_limit = 0.0f;
 };
 // what a layer's positions may see: one attention mask per distinct rule of a model
 struct llm_mask_rule {
     int chunk = 0, window = 0, keep_first = 0;
     bool distance = false;  // the mask holds i - j for visible pairs instead of 0 (layers with a distance penalty)
     bool operator==(const llm_mask_rule & o) const { return chunk == o.chunk && window == o.window && keep_first == o.keep_first && distance == o.distance; }
+};
+// a factor on the queries that grows with the position: 1 + coef ln(floor((p + 1) / every) + 1).  One input per distinct rule of a model
+struct llm_q_temp {
+    double coef = 0.0;
+    int every = 1;
+    float at(int64_t p) const { return (float) (1.0 + coef * log((double) ((p + 1) / every) + 1.0)); }
+    bool operator==(const llm_q_temp & o) const { return coef == o.coef && every == o.every; }
 };
 // one execution of a layer: a model may run a range of its layers several times in a row with the same weights; every run has its own cache and state
 struct llm_run {
@@ -457,6 +475,9 @@ struct llm_model {
     // layers [loop_start, loop_stop) run loop_times times in a row; before each pass x <- loop_in [x; embedding output] + loop_step[pass]
     int loop_start = 0, loop_stop = 0, loop_times = 0;
     ggml_tensor *loop_in = nullptr, *loop_step = nullptr;
+    std::vector<llm_q_temp> q_temps;     // the distinct query factors of the layers
+    int n_streams = 0;                   // > 0: the residual stream is kept as this many streams, mixed around every sublayer (llm_layer::hc_*)
+    float residual_mult = 1.0f;          // ... and a sublayer's output joins them times this
     bool has_shift = false;              // some layer keeps the previous token's normed input as sequence state
     bool has_seq_state = false;          // some layer keeps convolution inputs / a recurrence's matrices per sequence: the batch is described by (hist, upd, tok, info)
     int hist_rows = 0;                   // the longest look-back of those layers (taps - 1)
@@ -845,6 +866,27 @@ static int mask_rule_id(llm_model * m, const llm_mask_rule & r) {
     return (int) k;
 }
 
+// config key 'loop': layers start .. stop - 1 run `times` times in a row
+static bool parse_loop(const json_value & cfg, llm_model * m, std::string & err) {
+    const json_value * lp = cfg.get("loop");
+    if (!lp || lp->kind != json_value::OBJ) return true;
+    auto num = [&](const char * k, double d) { const json_value * x = lp->get(k); return x ? x->number(d) : d; };
+    m->loop_start = (int) num("start", 0);
+    m->loop_stop = (int) num("stop", 0);
+    m->loop_times = (int) num("times", 1);
+    if (m->loop_start < 0 || m->loop_stop > m->hp.n_layer || m->loop_start >= m->loop_stop || m->loop_times < 1) { err = "config: inconsistent loop"; return false; }
+    return true;
+}
+// the order of execution: layers before the repeated range, the range `times` times, the rest (between_passes: something happens to the stream where a pass begins)
+static void make_runs(llm_model * m, bool between_passes) {
+    const int n = m->hp.n_layer;
+    for (int il = 0; il < (m->loop_times > 0 ? m->loop_start : n); ++il) m->runs.push_back({il, -1, false});
+    if (m->loop_times <= 0) return;
+    for (int t = 0; t < m->loop_times; ++t)
+        for (int il = m->loop_start; il < m->loop_stop; ++il) m->runs.push_back({il, t, between_passes && il == m->loop_start});
+    for (int il = m->loop_stop; il < n; ++il) m->runs.push_back({il, -1, false});
+}
+
 static bool parse_nigozen_config(const json_value & cfg, llm_model * m, std::string & err) {
     llm_hparams & hp = m->hp;
     snprintf(hp.arch, sizeof(hp.arch), "nigozen");
@@ -935,12 +977,7 @@ static bool parse_zigipel_config(const json_value & cfg, llm_model * m, std::str
         m->bg_mul_cur = (int) num(bg, "mul_cur", nullptr, 0);
         if (m->bg_buckets <= 0) { err = "config: bigram embedding without buckets"; return false; }
     }
-    if (const json_value * lp = cfg.get("loop")) {
-        m->loop_start = (int) num(lp, "start", nullptr, 0);
-        m->loop_stop = (int) num(lp, "stop", nullptr, 0);
-        m->loop_times = (int) num(lp, "times", nullptr, 1);
-        if (m->loop_start < 0 || m->loop_stop > hp.n_layer || m->loop_start >= m->loop_stop || m->loop_times < 1) { err = "config: inconsistent loop"; return false; }
-    }
+    if (!parse_loop(cfg, m, err)) return false;
     m->lcfg.resize((size_t) hp.n_layer);
     for (int il = 0; il < hp.n_layer; ++il) {
         const json_value & L = layers->arr[(size_t) il];
@@ -1001,13 +1038,7 @@ static bool parse_zigipel_config(const json_value & cfg, llm_model * m, std::str
     m->has_shift = true;
     hp.n_head = m->lcfg[0].n_head; hp.n_head_kv = m->lcfg[0].n_head_kv; hp.n_embd_head = m->lcfg[0].dk; hp.n_ff = m->lcfg[0].n_ff;
     hp.rope_freq_base = m->lcfg[0].rot_base;
-    // the order of execution: layers before the repeated range, the range `times` times, the rest
-    for (int il = 0; il < (m->loop_times > 0 ? m->loop_start : hp.n_layer); ++il) m->runs.push_back({il, -1, false});
-    if (m->loop_times > 0) {
-        for (int t = 0; t < m->loop_times; ++t)
-            for (int il = m->loop_start; il < m->loop_stop; ++il) m->runs.push_back({il, t, il == m->loop_start});
-        for (int il = m->loop_stop; il < hp.n_layer; ++il) m->runs.push_back({il, -1, false});
-    }
+    make_runs(m, true);
     return true;
 }
 
@@ -1029,14 +1060,7 @@ static bool parse_rarelorn_config(const json_value & cfg, const st_file * file, 
     hp.n_ctx_train = 1 << 20;
     if (hp.n_embd <= 0 || hp.n_vocab <= 0) { err = "config: width / vocab missing"; return false; }
     auto num = [&](const json_value * o, const char * k0, const char * k1, double d) { const json_value * x = o->path(k0, k1); return x ? x->number(d) : d; };
-    if (const json_value * lp = cfg.get("loop")) {
-        if (lp->kind == json_value::OBJ) {
-            m->loop_start = (int) num(lp, "start", nullptr, 0);
-            m->loop_stop = (int) num(lp, "stop", nullptr, 0);
-            m->loop_times = (int) num(lp, "times", nullptr, 1);
-            if (m->loop_start < 0 || m->loop_stop > hp.n_layer || m->loop_start >= m->loop_stop || m->loop_times < 1) { err = "config: inconsistent loop"; return false; }
-        }
-    }
+    if (!parse_loop(cfg, m, err)) return false;
     m->lcfg.resize((size_t) hp.n_layer);
     m->has_attn = false;
     m->has_seq_state = true;
@@ -1121,12 +1145,7 @@ static bool parse_rarelorn_config(const json_value & cfg, const st_file * file, 
     }
     hp.n_head = m->lcfg[0].n_head; hp.n_head_kv = m->lcfg[0].n_head_kv; hp.n_embd_head = m->lcfg[0].dk; hp.n_ff = m->lcfg[0].n_ff;
     hp.rope_freq_base = m->lcfg[0].rot_base;
-    for (int il = 0; il < (m->loop_times > 0 ? m->loop_start : hp.n_layer); ++il) m->runs.push_back({il, -1, false});
-    if (m->loop_times > 0) {
-        for (int t = 0; t < m->loop_times; ++t)
-            for (int il = m->loop_start; il < m->loop_stop; ++il) m->runs.push_back({il, t, il == m->loop_start});
-        for (int il = m->loop_stop; il < hp.n_layer; ++il) m->runs.push_back({il, -1, false});
-    }
+    make_runs(m, true);
     return true;
 }
 
@@ -1529,6 +1548,167 @@ static std::vector<dir_tensor> nogavik_plan(const llm_model * m) {
     return plan;
 }
 
+// Pisulorn: pre-norm layers over SEVERAL residual streams (hyper-connections: in front of a sublayer the streams are weighted into one row, behind it every stream becomes a mixture of all
+// plus a share of the output times residual_mult).  Mixers: grouped-query attention without rotation (per-head normed queries and keys, a query factor that grows with the position, a linear
+// distance penalty per head, a sliding window) and a gated delta rule behind short convolutions.  Feed-forward: tanh-GELU, or experts with a limited gated activation chosen by sigmoid scores
+// plus a correction.  A range of layers repeats, nothing happening between its passes.
+static bool parse_pisulorn_config(const json_value & cfg, llm_model * m, std::string & err) {
+    llm_hparams & hp = m->hp;
+    snprintf(hp.arch, sizeof(hp.arch), "pisulorn");
+    const json_value * layers = cfg.get("layers");
+    if (!layers || layers->kind != json_value::ARR || layers->arr.empty()) { err = "config: no layers"; return false; }
+    const json_value * v;
+    hp.n_embd = (v = cfg.get("width")) ? (int) v->number(0) : 0;
+    hp.n_vocab = (v = cfg.get("vocab")) ? (int) v->number(0) : 0;
+    hp.rms_eps = (v = cfg.path("norm", "eps")) ? (float) v->number(1e-5) : 1e-5f;
+    m->residual_mult = (v = cfg.get("residual_mult")) ? (float) v->number(1.0) : 1.0f;
+    m->n_streams = (v = cfg.get("streams")) ? (int) v->number(1) : 1;
+    hp.n_layer = (int) layers->arr.size();
+    hp.n_ctx_train = 1 << 20;
+    if (hp.n_embd <= 0 || hp.n_vocab <= 0) { err = "config: width / vocab missing"; return false; }
+    if (m->n_streams < 1 || m->n_streams > 8) { err = "config: 1 to 8 streams"; return false; }
+    if (!parse_loop(cfg, m, err)) return false;
+    auto num = [&](const json_value * o, const char * k0, const char * k1, double d) { const json_value * x = o->path(k0, k1); return x ? x->number(d) : d; };
+    auto sub = [&](const json_value * o, const char * k) { const json_value * x = o->get(k); return x && x->kind == json_value::OBJ ? x : nullptr; };
+    m->lcfg.resize((size_t) hp.n_layer);
+    m->has_attn = false;
+    m->has_seq_state = false;
+    m->hist_rows = 0;
+    for (int il = 0; il < hp.n_layer; ++il) {
+        const json_value & L = layers->arr[(size_t) il];
+        llm_layer_cfg & c = m->lcfg[(size_t) il];
+        const std::string lname = "config: layer " + std::to_string(il);
+        const json_value * type = L.get("type");
+        const json_value * mx = L.get("mixer");
+        if (!type || type->kind != json_value::STR || !mx || mx->kind != json_value::OBJ) { err = lname + ": no mixer"; return false; }
+        c.rms = true;
+        c.n_head = (int) num(mx, "heads", nullptr, 0);
+        c.n_head_kv = (int) num(mx, "kv_heads", nullptr, c.n_head);
+        c.dk = (int) num(mx, "dim", nullptr, 0);
+        c.dv = (int) num(mx, "vdim", nullptr, c.dk);
+        if (c.n_head <= 0 || c.n_head_kv <= 0 || c.n_head % c.n_head_kv || c.dk <= 0 || c.dv <= 0) { err = lname + ": inconsistent head sizes"; return false; }
+        if (type->str == "attention") {
+            c.mixer = LLM_MIX_ATTN;
+            c.scale = (float) num(mx, "scale", nullptr, 1.0 / sqrt((double) c.dk));
+            c.qk_norm = c.dist_linear = true;
+            llm_mask_rule rule;
+            rule.distance = true;
+            if (const json_value * mk = sub(mx, "mask")) {
+                rule.window = c.window = (int) num(mk, "size", nullptr, 0);
+                if (c.window < 1) { err = lname + ": a window of less than one token"; return false; }
+            }
+            c.mask_id = mask_rule_id(m, rule);
+            if (const json_value * qt = sub(mx, "q_temp")) {
+                llm_q_temp t;
+                t.coef = num(qt, "coef", nullptr, 0.0);
+                t.every = (int) num(qt, "every", nullptr, 0);
+                if (t.every < 1) { err = lname + ": q_temp.every must be at least 1"; return false; }
+                size_t k = 0;
+                while (k < m->q_temps.size() && !(m->q_temps[k] == t)) ++k;
+                if (k == m->q_temps.size()) m->q_temps.push_back(t);
+                c.q_temp_id = (int) k;
+            }
+            m->has_attn = true;
+            m->max_embd_k = std::max(m->max_embd_k, c.n_head_kv * c.dk);
+            m->max_embd_v = std::max(m->max_embd_v, c.n_head_kv * c.dv);
+        } else if (type->str == "delta") {
+            c.mixer = LLM_MIX_DELTA;
+            c.conv_taps = (int) num(mx, "conv", nullptr, 1);
+            if (c.conv_taps < 1 || c.conv_taps > 16 || c.dk > 256) { err = lname + ": inconsistent delta-rule sizes"; return false; }
+            m->has_seq_state = true;
+            m->hist_rows = std::max(m->hist_rows, c.conv_taps - 1);
+        } else { err = lname + ": unknown mixer type"; return false; }
+        if (const json_value * ml = sub(&L, "mlp")) {
+            const json_value * kind = ml->get("kind");
+            if (kind && kind->kind == json_value::STR && kind->str == "dense") {
+                c.mlp = LLM_MLP_DENSE;
+                c.ffn_gelu_tanh = true;
+                c.n_ff = (int) num(ml, "ff", nullptr, 0);
+            } else if (kind && kind->kind == json_value::STR && kind->str == "moe") {
+                c.mlp = LLM_MLP_MOE;
+                c.moe_sigmoid = true;
+                c.n_ff = (int) num(ml, "expert", "ff", 0);
+                c.moe_limit = (float) num(ml, "expert", "limit", 0.0);
+                c.n_expert = (int) num(ml, "router", "experts", 0);
+                c.n_top = (int) num(ml, "router", "top", 0);
+                if (c.n_expert <= 0 || c.n_top <= 0 || c.n_top > c.n_expert || !(c.moe_limit > 0.0f)) { err = lname + ": inconsistent experts"; return false; }
+            } else { err = lname + ": unknown mlp kind"; return false; }
+            if (c.n_ff <= 0) { err = lname + ": ff missing"; return false; }
+        }
+    }
+    hp.n_head = m->lcfg[0].n_head; hp.n_head_kv = m->lcfg[0].n_head_kv; hp.n_embd_head = m->lcfg[0].dk; hp.n_ff = m->lcfg[0].n_ff;
+    make_runs(m, false);
+    return true;
+}
+
+static std::vector<dir_tensor> pisulorn_plan(const llm_model * m) {
+    const llm_hparams & hp = m->hp;
+    const ggml_type wt = m->wtype;
+    const int64_t E = hp.n_embd, N = m->n_streams;
+    std::vector<dir_tensor> plan;
+    auto add = [&](const std::string & name, ggml_type t, int64_t n0, int64_t n1, int64_t n2, std::vector<std::string> src, float gain) -> dir_tensor & {
+        dir_tensor d;
+        d.name = name; d.type = t; d.ne[0] = n0; d.ne[1] = n1; d.ne[2] = n2; d.src = std::move(src); d.synth_gain = gain;
+        plan.push_back(std::move(d));
+        return plan.back();
+    };
+    auto uniform = [&](const std::string & name, int64_t n0, int64_t n1, std::vector<std::string> src, float lo, float hi) {
+        dir_tensor & t = add(name, GGML_TYPE_F32, n0, n1, 1, std::move(src), 0.0f);
+        t.synth_lo = lo; t.synth_hi = hi;
+    };
+    add("token_embd.weight", wt, E, hp.n_vocab, 1, {"embed"}, sqrtf((float) E));
+    for (int il = 0; il < hp.n_layer; ++il) {
+        const llm_layer_cfg & c = m->lcfg[(size_t) il];
+        const std::string p = "blk." + std::to_string(il) + ".", q = "l" + std::to_string(il) + ".", x = q + "mix.";
+        const int64_t H = c.n_head, G = c.n_head_kv;
+        for (int k = 0; k < (c.mlp == LLM_MLP_NONE ? 1 : 2); ++k) {
+            const std::string hc = q + "hc" + std::to_string(k + 1) + ".", f = p + (k == 0 ? "attn_" : "ffn_");
+            uniform(f + "norm.weight", E, 1, {q + "norm" + std::to_string(k + 1)}, 0.7f, 1.4f);
+            uniform(f + "streams_in.weight", N, 1, {hc + "in"}, 0.2f, 1.0f);
+            uniform(f + "streams_out.weight", N, 1, {hc + "out"}, 0.5f, 1.5f);
+            uniform(f + "streams_mix.weight", N, N, {hc + "mix"}, 0.0f, 1.0f / (float) N);
+        }
+        if (c.mixer == LLM_MIX_ATTN) {
+            add(p + "attn_q.weight", wt, E, H * c.dk, 1, {x + "q"}, 1.0f);
+            add(p + "attn_k.weight", wt, E, G * c.dk, 1, {x + "k"}, 1.0f);
+            add(p + "attn_v.weight", wt, E, G * c.dv, 1, {x + "v"}, 1.0f);
+            uniform(p + "attn_q_norm.weight", c.dk, 1, {x + "q.norm"}, 0.7f, 1.4f);
+            uniform(p + "attn_k_norm.weight", c.dk, 1, {x + "k.norm"}, 0.7f, 1.4f);
+            std::vector<float> slopes((size_t) H);
+            for (int64_t h = 0; h < H; ++h) slopes[(size_t) h] = (float) exp2(-8.0 * (double) (h + 1) / (double) H);
+            add(p + "attn_slopes.weight", GGML_TYPE_F32, H, 1, 1, {}, 0.0f).values = slopes;
+        } else {
+            const int64_t C = 2 * G * c.dk + H * c.dv;
+            add(p + "attn_qkv.weight", wt, E, C, 1, {x + "q", x + "k", x + "v"}, 2.0f);
+            add(p + "ssm_conv1d.weight", GGML_TYPE_F32, c.conv_taps, C, 1, {x + "q.conv", x + "k.conv", x + "v.conv"}, 1.0f);
+            add(p + "attn_gates.weight", wt, E, 2 * H, 1, {x + "b", x + "a"}, 2.0f);
+            uniform(p + "attn_gates.param", 2 * H, 1, {x + "A_log", x + "dt_bias"}, -1.5f, 0.5f);
+            add(p + "attn_gate.weight", wt, E, H * c.dv, 1, {x + "g"}, 1.0f);
+            uniform(p + "attn_sub_norm.weight", c.dv, 1, {x + "norm"}, 0.7f, 1.4f);
+        }
+        add(p + "attn_output.weight", wt, H * c.dv, E, 1, {x + "o"}, 1.0f);
+        if (c.mlp == LLM_MLP_DENSE) {
+            add(p + "ffn_up.weight", wt, E, c.n_ff, 1, {q + "mlp.up"}, 1.4f);
+            add(p + "ffn_down.weight", wt, c.n_ff, E, 1, {q + "mlp.down"}, 1.0f);
+        } else if (c.mlp == LLM_MLP_MOE) {
+            std::vector<std::string> gu, downs;
+            for (int e = 0; e < c.n_expert; ++e) {
+                const std::string pe = q + "mlp.e" + std::to_string(e) + ".";
+                gu.push_back(pe + "gate");
+                gu.push_back(pe + "up");
+                downs.push_back(pe + "down");
+            }
+            add(p + "ffn_gate_inp.weight", GGML_TYPE_F32, E, c.n_expert, 1, {q + "mlp.router"}, 3.0f);  // router logits are 32-bit in every mode
+            uniform(p + "ffn_choice.bias", c.n_expert, 1, {q + "mlp.correction"}, -0.3f, 0.3f);
+            add(p + "ffn_gate_up_exps.weight", wt, E, 2 * c.n_ff, c.n_expert, gu, 1.4f);                // per expert: its gate rows, then its up rows
+            add(p + "ffn_down_exps.weight", wt, c.n_ff, E, c.n_expert, downs, 1.0f);
+        }
+    }
+    uniform("output_norm.weight", E, 1, {"final.norm"}, 0.7f, 1.4f);
+    add("output.weight", wt, E, hp.n_vocab, 1, {"head"}, 1.0f);
+    return plan;
+}
+
 // values of one checkpoint tensor (bf16 / f32 / f16 in the file) as `type` (bf16 or f32) into dst
 static bool convert_values(const st_tensor & t, ggml_type type, uint8_t * dst) {
     const int64_t n = t.numel();
@@ -1570,6 +1750,9 @@ static llm_model * model_from_config(const json_value & cfg, const st_file * fil
     } else if (arch->str == "Nogavik") {
         if (!parse_nogavik_config(cfg, file, m, err)) { fprintf(stderr, "llm_model_load_dir: %s\n", err.c_str()); delete m; return nullptr; }
         plan = nogavik_plan(m);
+    } else if (arch->str == "Pisulorn") {
+        if (!parse_pisulorn_config(cfg, m, err)) { fprintf(stderr, "llm_model_load_dir: %s\n", err.c_str()); delete m; return nullptr; }
+        plan = pisulorn_plan(m);
     } else {
         fprintf(stderr, "llm_model_load_dir: unknown architecture \"%s\"\n", arch->str.c_str());
         delete m;
@@ -1748,12 +1931,18 @@ static llm_model * model_from_config(const json_value & cfg, const st_file * fil
         L.ssm_in_z = g("ssm_in_z.weight"); L.ssm_in_xbc = g("ssm_in_xbc.weight"); L.ssm_in_dt = g("ssm_in_dt.weight"); L.conv_b = g("ssm_conv1d.bias");
         if (!L.gate_par) L.gate_par = g("ssm_params.weight");
         L.side_embd = g("side_embd.weight"); L.side_gate = g("side_gate.weight"); L.side_proj = g("side_proj.weight"); L.side_norm = g("side_norm.weight");
+        for (int k = 0; k < 2; ++k) {
+            const std::string f = k == 0 ? "attn_streams_" : "ffn_streams_";
+            L.hc_in[k] = g((f + "in.weight").c_str()); L.hc_out[k] = g((f + "out.weight").c_str()); L.hc_mix[k] = g((f + "mix.weight").c_str());
+        }
+        L.attn_slopes = g("attn_slopes.weight"); L.ffn_corr = g("ffn_choice.bias");
         L.wdkv = g("attn_kv_a.weight"); L.dkv_norm = g("attn_kv_a_norm.weight"); L.wuk_t = g("attn_k_b_t.weight"); L.wuv = g("attn_v_b.weight"); L.rope_freq = g("rope_freq.weight");
         for (ggml_tensor * t : {L.attn_norm, L.attn_post_norm, L.wq, L.wk, L.wv, L.attn_gate, L.wo, L.ffn_norm, L.ffn_post_norm, L.ffn_up, L.ffn_down, L.ffn_gate_inp,
                                 L.attn_sink, L.attn_r12, L.shift, L.ffn_gate, L.ffn_gate_b, L.ffn_up_b, L.ffn_down_b, L.wdkv, L.dkv_norm, L.wuk_t, L.wuv, L.rope_freq,
                                 L.wqkv, L.bqkv, L.conv, L.wgates, L.gate_par, L.sub_norm, L.bo, L.attn_fb, L.tm_taps, L.tm_rkvg, L.tm_w1, L.tm_w2, L.tm_w0, L.tm_u, L.tm_norm, L.tm_out,
                                 L.bq, L.bk, L.bv, L.q_norm, L.k_norm, L.wdq, L.dq_norm, L.wbeta, L.wa1, L.wa2, L.wg1, L.wg2, L.wo_r, L.left_norm, L.right_norm, L.ssm_in_z, L.ssm_in_xbc,
-                                L.ssm_in_dt, L.conv_b, L.side_gate, L.side_proj, L.side_norm})
+                                L.ssm_in_dt, L.conv_b, L.side_gate, L.side_proj, L.side_norm, L.hc_in[0], L.hc_in[1], L.hc_out[0], L.hc_out[1], L.hc_mix[0], L.hc_mix[1],
+                                L.attn_slopes, L.ffn_corr})
             if (t) sbytes += ggml_nbytes(t) * (uint64_t) std::max(1, times_run[(size_t) il]);  // (a layer of a repeated range is streamed once per run)
         if (L.side_embd) sbytes += ggml_row_size(L.side_embd->type, L.side_embd->ne[0]);  // (one row of the layer's part of the side table)
         if (c.mlp == LLM_MLP_MOE) sbytes += (ggml_nbytes(L.ffn_gate_up_exps ? L.ffn_gate_up_exps : L.ffn_up_exps) + ggml_nbytes(L.ffn_down_exps)) / (uint64_t) c.n_expert * (uint64_t) c.n_top *
@@ -1866,6 +2055,7 @@ struct seg_io {
     ggml_tensor * bigram_rows = nullptr;  // row of the bigram table per token (hashed on the host from the previous and the current token)
     // token shift: per token the row of [h of this batch | state rows] that holds the previous token's h; per sequence of the batch its last token and its state row
     ggml_tensor *shift_src = nullptr, *shift_last = nullptr, *shift_slot = nullptr;
+    std::vector<ggml_tensor *> q_temps;   // per distinct rule: the factor of every token's query, [1, 1, T]
     // layers with convolution / recurrence state: where a token's predecessors are found, where the new state rows come from, the batch rows grouped by sequence,
     // and per sequence of the batch (first entry, count, state slot, starts here)
     ggml_tensor *seq_hist = nullptr, *seq_upd = nullptr, *seq_tok = nullptr, *seq_info = nullptr;
@@ -1906,6 +2096,7 @@ struct llm_context {
     ggml_tensor *inp_tokens = nullptr, *inp_pos = nullptr, *inp_mask = nullptr, *inp_k_idxs = nullptr, *inp_v_idxs = nullptr, *inp_out_ids = nullptr;
     ggml_tensor *inp_bigram = nullptr, *inp_shift_src = nullptr, *inp_shift_last = nullptr, *inp_shift_slot = nullptr;
     ggml_tensor *inp_seq_hist = nullptr, *inp_seq_upd = nullptr, *inp_seq_tok = nullptr, *inp_seq_info = nullptr;
+    std::vector<ggml_tensor *> inp_q_temps;
     std::vector<ggml_tensor *> inp_masks;  // all masks of the graph (inp_masks[0] == inp_mask)
     ggml_tensor * t_logits = nullptr;
     // outputs
@@ -2011,6 +2202,10 @@ static void make_inputs(llm_context * c, ggml_context * ctx, int l0, int l1, boo
         ggml_set_input(named(io.shift_last, "shift_last_rows", -1));
         io.shift_slot = ggml_new_tensor_1d(ctx, GGML_TYPE_I64, std::max(1, n_seqs));
         ggml_set_input(named(io.shift_slot, "shift_slots", -1));
+    }
+    for (size_t k = 0; k < m->q_temps.size(); ++k) {
+        io.q_temps.push_back(ggml_new_tensor_3d(ctx, GGML_TYPE_F32, 1, 1, n_tokens));
+        ggml_set_input(named(io.q_temps.back(), "q_temp", (int) k));
     }
     if (m->has_attn) {
         io.k_idxs = ggml_new_tensor_1d(ctx, GGML_TYPE_I64, n_tokens);
@@ -2178,12 +2373,18 @@ static ggml_tensor * build_mixer_attention(llm_context * c, ggml_context * ctx, 
     if (L.bq) Qcur = named(ggml_add(ctx, Qcur, L.bq), "Qcur_b", run);
     if (L.bk) Kcur = named(ggml_add(ctx, Kcur, L.bk), "Kcur_b", run);
     if (L.bv) Vcur = named(ggml_add(ctx, Vcur, L.bv), "Vcur_b", run);
+    if (lc.dist_linear) {  // (the three products of the one input follow one another; the per-head norms and the cache stores then do too, which the backend runs as one launch)
+        ggml_build_forward_expand(gf, Qcur);
+        ggml_build_forward_expand(gf, Kcur);
+        ggml_build_forward_expand(gf, Vcur);
+    }
     Qcur = ggml_reshape_3d(ctx, Qcur, DK, H, n_tokens);
     Kcur = ggml_reshape_3d(ctx, Kcur, DK, G, n_tokens);
     if (lc.qk_norm) {  // every head's query and key divided by its root mean square, times a weight row shared by the heads
         Qcur = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, Qcur, hp.rms_eps), "Qcur_rnorm", run), L.q_norm), "Qcur_normed", run);
         Kcur = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, Kcur, hp.rms_eps), "Kcur_rnorm", run), L.k_norm), "Kcur_normed", run);
     }
+    if (lc.q_temp_id >= 0) Qcur = named(ggml_mul(ctx, Qcur, io.q_temps[(size_t) lc.q_temp_id]), "Qcur_temp", run);
     if (lc.rot_dims > 0) {  // neighbouring pairs (2i, 2i + 1) of the leading rot_dims entries; the rest of the head passes through
         Qcur = named(ggml_rope_ext(ctx, Qcur, io.pos, nullptr, lc.rot_dims, lc.rot_half ? GGML_ROPE_TYPE_NEOX : 0, hp.n_ctx_train, lc.rot_base, 1.0f, 0.0f, 1.0f, 32.0f, 1.0f), "Qcur_rope", run);
         Kcur = named(ggml_rope_ext(ctx, Kcur, io.pos, nullptr, lc.rot_dims, lc.rot_half ? GGML_ROPE_TYPE_NEOX : 0, hp.n_ctx_train, lc.rot_base, 1.0f, 0.0f, 1.0f, 32.0f, 1.0f), "Kcur_rope", run);
@@ -2213,6 +2414,7 @@ static ggml_tensor * build_mixer_attention(llm_context * c, ggml_context * ctx, 
     cur = ggml_flash_attn_ext(ctx, q, k, v, io.masks[(size_t) lc.mask_id], lc.scale, 0.0f, 0.0f);
     ggml_flash_attn_ext_set_prec(cur, GGML_PREC_F32);
     if (lc.sink) ggml_flash_attn_ext_add_sinks(cur, lc.sink_learned ? L.attn_sink : ggml_view_1d(ctx, m->attn_sinks, H, 0));
+    if (lc.dist_linear) ggml_flash_attn_ext_add_linear_distance(cur, L.attn_slopes);
     if (lc.dist_pen) ggml_flash_attn_ext_add_log_distance(cur, ggml_reshape_2d(ctx, L.attn_r12, H, 2));
     named(cur, "fattn", run);
     if (gate && lc.gate_heads) {  // one number per head and token
@@ -2510,7 +2712,33 @@ static ggml_tensor * build_moe_grouped(ggml_context * ctx, ggml_cgraph * gf, con
     return named(out, "ffn_moe_out", il);
 }
 
+// experts chosen by sigmoid scores plus a correction; the weights are the chosen scores themselves divided by their sum; experts with a limited gated activation
+static ggml_tensor * build_moe_sigmoid(ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & c, ggml_tensor * cur, int run) {
+    const int64_t E = cur->ne[0], T = cur->ne[1], FF = c.n_ff;
+    ggml_tensor * logits = named(ggml_mul_mat(ctx, L.ffn_gate_inp, cur), "ffn_moe_logits", run);  // [n_expert, T], f32 weights: 32-bit
+    ggml_tensor * probs = named(ggml_unary(ctx, logits, GGML_UNARY_OP_SIGMOID), "ffn_moe_probs", run);
+    ggml_tensor * order = named(ggml_argsort(ctx, L.ffn_corr ? named(ggml_add(ctx, probs, L.ffn_corr), "ffn_moe_choice", run) : probs, 1), "ffn_moe_order", run);
+    ggml_tensor * sel = ggml_view_2d(ctx, order, c.n_top, T, order->nb[1], 0);  // [n_top, T] i32
+    ggml_tensor * w = named(ggml_get_rows(ctx, ggml_reshape_3d(ctx, probs, 1, c.n_expert, T), sel), "ffn_moe_sel_probs", run);  // [1, n_top, T]
+    w = ggml_reshape_2d(ctx, w, c.n_top, T);
+    w = named(ggml_div(ctx, w, named(ggml_scale_bias(ctx, named(ggml_sum_rows(ctx, w), "ffn_moe_sum", run), 1.0f, 1e-20f), "ffn_moe_sum_eps", run)), "ffn_moe_weights", run);
+    ggml_build_forward_expand(gf, w);  // (the weights before the experts' products: the router is then one run of nodes, which the backend takes as one launch)
+    ggml_tensor * gu = named(ggml_mul_mat_id(ctx, L.ffn_gate_up_exps, ggml_reshape_3d(ctx, cur, E, 1, T), sel), "ffn_moe_gate_up", run);  // [2 ff, n_top, T]: gate rows, then up rows
+    ggml_tensor * act = named(ggml_swiglu_oai(ctx, ggml_reshape_2d(ctx, gu, 2 * FF, c.n_top * T), nullptr, 1.702f, c.moe_limit), "ffn_moe_act", run);
+    ggml_tensor * down = named(ggml_mul_mat_id(ctx, L.ffn_down_exps, ggml_reshape_3d(ctx, act, FF, c.n_top, T), sel), "ffn_moe_down", run);  // [E, n_top, T]
+    down = named(ggml_mul(ctx, down, ggml_reshape_3d(ctx, w, 1, c.n_top, T)), "ffn_moe_weighted", run);
+    ggml_build_forward_expand(gf, down);
+    ggml_tensor * out = nullptr;
+    for (int j = 0; j < c.n_top; ++j) {
+        ggml_tensor * v = ggml_view_2d(ctx, down, E, T, down->nb[2], (size_t) j * down->nb[1]);
+        out = out ? ggml_add(ctx, out, v) : v;
+    }
+    if (c.n_top == 1) out = ggml_cont(ctx, out);
+    return named(out, "ffn_moe_out", run);
+}
+
 static ggml_tensor * build_ffn(ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * cur, int il, int run) {
+    if (lc.mlp == LLM_MLP_MOE && lc.moe_sigmoid) return build_moe_sigmoid(ctx, gf, L, lc, cur, run);
     if (lc.mlp == LLM_MLP_MOE) return lc.moe_scores_all ? build_moe_grouped(ctx, gf, L, lc, cur, il) : build_moe(ctx, gf, L, lc, cur, il);
     if (lc.ffn_gated_tanh) {
         ggml_tensor * g = named(ggml_add(ctx, named(ggml_mul_mat(ctx, L.ffn_gate, cur), "ffn_gate", run), L.ffn_gate_b), "ffn_gate_b", run);
@@ -2520,8 +2748,56 @@ static ggml_tensor * build_ffn(ggml_context * ctx, ggml_cgraph * gf, const llm_l
     }
     cur = named(ggml_mul_mat(ctx, L.ffn_up, cur), "ffn_up", run);
     if (lc.ffn_relu_sq) cur = named(ggml_sqr(ctx, named(ggml_unary(ctx, cur, GGML_UNARY_OP_RELU), "ffn_relu", run)), "ffn_act", run);
-    else cur = named(ggml_unary(ctx, cur, GGML_UNARY_OP_GELU_ERF), "ffn_gelu", run);
+    else cur = named(ggml_unary(ctx, cur, lc.ffn_gelu_tanh ? GGML_UNARY_OP_GELU : GGML_UNARY_OP_GELU_ERF), "ffn_gelu", run);
     return named(ggml_mul_mat(ctx, L.ffn_down, cur), "ffn_out", run);
+}
+
+// the mixer of one layer run, its output projection included: [n_embd, T]
+static ggml_tensor * build_mixer(llm_context * c, ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * cur, int il, int run, int n_tokens, int n_kv,
+                                 seg_io & io, ggml_tensor ** v_first) {
+    switch (lc.mixer) {
+        case LLM_MIX_MLSTM: return build_mixer_mlstm(c, ctx, gf, L, lc, cur, run, n_tokens, io);
+        case LLM_MIX_DELTA: return build_mixer_delta(c, ctx, gf, L, lc, cur, run, n_tokens, io);
+        case LLM_MIX_SIGMOID_WKV: return build_mixer_sigmoid_wkv(c, ctx, gf, L, lc, cur, run, n_tokens, n_kv, io);
+        case LLM_MIX_SSD: return build_mixer_ssd(c, ctx, gf, L, lc, cur, run, n_tokens, io);
+        case LLM_MIX_ATTN_DELTA: return build_mixer_attn_delta(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io);
+        case LLM_MIX_LATENT: cur = build_mixer_latent(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io); break;
+        default: cur = build_mixer_attention(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, v_first); break;
+    }
+    return named(ggml_mul_mat(ctx, L.wo, cur), "attn_out", run);
+}
+
+// the layers of a model whose residual stream is kept as several streams: one op per boundary between two sublayers (the streams' update behind one, the weighting and the norm in front of
+// the next), the first one spreading the embedding over the streams, the last one summing them under the output norm.  Returns the normed rows the output matrix reads
+static ggml_tensor * build_stream_layers(llm_context * c, ggml_context * ctx, ggml_cgraph * gf, ggml_tensor * x, int n_tokens, int n_kv, seg_io & io) {
+    llm_model * m = c->model;
+    const float eps = m->hp.rms_eps, mult = m->residual_mult;
+    const int N = m->n_streams, n_runs = (int) m->runs.size();
+    ggml_tensor * y = x, * streams = nullptr, * v_first = nullptr;  // what joins the streams next, and the streams
+    const llm_layer * from = nullptr;                               // ... with the (mix, out) of this layer's sublayer `from_sub`
+    int from_sub = 0;
+    auto boundary = [&](ggml_tensor * in, ggml_tensor * norm, bool rows_out, bool keep, const char * name, int run) {
+        ggml_tensor * st = named(ggml_stream_step(ctx, y, streams, from ? from->hc_mix[from_sub] : nullptr, from ? from->hc_out[from_sub] : nullptr, in, norm, rows_out ? io.out_ids : nullptr,
+                                                  N, keep ? 1 : 0, mult, eps), name, run);
+        streams = keep ? ggml_stream_step_streams(ctx, st) : nullptr;
+        return ggml_stream_step_rows(ctx, st);
+    };
+    bool rows_chosen = false;
+    for (int run = 0; run < n_runs; ++run) {
+        const int il = m->runs[(size_t) run].il;
+        const llm_layer & L = m->layers[(size_t) il];
+        const llm_layer_cfg & lc = m->lcfg[(size_t) il];
+        ggml_tensor * h = boundary(L.hc_in[0], L.attn_norm, false, true, "streams_attn", run);
+        y = build_mixer(c, ctx, gf, L, lc, h, il, run, n_tokens, n_kv, io, &v_first);
+        from = &L;
+        from_sub = 0;
+        if (lc.mlp == LLM_MLP_NONE) continue;
+        rows_chosen = run == n_runs - 1;  // (behind the last mixer only the rows whose logits are wanted go on)
+        h = boundary(L.hc_in[1], L.ffn_norm, rows_chosen, true, "streams_ffn", run);
+        y = build_ffn(ctx, gf, L, lc, h, il, run);
+        from_sub = 1;
+    }
+    return boundary(nullptr, m->output_norm, !rows_chosen, false, "result_norm", -1);
 }
 
 static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * gf, int n_tokens, int n_kv, seg_io & io) {
@@ -2533,7 +2809,7 @@ static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * g
     if (m->bigram) inpL = named(ggml_add(ctx, inpL, named(ggml_get_rows(ctx, m->bigram, io.bigram_rows), "inp_bigram", -1)), "inp_sum", -1);
     ggml_tensor * const embd_out = inpL;
     ggml_tensor * v_first = nullptr;
-    const int n_runs = (int) m->runs.size();
+    const int n_runs = m->n_streams > 0 ? 0 : (int) m->runs.size();
     for (int run = 0; run < n_runs; ++run) {
         const int il = m->runs[(size_t) run].il;
         const llm_layer & L = m->layers[(size_t) il];
@@ -2549,16 +2825,7 @@ static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * g
         ggml_tensor * inpSA = inpL;
         ggml_tensor * h = norm_w(ctx, lc, inpL, L.attn_norm, eps, "attn_norm", run);
         ggml_tensor * cur = lc.shift ? build_token_shift(c, ctx, gf, h, L.shift, run, io) : h;
-        if (lc.mixer == LLM_MIX_MLSTM) cur = build_mixer_mlstm(c, ctx, gf, L, lc, cur, run, n_tokens, io);
-        else if (lc.mixer == LLM_MIX_DELTA) cur = build_mixer_delta(c, ctx, gf, L, lc, cur, run, n_tokens, io);
-        else if (lc.mixer == LLM_MIX_SIGMOID_WKV) cur = build_mixer_sigmoid_wkv(c, ctx, gf, L, lc, cur, run, n_tokens, n_kv, io);
-        else if (lc.mixer == LLM_MIX_SSD) cur = build_mixer_ssd(c, ctx, gf, L, lc, cur, run, n_tokens, io);
-        else if (lc.mixer == LLM_MIX_ATTN_DELTA) cur = build_mixer_attn_delta(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io);
-        else {
-            cur = lc.mixer == LLM_MIX_LATENT ? build_mixer_latent(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io)
-                                             : build_mixer_attention(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, &v_first);
-            cur = named(ggml_mul_mat(ctx, L.wo, cur), "attn_out", run);
-        }
+        cur = build_mixer(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, &v_first);
         if (lc.parallel) {  // both sublayers read the one normed input (the feed-forward the unshifted one); their sum joins the stream
             if (last && io.out_ids) {  // only the rows whose logits are wanted go on from here
                 cur = ggml_get_rows(ctx, cur, io.out_ids);
@@ -2589,7 +2856,8 @@ static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * g
         inpL = named(ggml_add(ctx, cur, ffn_inp), "l_out", run);
     }
     const bool rms_out = !m->lcfg.empty() && m->lcfg[0].rms;
-    ggml_tensor * cur = rms_out ? named(ggml_mul(ctx, named(ggml_rms_norm(ctx, inpL, eps), "rnorm", -1), m->output_norm), "result_norm", -1)
+    ggml_tensor * cur = m->n_streams > 0 ? build_stream_layers(c, ctx, gf, inpL, n_tokens, n_kv, io)
+                      : rms_out ? named(ggml_mul(ctx, named(ggml_rms_norm(ctx, inpL, eps), "rnorm", -1), m->output_norm), "result_norm", -1)
                                 : layer_norm_w(ctx, inpL, m->output_norm, eps, "result_norm", -1);
     cur = named(ggml_mul_mat(ctx, m->output, cur), m->logit_scale != 1.0f ? "result_unscaled" : "result_output", -1);
     if (m->logit_scale != 1.0f) cur = named(ggml_scale(ctx, cur, m->logit_scale), "result_output", -1);
@@ -2607,6 +2875,7 @@ static void build_graph(llm_context * c, int n_tokens, int n_kv, int n_outputs, 
     if (!c->model->lcfg.empty()) build_layerwise(c, c->ctx_compute, gf, n_tokens, n_kv, io);
     else build_segment(c, c->ctx_compute, gf, 0, c->model->hp.n_layer, true, n_tokens, n_kv, io);
     c->inp_masks = io.masks;
+    c->inp_q_temps = io.q_temps;
     c->inp_tokens = io.tokens;
     c->inp_pos = io.pos;
     c->inp_mask = io.mask;
@@ -2739,6 +3008,7 @@ extern "C" struct llm_context * llm_context_new(struct llm_model * m, ggml_backe
             size_t in_bytes = nub * (4 + 4 + 8 + 4) + std::max<size_t>(1, m->mask_rules.size()) * (n_tok_pad * (size_t) c->p.n_ctx * 4 + 64) + 256;
             in_bytes += nub * (4 + 4) + (size_t) c->n_seq_max * (4 + 8) + 4 * 64;  // bigram rows, token-shift sources, the sequences' last rows and state rows
             in_bytes += (nub + (size_t) c->n_seq_max) * (size_t) (m->hist_rows + 4) * 4 + 4 * 64;  // predecessors, new state rows, rows grouped by sequence, the sequences' entries
+            in_bytes += m->q_temps.size() * (nub * 4 + 64);
             if (!c->p.flash_attn) in_bytes += nub * (size_t) n_embd_k * 8;
             in_bytes = (in_bytes + 255) / 256 * 256;
             c->pin_out_rows = 64;
@@ -3160,6 +3430,11 @@ static int decode_ubatch(llm_context * c, int n_tokens, const int32_t * tokens, 
     };
     upload(c->inp_tokens, (size_t) n_tokens * 4, [&](char * d) { memcpy(d, tokens, (size_t) n_tokens * 4); });
     if (c->inp_pos) upload(c->inp_pos, (size_t) n_tokens * 4, [&](char * d) { memcpy(d, pos, (size_t) n_tokens * 4); });
+    for (size_t k = 0; k < c->inp_q_temps.size(); ++k)
+        upload(c->inp_q_temps[k], (size_t) n_tokens * 4, [&](char * d) {
+            float * f = (float *) d;
+            for (int i = 0; i < n_tokens; ++i) f[i] = m->q_temps[k].at(pos[i]);
+        });
     if (c->inp_k_idxs) upload(c->inp_k_idxs, (size_t) n_tokens * 8, [&](char * d) {
         int64_t * k = (int64_t *) d;
         for (int i = 0; i < n_tokens; ++i) k[i] = slots[i];
