@@ -224,6 +224,32 @@ def nogavik_config(z):
     return {"architecture": "Nogavik", "layers": [latent(), ssm, latent(0), par, ssm, par], "norm": {"eps": 1e-5}, "token_side": {"dim": z["side"]}, "vocab": z["vocab"], "width": z["width"]}
 
 
+# ------------------------------------------------------------------------------------------------ --pisulorn: several residual streams, windowed attention with a linear distance
+# penalty beside a gated delta rule, dense and expert feed-forwards; beside Rarelorn (delta rule, experts) and Zigipel (windowed attention with a distance penalty) at equal size
+PISULORN_SIZES = {
+    # width, heads, kv heads, head size, window, taps, streams, dense ff (ungated: two matrices), experts, top, expert ff (gated: three matrices), vocab.  Four layers (delta + dense, attention +
+    # experts, delta + experts, attention + dense), the middle two run twice: six layer runs, as many as the models beside it have
+    "s": dict(width=1024, heads=8, kv=2, hd=64, window=512, taps=4, streams=4, ff=4128, experts=8, top=2, eff=1024, vocab=32000),
+    "m": dict(width=2048, heads=16, kv=4, hd=128, window=1024, taps=4, streams=4, ff=8256, experts=8, top=2, eff=2048, vocab=32000),
+    "l": dict(width=4096, heads=32, kv=8, hd=128, window=2048, taps=4, streams=4, ff=14400, experts=8, top=2, eff=4096, vocab=32000),
+}
+
+
+def pisulorn_config(z):
+    H, G, D = z["heads"], z["kv"], z["hd"]
+    dense = {"kind": "dense", "ff": z["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": z["eff"], "limit": 7.0}, "router": {"experts": z["experts"], "top": z["top"]}}
+
+    def delta(mlp):
+        return {"type": "delta", "mlp": mlp, "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "conv": z["taps"]}}
+
+    def attention(mlp):
+        return {"type": "attention", "mlp": mlp, "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": z["window"]}, "q_temp": {"coef": 0.1, "every": 512}}}
+
+    return {"architecture": "Pisulorn", "layers": [delta(dense), attention(moe), delta(moe), attention(dense)], "loop": {"start": 1, "stop": 3, "times": 2}, "norm": {"eps": 1e-5},
+            "residual_mult": 0.5, "streams": z["streams"], "vocab": z["vocab"], "width": z["width"]}
+
+
 def bench_nigozen(args):
     """Prefill and decode throughput of Nigozen models (bf16 matrices, bf16 cache, random weights) at sizes that resemble real layers, beside the
     closest existing class at equal size: llama with f16 matrices and an f16 cache (same width, layers, heads, head size, dense ff and vocabulary;
@@ -239,7 +265,8 @@ def bench_nigozen(args):
 
     be = L.Backend(0)
     n_prompt, n_dec, ub = args.prefill, max(8, min(args.steps, 64)), args.ubatch
-    if (args.zigipel or args.rarelorn or args.nogavik) and n_prompt == 2048:
+    many_sided = bool(args.zigipel or args.rarelorn or args.nogavik or args.pisulorn)
+    if many_sided and n_prompt == 2048:
         # decoded positions 1984 .. 2047: a model confined to chunks of 512 / 1024 / 2048 positions then sees 449 .. 512 / 961 .. 1024 / 1985 .. 2048 cells, about as many as a
         # sliding window of the same length does (right behind a chunk's start it would see next to nothing, and the two decode steps would not compare)
         n_prompt = 1984
@@ -252,7 +279,7 @@ def bench_nigozen(args):
         prompt = rng.integers(0, n_vocab, n_prompt).tolist()
         res = {}
         best_p, best_d = None, None
-        best_of = bool(args.zigipel or args.rarelorn or args.nogavik)
+        best_of = many_sided
         for rep in range(4 if best_of else 2):  # the first pass warms up (graph capture, scratch growth); the Zigipel comparison keeps the best of the three that follow
             ctx.clear()
             be.synchronize()
@@ -288,6 +315,27 @@ def bench_nigozen(args):
         ctx.free()
         return res
 
+    if args.pisulorn:  # Pisulorn beside Rarelorn (its delta rule and experts) and Zigipel (its windowed attention): as many layer runs, equal width, heads, head size, vocabulary and parameters
+        out["metric"] = "pisulorn_vs_rarelorn_tokens_per_s"
+        out["dtype"] = "bf16 (all)"
+        be.close()
+        for name in args.pisulorn.split(","):
+            z = PISULORN_SIZES[name]
+            res = {}
+            for side, cfg in (("pisulorn", pisulorn_config(z)), ("rarelorn", rarelorn_config(RARELORN_SIZES[name])), ("zigipel", zigipel_config(dict(ZIGIPEL_SIZES[name], ff=z["ff"] * 2 // 3)))):
+                be = L.Backend(0)
+                mdl = Model(config_json=_json.dumps(cfg), seed=7, buft=be.buft, wtype=L.BF16)
+                res[side] = run(mdl, z["vocab"])
+                res[side]["weight_bytes"] = int(L.host().llm_model_total_bytes(mdl.m))
+                res[side]["stream_bytes_per_token"] = mdl.stream_bytes()
+                mdl.free()
+                be.close()
+            out["sizes"][name] = {"config": z, **res}
+            for other in ("rarelorn", "zigipel"):
+                out["sizes"][name]["prefill_ratio_" + other] = round(res["pisulorn"]["prefill_tok_s"] / res[other]["prefill_tok_s"], 3)
+                out["sizes"][name]["decode_ratio_" + other] = round(res["pisulorn"]["decode_tok_s"] / res[other]["decode_tok_s"], 3)
+        print(_json.dumps(out))
+        return
     if args.nogavik:  # Nogavik beside Zigipel (as many layer runs, equal width, heads, head size, latent, vocabulary and feed-forward parameters) and Rarelorn (the recurrences)
         out["metric"] = "nogavik_vs_zigipel_tokens_per_s"
         out["dtype"] = "bf16 (all)"
@@ -382,6 +430,9 @@ def main():
     ap.add_argument("--nogavik", default="", help="comma-separated sizes (s, m, l): time prefill and decode of Nogavik models (latent attention with shared cache rows, a state-space "
                     "mixer, attention beside a delta rule with channel decay, a per-layer token input) beside Zigipel and Rarelorn models of equal size, print one JSON line and exit; "
                     "the default workload is not run")
+    ap.add_argument("--pisulorn", default="", help="comma-separated sizes (s, m, l): time prefill and decode of Pisulorn models (several residual streams, windowed attention with a linear "
+                    "distance penalty, a gated delta rule, dense and expert feed-forwards, a repeated range) beside Rarelorn and Zigipel models of equal size, print one JSON line and exit; "
+                    "the default workload is not run")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
     ap.add_argument("--warmup", type=int, default=8)
@@ -410,7 +461,7 @@ def main():
     ap.add_argument("--pmc-traffic", type=int, default=1, help="1: re-run a short decode under rocprofv3 --pmc FETCH_SIZE (own pass) for roofline.traffic")
     args = ap.parse_args()
 
-    if args.nigozen or args.zigipel or args.rarelorn or args.nogavik:
+    if args.nigozen or args.zigipel or args.rarelorn or args.nogavik or args.pisulorn:
         bench_nigozen(args)
         return
 

@@ -2722,6 +2722,7 @@ static ggml_tensor * build_moe_sigmoid(ggml_context * ctx, ggml_cgraph * gf, con
     ggml_tensor * w = named(ggml_get_rows(ctx, ggml_reshape_3d(ctx, probs, 1, c.n_expert, T), sel), "ffn_moe_sel_probs", run);  // [1, n_top, T]
     w = ggml_reshape_2d(ctx, w, c.n_top, T);
     w = named(ggml_div(ctx, w, named(ggml_scale_bias(ctx, named(ggml_sum_rows(ctx, w), "ffn_moe_sum", run), 1.0f, 1e-20f), "ffn_moe_sum_eps", run)), "ffn_moe_weights", run);
+    ggml_set_output(w);                // (its few bytes are not handed to another tensor: the weighted sum over the experts reads them to its last row)
     ggml_build_forward_expand(gf, w);  // (the weights before the experts' products: the router is then one run of nodes, which the backend takes as one launch)
     ggml_tensor * gu = named(ggml_mul_mat_id(ctx, L.ffn_gate_up_exps, ggml_reshape_3d(ctx, cur, E, 1, T), sel), "ffn_moe_gate_up", run);  // [2 ff, n_top, T]: gate rows, then up rows
     ggml_tensor * act = named(ggml_swiglu_oai(ctx, ggml_reshape_2d(ctx, gu, 2 * FF, c.n_top * T), nullptr, 1.702f, c.moe_limit), "ffn_moe_act", run);
