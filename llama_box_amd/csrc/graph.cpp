@@ -137,7 +137,8 @@ static int rope_exact_freq(const ggml_tensor * n) {
 //   RWKV_WKV6, op_params (H): src (r, k, v, w_pre [D H, T], w0 [D H], u [D H], state, tok [T] i32, info) -> [D, H, T]
 //   GATED_LINEAR_ATTN, op_params (kind 1 delta rule / 2 matrix memory, H, G, tag, cap, q scale): src (q, k [DK G, T], v [DV H, T], gates [2 H, T], params [2 H], state, tok, info) -> [DV, H, T]
 //                      kind 3 (delta rule, one decay per key channel): gates = a_pre [DK H, T], params = A_log [H] then dt_bias [DK H], src[8] = b_pre [H, T];
-//                      kind 4 (state-space duality): q = C, k = B [N G, T], v = x, gates = dt_pre [H, T], params = A_log, dt_bias, D [3 H]
+//                      kind 4 (state-space duality): q = C, k = B [N G, T], v = x, gates = dt_pre [H, T], params = A_log, dt_bias, D [3 H];
+//                      kind 5 (gated linear attention, G = H): gates = a_pre [DK H, T], params = offset [DK H], cap = tau
 //   SSM_CONV mode 0 may carry src[4]: a bias [C, M] added before the activation
 static constexpr int32_t MI_SEQ_OP_TAG = 0x5E9;
 static bool seq_op_ok(const ggml_tensor * op) {
@@ -157,7 +158,7 @@ static bool seq_op_ok(const ggml_tensor * op) {
     }
     const bool wkv = op->op == GGML_OP_RWKV_WKV6;
     const int kind = wkv ? SEQ_WKV6 : op->op_params[0];
-    if (!wkv && kind != SEQ_DELTA && kind != SEQ_MLSTM && kind != SEQ_DELTA_CH && kind != SEQ_SSD) return false;
+    if (!wkv && kind != SEQ_DELTA && kind != SEQ_MLSTM && kind != SEQ_DELTA_CH && kind != SEQ_SSD && kind != SEQ_LINEAR) return false;
     const int H = wkv ? op->op_params[0] : op->op_params[1], G = wkv ? H : op->op_params[2];
     const ggml_tensor * state = src[wkv ? 6 : 5], * tok = src[wkv ? 7 : 6], * info = src[wkv ? 8 : 7];
     if (H < 1 || G < 1 || H % G || !f32rows(src[0]) || !f32rows(src[1]) || !f32rows(src[2]) || !f32rows(src[3]) || !f32c(src[4]) || !f32c(state) || !i32c(tok) || !i32c(info)) return false;
@@ -166,8 +167,9 @@ static bool seq_op_ok(const ggml_tensor * op) {
     if (src[0]->ne[0] % G || src[2]->ne[0] % H) return false;
     const int64_t DK = src[0]->ne[0] / G, DV = src[2]->ne[0] / H;
     if (!seq_recurrence_ok((int) DK, (int) DV) || src[1]->ne[0] != DK * G || src[1]->ne[1] != T || src[2]->ne[1] != T || src[3]->ne[1] != T) return false;
-    const int64_t n_gates = (wkv || kind == SEQ_DELTA_CH) ? DK * H : kind == SEQ_SSD ? H : 2 * H;
-    const int64_t n_par = wkv ? DK * H : kind == SEQ_DELTA_CH ? H + DK * H : kind == SEQ_SSD ? 3 * H : 2 * H;
+    const int64_t n_gates = (wkv || kind == SEQ_DELTA_CH || kind == SEQ_LINEAR) ? DK * H : kind == SEQ_SSD ? H : 2 * H;
+    if (kind == SEQ_LINEAR && (G != H || !(ggml_abi_op_param_f32(op, 4) > 0.0f))) return false;
+    const int64_t n_par = (wkv || kind == SEQ_LINEAR) ? DK * H : kind == SEQ_DELTA_CH ? H + DK * H : kind == SEQ_SSD ? 3 * H : 2 * H;
     if (src[3]->ne[0] != n_gates || ggml_abi_nelements(src[4]) != n_par || (wkv && ggml_abi_nelements(src[5]) != DK * H)) return false;
     if (kind == SEQ_DELTA_CH && (!f32rows(src[8]) || src[8]->ne[0] != H || src[8]->ne[1] != T)) return false;
     if (ggml_abi_nelements(tok) != T || info->ne[0] != 4 || state->ne[0] != seq_recurrence_state_floats(kind, H, (int) DK, (int) DV)) return false;
@@ -356,8 +358,8 @@ static ws_plan plan_ws(backend_ctx * c, const ggml_cgraph * g) {
                 p.aux_bytes = std::max(p.aux_bytes, attn_nf_mma_ws_bytes(TD(n->src[1]), fattn_mma_pick_splits(TD(n->src[1]), TD(n->src[0]))));
         } else if (n->op == GGML_OP_MUL_MAT_ID && n->src[2]) {
             p.aux_bytes = std::max(p.aux_bytes, mul_mat_id_workspace_bytes(TD(n->src[0]), TD(n->src[2])));
-        } else if (n->op == GGML_OP_GATED_LINEAR_ATTN && n->op_params[3] == MI_SEQ_OP_TAG && n->op_params[0] == SEQ_DELTA_CH && n->src[0] && n->src[3]) {
-            p.aux_bytes = std::max(p.aux_bytes, seq_recurrence_scratch_bytes(SEQ_DELTA_CH, n->op_params[1], (int) (n->src[0]->ne[0] / std::max(1, n->op_params[2])), n->src[3]->ne[1]));
+        } else if (n->op == GGML_OP_GATED_LINEAR_ATTN && n->op_params[3] == MI_SEQ_OP_TAG && (n->op_params[0] == SEQ_DELTA_CH || n->op_params[0] == SEQ_LINEAR) && n->src[0] && n->src[3]) {
+            p.aux_bytes = std::max(p.aux_bytes, seq_recurrence_scratch_bytes(n->op_params[0], n->op_params[1], (int) (n->src[0]->ne[0] / std::max(1, n->op_params[2])), n->src[3]->ne[1]));
         } else if (n->op == GGML_OP_FLASH_ATTN_EXT && fa_route(n) == 4) {
             continue;  // the 32-bit kernels keep their running sums on chip
         } else if (n->op == GGML_OP_FLASH_ATTN_EXT) {

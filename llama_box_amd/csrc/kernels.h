@@ -389,10 +389,10 @@ void launch_seq_conv(hipStream_t s, const tdesc & x, const float * w, const floa
 void launch_seq_conv_store(hipStream_t s, const tdesc & x, float * state, const int32_t * upd, int hs, const int32_t * info, int n_seqs, int taps);
 struct seq_rec_args {
     tdesc q, k, v;             // [rows, T] f32 (rows contiguous): q / r, k and v of all heads
-    tdesc g;                   // wkv6: w_pre [D H, T]; delta: (b_pre, a_pre) [2 H, T]; mlstm: (i_pre, f_pre) [2 H, T]; channel decay: a_pre [DK H, T]; state space: dt_pre [H, T]
+    tdesc g;                   // wkv6: w_pre [D H, T]; delta: (b_pre, a_pre) [2 H, T]; mlstm: (i_pre, f_pre) [2 H, T]; channel decay, linear: a_pre [DK H, T]; state space: dt_pre [H, T]
     tdesc b;                   // channel decay: b_pre [H, T]
     const float * p0;          // wkv6: w0 [D H]; delta: A_log [H] then dt_bias [H]; mlstm: bias of (i, f) [2 H]; channel decay: A_log [H] then dt_bias [DK H];
-                               // state space: A_log [H], dt_bias [H], D [H]
+                               // state space: A_log [H], dt_bias [H], D [H]; linear: offset of every (head, channel) [DK H]
     const float * p1;          // wkv6: u [D H]
     float * state;             // per slot: H matrices of 4 ceil(DK / 4) DV values, then (mlstm) H x DK normaliser entries and H running maxima
     int64_t state_stride;      // floats per slot
@@ -400,14 +400,14 @@ struct seq_rec_args {
     const int32_t * info;
     tdesc dst;                 // [DV, H, T]
     int DK, DV, H, G;          // G: key heads (head h reads q / k head h / (H / G))
-    float cap, qscale;
-    int w_ready;               // channel decay: g already holds the decays themselves (a pass of their own computed them)
+    float cap, qscale;         // cap: the matrix memory's gate cap; linear: tau
+    int w_ready;               // channel decay, linear: g already holds the decays themselves (a pass of their own computed them)
 };
 
-enum { SEQ_WKV6 = 0, SEQ_DELTA = 1, SEQ_MLSTM = 2, SEQ_DELTA_CH = 3, SEQ_SSD = 4 };
+enum { SEQ_WKV6 = 0, SEQ_DELTA = 1, SEQ_MLSTM = 2, SEQ_DELTA_CH = 3, SEQ_SSD = 4, SEQ_LINEAR = 5 };
 int64_t seq_recurrence_state_floats(int kind, int H, int DK, int DV);
 bool seq_recurrence_ok(int DK, int DV);
-// scratch (optional): seq_recurrence_scratch_bytes() bytes let the channel-decay kind compute a prompt portion's decays in one parallel pass
+// scratch (optional): seq_recurrence_scratch_bytes() bytes let the kinds with a decay per key channel compute a prompt portion's decays in one parallel pass
 size_t seq_recurrence_scratch_bytes(int kind, int H, int DK, int64_t T);
 void launch_seq_recurrence(hipStream_t s, int kind, const seq_rec_args & a, int n_seqs, void * scratch = nullptr, size_t scratch_bytes = 0);
 // SOFT_MAX over a router's logits, the (group-limited) descending ARGSORT of the scores, GET_ROWS of the k first and SCALE in one launch (n <= 256 experts)

@@ -18,6 +18,7 @@
 //                     raw a [DK H, T] being a projection of its own; beta = sigmoid(b_pre) from a [H, T] projection; the rest as SEQ_DELTA
 //   k_seq_recurrence<SEQ_SSD>    state-space duality (Mamba-2): dt = softplus(dt_pre + dt_bias); S <- exp(-exp(A_log) dt) S + dt B x^T; y = S^T C + D x, with B as the keys,
 //                     C as the queries (grouped: head h reads group h / (H / G)) and x as the values
+//   k_seq_recurrence<SEQ_LINEAR>  gated linear attention: S <- diag(w) S + k v^T, w = sigmoid(a + offset)^(1 / tau) per key channel; o = S^T q dk^-1/2
 //   k_seq_recurrence<SEQ_MLSTM>  matrix memory with exponential gates under a running maximum m: m' = max(f + m, i); S <- e^(f + m - m') S + e^(i - m') k v^T; n likewise with k;
 //                     o = S^T q / (max(|n . q|, e^(-m')) + 1e-6); log gates capped by cap tanh(. / cap), f through log-sigmoid
 // All arithmetic is f32; the state is f32.  The three recurrences share one thread layout: a wave per (sequence of the batch, head, 4 value columns); value column j
@@ -99,6 +100,7 @@ __device__ __forceinline__ float quad_sum(float x) {  // sum over the 16 lanes o
 }
 __device__ __forceinline__ float seq_softplus(const float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float seq_log_sigmoid(const float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float seq_linear_decay(const float z, const float tau) { return expf(seq_log_sigmoid(z) / tau); }  // sigmoid(z)^(1 / tau)
 
 
 // One WAVE per (sequence of the batch, head, group of 4 value columns).  The tokens' vectors come in blocks of TB tokens: while block b is worked on out of LDS, block
@@ -114,8 +116,8 @@ constexpr int SEQ_DECAY_PREPASS_MIN = 32;  // batches of this many tokens and mo
 // key rows a lane owns: a sixteenth of the head's rows, rounded up to whole groups of four (its rows are neighbours, read from LDS sixteen bytes at a time)
 static inline __host__ __device__ int seq_rows_per_lane(const int DK) { return (((DK + SEQ_LPC - 1) / SEQ_LPC) + 3) / 4 * 4; }
 // which kinds carry a decay per key channel among a token's entries, and which carry raw gates of the head
-static inline __host__ __device__ bool seq_has_w(const int kind) { return kind == SEQ_WKV6 || kind == SEQ_DELTA_CH; }
-static inline __host__ __device__ bool seq_has_gates(const int kind) { return kind != SEQ_WKV6; }
+static inline __host__ __device__ bool seq_has_w(const int kind) { return kind == SEQ_WKV6 || kind == SEQ_DELTA_CH || kind == SEQ_LINEAR; }
+static inline __host__ __device__ bool seq_has_gates(const int kind) { return kind != SEQ_WKV6 && kind != SEQ_LINEAR; }
 // floats a token occupies in a staged block (at least a wave's stride: the walk over a block's entries then crosses at most one token per step)
 static inline __host__ __device__ int seq_per_tok(const int kind, const int DK) {
     const int n = (seq_has_w(kind) ? 3 : 2) * SEQ_LPC * seq_rows_per_lane(DK) + SEQ_COLS + (seq_has_gates(kind) ? 4 : 0);
@@ -133,7 +135,7 @@ __global__ void __launch_bounds__(64) k_seq_recurrence(const seq_rec_args A, con
     const bool col = j < DV;
     const int RL = seq_rows_per_lane(DK), KP = SEQ_LPC * RL;  // lane ks owns rows ks RL .. ks RL + RL - 1; a token's key-sized vectors are padded with zeros to KP entries
     const int kh = KIND == SEQ_WKV6 ? h : h / (H / A.G);
-    constexpr bool HAS_W = KIND == SEQ_WKV6 || KIND == SEQ_DELTA_CH, HAS_G = KIND != SEQ_WKV6, IS_DELTA = KIND == SEQ_DELTA || KIND == SEQ_DELTA_CH;
+    constexpr bool HAS_W = KIND == SEQ_WKV6 || KIND == SEQ_DELTA_CH || KIND == SEQ_LINEAR, HAS_G = KIND != SEQ_WKV6 && KIND != SEQ_LINEAR, IS_DELTA = KIND == SEQ_DELTA || KIND == SEQ_DELTA_CH;
     const int off_w = 2 * KP, off_v = HAS_W ? 3 * KP : 2 * KP, off_g = off_v + SEQ_COLS;
     const int per_tok = seq_per_tok(KIND, DK);
     float * __restrict__ Sm = A.state + (int64_t) slot * A.state_stride + (int64_t) h * RL * DV * SEQ_LPC;
@@ -172,9 +174,9 @@ __global__ void __launch_bounds__(64) k_seq_recurrence(const seq_rec_args A, con
             const int idx = (is_k || is_q) ? kh * DK + fe : is_w ? h * DK + fe : is_v ? h * DV + j0 + fe : (KIND == SEQ_DELTA_CH || KIND == SEQ_SSD) ? h : fe * H + h;
             const int64_t t = rows[valid ? u : 0];
             float val = ((const float *) (base + t * nb1))[valid ? idx : 0];
-            if (HAS_W) {  // the decay's offset: w0 (time mixing), or the dt_bias entries behind the heads' A_log (channel decay)
+            if (HAS_W) {  // the decay's offset: w0 (time mixing), the dt_bias entries behind the heads' A_log (channel decay), or the offsets alone (linear)
                 const float off = A.p0[(is_w && valid) ? (KIND == SEQ_DELTA_CH ? H : 0) + h * DK + fe : 0];
-                val = (is_w && !(KIND == SEQ_DELTA_CH && A.w_ready)) ? val + off : val;  // (w_ready: the operand already holds the decays themselves)
+                val = (is_w && !((KIND == SEQ_DELTA_CH || KIND == SEQ_LINEAR) && A.w_ready)) ? val + off : val;  // (w_ready: the operand already holds the decays themselves)
             }
             pre[i] = valid ? val : 0.0f;
             f += 64;
@@ -207,14 +209,14 @@ __global__ void __launch_bounds__(64) k_seq_recurrence(const seq_rec_args A, con
             *gp = y;
         }
     };
-    // channel decay: the parked raw values (projection + offset) of a block's n_tok tokens become exp(-e^A softplus(.)) — the lanes walk over the DK real entries of
+    // channel decay: the parked raw values (projection + offset) of a block's n_tok tokens become exp(-e^A softplus(.)) (linear: sigmoid(.)^(1 / tau)) — the lanes walk over the DK real entries of
     // every token only, so the softplus and the two exponentials are paid once per entry (not once per staged float)
     auto finish_decay = [&](float * dstb, const int n_tok) {
-        if (KIND == SEQ_DELTA_CH && !A.w_ready)
+        if ((KIND == SEQ_DELTA_CH || KIND == SEQ_LINEAR) && !A.w_ready)
             for (int idx = lane; idx < n_tok * DK; idx += 64) {
                 const int u = idx / DK, fe = idx - u * DK;
                 float * wp = dstb + u * per_tok + off_w + fe;
-                *wp = expf(-a_exp * seq_softplus(*wp));
+                *wp = KIND == SEQ_LINEAR ? seq_linear_decay(*wp, A.cap) : expf(-a_exp * seq_softplus(*wp));
             }
     };
     float pre[SEQ_NV];
@@ -238,7 +240,46 @@ __global__ void __launch_bounds__(64) k_seq_recurrence(const seq_rec_args A, con
             fetch(rows_of[(b + 1) & 1], n_next, pre);
             if (lane < TB && b0 + 2 * TB + lane < count) row_after = A.tok[begin + b0 + 2 * TB + lane];
         }
-        if (KIND == SEQ_SSD) {
+        if (KIND == SEQ_LINEAR) {
+            // as below, the state's update waits for nothing but the state: the next token's vectors are requested ahead
+            float4 nk[R / 4], nq[R / 4], nw[R / 4];
+            float nv;
+            auto stage = [&](const int u) {
+                const float * lt = cur + u * per_tok;
+                const float4 * k4 = (const float4 *) (lt + ks * RL), * q4 = (const float4 *) (lt + KP + ks * RL), * w4 = (const float4 *) (lt + off_w + ks * RL);
+#pragma unroll
+                for (int m = 0; m < R / 4; ++m) {
+                    nk[m] = make_float4(0.f, 0.f, 0.f, 0.f);
+                    nq[m] = nw[m] = nk[m];
+                    if (EXACT || 4 * m < RL) { nk[m] = k4[m]; nq[m] = q4[m]; nw[m] = w4[m]; }
+                }
+                nv = lt[off_v + (lane >> 4)];
+            };
+            stage(0);
+            for (int u = 0; u < n_here; ++u) {
+                float4 kk[R / 4], qq[R / 4], ww[R / 4];
+#pragma unroll
+                for (int m = 0; m < R / 4; ++m) { kk[m] = nk[m]; qq[m] = nq[m]; ww[m] = nw[m]; }
+                const float vj = nv;
+                if (u + 1 < n_here) stage(u + 1);
+                float p0 = 0.0f, p1 = 0.0f, p2 = 0.0f, p3 = 0.0f;
+#pragma unroll
+                for (int m = 0; m < R / 4; ++m) {
+                    if (EXACT || 4 * m < RL) {
+                        S[4 * m] = fmaf(ww[m].x, S[4 * m], kk[m].x * vj);
+                        S[4 * m + 1] = fmaf(ww[m].y, S[4 * m + 1], kk[m].y * vj);
+                        S[4 * m + 2] = fmaf(ww[m].z, S[4 * m + 2], kk[m].z * vj);
+                        S[4 * m + 3] = fmaf(ww[m].w, S[4 * m + 3], kk[m].w * vj);
+                        p0 = fmaf(S[4 * m], qq[m].x, p0);
+                        p1 = fmaf(S[4 * m + 1], qq[m].y, p1);
+                        p2 = fmaf(S[4 * m + 2], qq[m].z, p2);
+                        p3 = fmaf(S[4 * m + 3], qq[m].w, p3);
+                    }
+                }
+                const float o = quad_sum((p0 + p1) + (p2 + p3)) * A.qscale;
+                if (col && ks == 0) ((float *) (A.dst.data + (int64_t) h * A.dst.nb[1] + (int64_t) trow[u] * A.dst.nb[2]))[j] = o;
+            }
+        } else if (KIND == SEQ_SSD) {
             // the state's update waits for nothing but the state (the read-out is beside the chain), so what a token costs is the trip to LDS for its vectors: the next
             // token's are requested before the current token's arithmetic (the delta rules and the matrix memory, whose tokens are chains of dependent reductions, gain
             // nothing from the same: measured, and left as they are)
@@ -408,7 +449,13 @@ __global__ void __launch_bounds__(256) k_seq_channel_decay(const tdesc a, const 
     const float val = ((const float *) (a.data + t * a.nb[1]))[c] + p0[H + c];
     out[t * C + c] = expf(-a_exp * seq_softplus(val));
 }
-size_t seq_recurrence_scratch_bytes(int kind, int H, int DK, int64_t T) { return (kind == SEQ_DELTA_CH && T >= SEQ_DECAY_PREPASS_MIN) ? (size_t) T * H * DK * sizeof(float) : 0; }
+// ... and those of linear attention, out[t][c] = sigmoid(a[t][c] + offset[c])^(1 / tau)
+__global__ void __launch_bounds__(256) k_seq_linear_decay(const tdesc a, const float * __restrict__ p0, const int64_t C, const float tau, float * __restrict__ out) {
+    const int64_t t = blockIdx.y, c = (int64_t) blockIdx.x * 256 + threadIdx.x;
+    if (c >= C) return;
+    out[t * C + c] = seq_linear_decay(((const float *) (a.data + t * a.nb[1]))[c] + p0[c], tau);
+}
+size_t seq_recurrence_scratch_bytes(int kind, int H, int DK, int64_t T) { return ((kind == SEQ_DELTA_CH || kind == SEQ_LINEAR) && T >= SEQ_DECAY_PREPASS_MIN) ? (size_t) T * H * DK * sizeof(float) : 0; }
 
 // floats of state one slot needs
 int64_t seq_recurrence_state_floats(int kind, int H, int DK, int DV) {
@@ -440,7 +487,8 @@ void launch_seq_recurrence(hipStream_t s, int kind, const seq_rec_args & a_in, i
     const size_t need = seq_recurrence_scratch_bytes(kind, a.H, a.DK, T);
     if (need > 0 && scratch && need <= scratch_bytes) {  // a prompt portion: the decays of all its tokens in one parallel pass
         const int64_t C = (int64_t) a.H * a.DK;
-        hipLaunchKernelGGL(k_seq_channel_decay, dim3((unsigned) ((C + 255) / 256), (unsigned) T), dim3(256), 0, s, a.g, a.p0, a.H, a.DK, (float *) scratch);
+        if (kind == SEQ_LINEAR) hipLaunchKernelGGL(k_seq_linear_decay, dim3((unsigned) ((C + 255) / 256), (unsigned) T), dim3(256), 0, s, a.g, a.p0, C, a.cap, (float *) scratch);
+        else hipLaunchKernelGGL(k_seq_channel_decay, dim3((unsigned) ((C + 255) / 256), (unsigned) T), dim3(256), 0, s, a.g, a.p0, a.H, a.DK, (float *) scratch);
         a.g.data = (char *) scratch;
         a.g.nb[0] = 4;
         a.g.nb[1] = C * 4;
@@ -450,6 +498,7 @@ void launch_seq_recurrence(hipStream_t s, int kind, const seq_rec_args & a_in, i
     else if (kind == SEQ_DELTA) seq_recurrence_launch<SEQ_DELTA>(s, a, n_seqs);
     else if (kind == SEQ_DELTA_CH) seq_recurrence_launch<SEQ_DELTA_CH>(s, a, n_seqs);
     else if (kind == SEQ_SSD) seq_recurrence_launch<SEQ_SSD>(s, a, n_seqs);
+    else if (kind == SEQ_LINEAR) seq_recurrence_launch<SEQ_LINEAR>(s, a, n_seqs);
     else seq_recurrence_launch<SEQ_MLSTM>(s, a, n_seqs);
 }
 

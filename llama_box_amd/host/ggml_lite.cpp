@@ -694,8 +694,9 @@ static ggml_tensor * seq_gla(ggml_context * ctx, int kind, ggml_tensor * q, ggml
     const int64_t DK = q->ne[0] / n_head_k, DV = v->ne[0] / n_head, T = q->ne[1];
     LITE_ASSERT(n_head % n_head_k == 0 && q->ne[0] == DK * n_head_k && k->ne[0] == q->ne[0] && v->ne[0] == DV * n_head && k->ne[1] == T && v->ne[1] == T);
     // raw gates per token and their parameters: two per head (delta rule, matrix memory), one per (head, key channel) with A_log per head in front of the offsets
-    // (channel decay), or one per head with (A_log, dt_bias, D) (state space)
-    const int64_t n_gates = kind == 3 ? DK * n_head : kind == 4 ? n_head : 2 * n_head, n_par = kind == 3 ? n_head + DK * n_head : kind == 4 ? 3 * n_head : 2 * n_head;
+    // (channel decay), one per head with (A_log, dt_bias, D) (state space), or one per (head, key channel) with an offset each (linear attention)
+    const int64_t n_gates = kind == 3 || kind == 5 ? DK * n_head : kind == 4 ? n_head : 2 * n_head;
+    const int64_t n_par = kind == 3 ? n_head + DK * n_head : kind == 4 ? 3 * n_head : kind == 5 ? DK * n_head : 2 * n_head;
     LITE_ASSERT(gates->ne[0] == n_gates && gates->ne[1] == T && ggml_nelements(params) == n_par && ggml_nelements(tok) == T && info->ne[0] == 4);
     LITE_ASSERT(state->ne[0] == ggml_seq_state_size(kind, n_head, (int) DK, (int) DV));
     ggml_tensor * o = ggml_new_tensor_3d(ctx, GGML_TYPE_F32, DV, n_head, T);
@@ -724,6 +725,11 @@ struct ggml_tensor * ggml_seq_delta_channel(struct ggml_context * ctx, struct gg
 struct ggml_tensor * ggml_seq_ssd(struct ggml_context * ctx, struct ggml_tensor * c, struct ggml_tensor * b, struct ggml_tensor * x, struct ggml_tensor * dt_pre, struct ggml_tensor * a_dt_d,
                                   struct ggml_tensor * state, struct ggml_tensor * tok, struct ggml_tensor * info, int n_head, int n_group) {
     return seq_gla(ctx, 4, c, b, x, dt_pre, a_dt_d, state, tok, info, n_head, n_group, 0.0f);
+}
+struct ggml_tensor * ggml_seq_linear(struct ggml_context * ctx, struct ggml_tensor * q, struct ggml_tensor * k, struct ggml_tensor * v, struct ggml_tensor * a_pre, struct ggml_tensor * a_bias,
+                                     struct ggml_tensor * state, struct ggml_tensor * tok, struct ggml_tensor * info, int n_head, float tau) {
+    LITE_ASSERT(tau > 0.0f);
+    return seq_gla(ctx, 5, q, k, v, a_pre, a_bias, state, tok, info, n_head, n_head, tau);
 }
 struct ggml_tensor * ggml_seq_mlstm(struct ggml_context * ctx, struct ggml_tensor * q, struct ggml_tensor * k, struct ggml_tensor * v, struct ggml_tensor * if_pre, struct ggml_tensor * if_bias,
                                     struct ggml_tensor * state, struct ggml_tensor * tok, struct ggml_tensor * info, int n_head, float cap) {

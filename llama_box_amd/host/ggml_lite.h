@@ -161,12 +161,16 @@ struct ggml_tensor * ggml_seq_delta_channel(struct ggml_context * ctx, struct gg
    h / (H / G) of b and c: c, b [N G, T]; x [DV H, T]; dt_pre [H, T]; a_dt_d [3 H] (A_log, dt_bias, D) -> [DV, H, T] */
 struct ggml_tensor * ggml_seq_ssd(struct ggml_context * ctx, struct ggml_tensor * c, struct ggml_tensor * b, struct ggml_tensor * x, struct ggml_tensor * dt_pre, struct ggml_tensor * a_dt_d,
                                   struct ggml_tensor * state, struct ggml_tensor * tok, struct ggml_tensor * info, int n_head, int n_group);
+/* gated linear attention per head: S <- diag(w) S + k v^T with one decay per (head, key channel), w = sigmoid(a_pre + a_bias)^(1 / tau); o = S^T q dk^-1/2 (read after the
+   update): q, k [DK H, T]; v [DV H, T]; a_pre [DK H, T]; a_bias [DK H] -> [DV, H, T] */
+struct ggml_tensor * ggml_seq_linear(struct ggml_context * ctx, struct ggml_tensor * q, struct ggml_tensor * k, struct ggml_tensor * v, struct ggml_tensor * a_pre, struct ggml_tensor * a_bias,
+                                     struct ggml_tensor * state, struct ggml_tensor * tok, struct ggml_tensor * info, int n_head, float tau);
 /* matrix memory with exponential gates under a running maximum: i = cap tanh((i_pre + b_i) / cap), f = log sigmoid(cap tanh((f_pre + b_f) / cap)); m' = max(f + m, i);
    S <- e^(f + m - m') S + e^(i - m') k v^T, n likewise with k alone; o = S^T q / (max(|n . q|, e^(-m')) + 1e-6), q times dk^-1/2: q, k [DK H, T]; v [DV H, T];
    if_pre [2 H, T]; if_bias [2 H] -> [DV, H, T] */
 struct ggml_tensor * ggml_seq_mlstm(struct ggml_context * ctx, struct ggml_tensor * q, struct ggml_tensor * k, struct ggml_tensor * v, struct ggml_tensor * if_pre, struct ggml_tensor * if_bias,
                                     struct ggml_tensor * state, struct ggml_tensor * tok, struct ggml_tensor * info, int n_head, float cap);
-/* f32 values of state one slot of a recurrence holds (kind: 0 wkv6, 1 gated delta, 2 mlstm, 3 delta with channel decay, 4 state space) */
+/* f32 values of state one slot of a recurrence holds (kind: 0 wkv6, 1 gated delta, 2 mlstm, 3 delta with channel decay, 4 state space, 5 linear attention) */
 int64_t ggml_seq_state_size(int kind, int n_head, int dk, int dv);
 
 /* graphs */

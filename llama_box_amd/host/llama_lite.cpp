@@ -343,6 +343,10 @@ struct llm_layer {
     ggml_tensor *wqkv = nullptr, *bqkv = nullptr, *conv = nullptr, *wgates = nullptr, *gate_par = nullptr, *sub_norm = nullptr, *bo = nullptr, *attn_fb = nullptr;
     ggml_tensor *tm_taps = nullptr, *tm_rkvg = nullptr, *tm_w1 = nullptr, *tm_w2 = nullptr, *tm_w0 = nullptr, *tm_u = nullptr, *tm_norm = nullptr, *tm_out = nullptr;
     ggml_tensor *ffn_gate_up_exps = nullptr;
+    // ... a dense feed-forward's gate and up projections as one matrix; an expert that runs for every token (likewise) and the projection to its gate (one number per token)
+    ggml_tensor *ffn_gate_up = nullptr, *ffn_gate_up_shexp = nullptr, *ffn_down_shexp = nullptr, *ffn_gate_inp_shexp = nullptr;
+    // ... linear attention beside an attention: its own q, k, v as one projection (its output gate is in wg1, its decay in wa1, wa2 and gate_par)
+    ggml_tensor *wqkv_r = nullptr;
     // ... a query latent in front of the query heads (down projection, its norm); the weights of a per-head norm on queries and keys (one row shared by the heads)
     ggml_tensor *wdq = nullptr, *dq_norm = nullptr, *q_norm = nullptr, *k_norm = nullptr;
     // ... a delta rule with one decay per key channel beside an attention (its own q, k, v as one projection in wqkv / conv; beta; the decay and the output gate through
@@ -361,7 +365,7 @@ struct llm_layer {
 // one layer of a model whose config lists its layers one by one (sizes and constants may differ from layer to layer)
 enum llm_mlp_kind { LLM_MLP_NONE = 0, LLM_MLP_DENSE = 1, LLM_MLP_MOE = 2 };
 // (from LLM_MIX_MLSTM on: mixers that keep state per sequence and bring their own output projection)
-enum llm_mixer_kind { LLM_MIX_ATTN = 0, LLM_MIX_LATENT = 1, LLM_MIX_MLSTM = 2, LLM_MIX_DELTA = 3, LLM_MIX_SIGMOID_WKV = 4, LLM_MIX_SSD = 5, LLM_MIX_ATTN_DELTA = 6 };
+enum llm_mixer_kind { LLM_MIX_ATTN = 0, LLM_MIX_LATENT = 1, LLM_MIX_MLSTM = 2, LLM_MIX_DELTA = 3, LLM_MIX_SIGMOID_WKV = 4, LLM_MIX_SSD = 5, LLM_MIX_ATTN_DELTA = 6, LLM_MIX_ATTN_LINEAR = 7 };
 struct llm_layer_cfg {
     int n_head = 0, n_head_kv = 0, dk = 0, dv = 0;  // query heads, key/value heads, per-head query/key size, per-head value size
     int rot_dims = 0;                               // leading dims of every head that are rotated, as neighbouring pairs
@@ -404,7 +408,7 @@ struct llm_layer_cfg {
     bool ffn_relu_sq = false;                       // dense feed-forward W_down relu(W_up h)^2
     bool qk_norm = false;                           // queries and keys are RMS-normed per head with a weight row shared by the heads
     int q_rank = 0;                                 // > 0: queries come through a normed latent of this size
-    int kv_from = -1;                               // >= 0: a latent-attention layer without a down projection of its own, reading that layer's cache rows
+    int kv_from = -1;                               // >= 0: an attention layer without keys and values (latents) of its own, reading that layer's cache rows
     int ssm_state = 0, ssm_groups = 1, ssm_norm_groups = 1;  // state-space mixer (LLM_MIX_SSD): state size per head, groups of (B, C), parts of the gated norm; n_head x dv = inner
     int r_head = 0, r_head_kv = 0, r_dk = 0, r_dv = 0, r_rank = 0;  // the delta rule beside an attention (LLM_MIX_ATTN_DELTA): heads, key heads, sizes, inner size of decay / gate
     int side_dim = 0;                               // > 0: the per-layer token input of this many entries
@@ -414,7 +418,18 @@ struct llm_layer_cfg {
     // mixture of experts: scores are sigmoids; the choice goes by score + correction (ffn_corr), the weights are the chosen scores divided by their sum (+ 1e-20); experts are
     // W_down (g sigmoid(1.702 g) (u + 1)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit)
     bool moe_sigmoid = false;
-    float moe_limit = 0.0f;
+    float moe_limit = 0.0f;                         // 0: the activation is silu(W_gate h) * W_up h, without limits
+    bool moe_raw = false;                           // ... the weights are the chosen scores as they are
+    bool moe_scale_in = false;                      // ... and multiply an expert's INPUT: the sum is of expert(w h)
+    int n_ff_shared = 0;                            // > 0: one more expert runs for every token, its output times sigmoid(W_sg h) (one number per token)
+    bool no_pre_norm = false;                       // the sublayers read the stream itself (their outputs are normed: attn_post_norm, ffn_post_norm)
+    bool ffn_silu_gated = false;                    // dense feed-forward W_down (silu(W_gate h) * W_up h)
+    bool qkv_first = false;                         // the projections precede the per-head steps in the graph's order (which the backend then runs as one launch)
+    bool rot_table = false;                         // rotation by a table of frequencies (rope_freq), cos and sin times rope_magnitude
+    float band_factor = 0.0f, band_low = 1.0f, band_high = 1.0f, band_orig = 0.0f;  // band_factor > 0: frequencies divided by it, kept or blended by their wavelength
+    bool qk_unit = false;                           // BEHIND the rotation every head's query and key is divided by its root mean square (no weight)
+    bool v_is_k = false;                            // no value projection: the values are the keys as they leave the convolution, before norm and rotation
+    float r_tau = 1.0f;                             // linear attention beside an attention (LLM_MIX_ATTN_LINEAR; r_head, r_dk, r_dv, r_rank): decay = sigmoid(.)^(1 / tau)
 };
 // what a layer's positions may see: one attention mask per distinct rule of a model
 struct llm_mask_rule {
@@ -469,6 +484,7 @@ struct llm_model {
     std::vector<llm_mask_rule> mask_rules;  // the distinct visibility rules of the layers ({} = plain causal): one attention mask each
     std::vector<llm_run> runs;           // the order in which layers execute (one entry per layer unless a range repeats)
     float embd_scale = 1.0f, logit_scale = 1.0f;
+    float logit_softcap = 0.0f;          // > 0: logits <- cap tanh(logits / cap)
     // a hashed bigram embedding added to the token embedding: row (prev * mul_prev + cur * mul_cur) mod buckets, row `buckets` for a sequence's first token
     ggml_tensor * bigram = nullptr;
     int bg_buckets = 0, bg_mul_prev = 0, bg_mul_cur = 0;
@@ -1221,7 +1237,8 @@ static std::vector<dir_tensor> rarelorn_plan(const llm_model * m) {
     return plan;
 }
 
-// frequency of every rotation pair, base^(-2 i / dims), blended with its 1 / factor over the ramp between the two correction dims (YaRN); computed in f64
+// frequency of every rotation pair, base^(-2 i / dims), optionally blended with its 1 / factor over the ramp between the two correction dims (YaRN), or by its wavelength: kept below
+// original / high, divided above original / low, blended in original / wavelength between the two (Llama 3.1); computed in f64
 static std::vector<float> rope_frequencies(const llm_layer_cfg & c) {
     const int dims = c.rot_dims, half = dims / 2;
     std::vector<float> f((size_t) half);
@@ -1237,6 +1254,13 @@ static std::vector<float> rope_frequencies(const llm_layer_cfg & c) {
         if (c.yarn_factor > 0.0f) {
             const double ramp = std::min(1.0, std::max(0.0, (i - lo) / std::max(hi - lo, 0.001)));
             v = fi / c.yarn_factor * ramp + fi * (1.0 - ramp);
+        } else if (c.band_factor > 0.0f) {
+            const double len = 2.0 * M_PI / fi, orig = c.band_orig, low = c.band_low, high = c.band_high;
+            if (len > orig / low) v = fi / c.band_factor;
+            else if (len >= orig / high) {
+                const double s = (orig / len - low) / (high - low);
+                v = (1.0 - s) * fi / c.band_factor + s * fi;
+            }
         }
         f[(size_t) i] = (float) v;
     }
@@ -1590,7 +1614,7 @@ static bool parse_pisulorn_config(const json_value & cfg, llm_model * m, std::st
         if (type->str == "attention") {
             c.mixer = LLM_MIX_ATTN;
             c.scale = (float) num(mx, "scale", nullptr, 1.0 / sqrt((double) c.dk));
-            c.qk_norm = c.dist_linear = true;
+            c.qk_norm = c.dist_linear = c.qkv_first = true;
             llm_mask_rule rule;
             rule.distance = true;
             if (const json_value * mk = sub(mx, "mask")) {
@@ -1709,6 +1733,235 @@ static std::vector<dir_tensor> pisulorn_plan(const llm_model * m) {
     return plan;
 }
 
+// Nidudra: layers whose norms stand on the sublayers' OUTPUTS only (x <- x + norm(mixer(x)), x <- x + norm(ff(x))).  Mixers: grouped-query attention over a window with kept first tokens
+// (per-head normed queries and keys, no positions, a gate per value entry, optionally an earlier layer's cache); grouped-query attention with rotation by banded frequencies, queries
+// and keys made unit behind it, a learned sink and a gate per head; attention whose values are its convolved keys beside gated linear attention.  Feed-forward: silu-gated, dense or
+// experts chosen by sigmoid scores that multiply their input, beside one that runs for every token.  Logits are soft-capped.
+static bool parse_nidudra_rotation(const json_value * mx, llm_layer_cfg & c, const std::string & lname, std::string & err) {
+    const json_value * r = mx->get("rot");
+    if (!r || r->kind != json_value::OBJ) return true;
+    auto num = [&](const json_value * o, const char * k, double d) { const json_value * x = o->get(k); return x ? x->number(d) : d; };
+    c.rot_dims = (int) num(r, "dims", 0);
+    c.rot_base = (float) num(r, "base", 10000.0);
+    c.rot_half = c.rot_table = true;
+    if (c.rot_dims < 0 || c.rot_dims > c.dk || (c.rot_dims & 1) || !(c.rot_base > 0.0f)) { err = lname + ": inconsistent rotation"; return false; }
+    const json_value * sc = r->get("scaling");
+    if (!sc || sc->kind != json_value::OBJ) return true;
+    const double factor = num(sc, "factor", 0.0), orig = num(sc, "original", 0.0);
+    if (!(factor > 0.0) || !(orig > 0.0)) { err = lname + ": inconsistent frequency scaling"; return false; }
+    if (sc->get("fast") || sc->get("slow")) {
+        c.yarn_factor = (float) factor;
+        c.yarn_orig = (float) orig;
+        c.yarn_fast = (float) num(sc, "fast", 32.0);
+        c.yarn_slow = (float) num(sc, "slow", 1.0);
+        if (!(c.yarn_fast > 0.0f) || !(c.yarn_slow > 0.0f)) { err = lname + ": inconsistent frequency scaling"; return false; }
+    } else {
+        c.band_factor = (float) factor;
+        c.band_orig = (float) orig;
+        c.band_low = (float) num(sc, "low", 1.0);
+        c.band_high = (float) num(sc, "high", 4.0);
+        if (!(c.band_low > 0.0f) || !(c.band_high > c.band_low)) { err = lname + ": inconsistent frequency scaling"; return false; }
+    }
+    return true;
+}
+static bool parse_nidudra_config(const json_value & cfg, const st_file * file, llm_model * m, std::string & err) {
+    llm_hparams & hp = m->hp;
+    snprintf(hp.arch, sizeof(hp.arch), "nidudra");
+    const json_value * layers = cfg.get("layers");
+    if (!layers || layers->kind != json_value::ARR || layers->arr.empty()) { err = "config: no layers"; return false; }
+    const json_value * v;
+    hp.n_embd = (v = cfg.get("width")) ? (int) v->number(0) : 0;
+    hp.n_vocab = (v = cfg.get("vocab")) ? (int) v->number(0) : 0;
+    hp.rms_eps = (v = cfg.path("norm", "eps")) ? (float) v->number(1e-5) : 1e-5f;
+    m->logit_softcap = (v = cfg.get("logit_softcap")) ? (float) v->number(0.0) : 0.0f;
+    hp.n_layer = (int) layers->arr.size();
+    hp.n_ctx_train = 1 << 20;
+    if (hp.n_embd <= 0 || hp.n_vocab <= 0) { err = "config: width / vocab missing"; return false; }
+    if (m->logit_softcap < 0.0f) { err = "config: logit_softcap must not be negative"; return false; }
+    auto num = [&](const json_value * o, const char * k0, const char * k1, double d) { const json_value * x = o->path(k0, k1); return x ? x->number(d) : d; };
+    auto sub = [&](const json_value * o, const char * k) { const json_value * x = o->get(k); return x && x->kind == json_value::OBJ ? x : nullptr; };
+    m->lcfg.resize((size_t) hp.n_layer);
+    m->has_attn = true;  // (every mixer of the design attends over the cell cache)
+    m->has_seq_state = false;
+    m->hist_rows = 0;
+    for (int il = 0; il < hp.n_layer; ++il) {
+        const json_value & L = layers->arr[(size_t) il];
+        llm_layer_cfg & c = m->lcfg[(size_t) il];
+        const std::string lname = "config: layer " + std::to_string(il);
+        const json_value * type = L.get("type");
+        const json_value * mx = sub(&L, "mixer");
+        if (!type || type->kind != json_value::STR || !mx) { err = lname + ": no mixer"; return false; }
+        c.rms = c.no_pre_norm = c.qkv_first = true;
+        const bool parallel = type->str == "parallel";
+        const json_value * at = parallel ? sub(mx, "left") : mx, * rt = parallel ? sub(mx, "right") : nullptr;
+        if (!at || (parallel && !rt)) { err = lname + ": a parallel mixer needs left and right"; return false; }
+        c.n_head = (int) num(at, "heads", nullptr, 0);
+        c.n_head_kv = (int) num(at, "kv_heads", nullptr, c.n_head);
+        c.dk = (int) num(at, "dim", nullptr, 0);
+        c.dv = (int) num(at, "vdim", nullptr, c.dk);
+        if (c.n_head <= 0 || c.n_head_kv <= 0 || c.n_head % c.n_head_kv || c.dk <= 0 || c.dv <= 0) { err = lname + ": inconsistent head sizes"; return false; }
+        c.scale = (float) num(at, "scale", nullptr, 1.0 / sqrt((double) c.dk));
+        llm_mask_rule rule;
+        if (type->str == "attention") {
+            c.mixer = LLM_MIX_ATTN;
+            c.qk_norm = c.out_gate = true;
+            if (const json_value * mk = sub(mx, "mask")) {
+                rule.window = c.window = (int) num(mk, "size", nullptr, 0);
+                rule.keep_first = c.keep_first = (int) num(mk, "keep_first", nullptr, 0);
+                if (c.window < 1 || c.keep_first < 0) { err = lname + ": a window of less than one token"; return false; }
+            }
+            const json_value * kf = mx->get("kv_from");
+            if (kf && kf->kind != json_value::NUL) {
+                c.kv_from = (int) kf->number(-1);
+                const llm_layer_cfg * o = c.kv_from >= 0 && c.kv_from < il ? &m->lcfg[(size_t) c.kv_from] : nullptr;
+                if (!o || o->mixer != LLM_MIX_ATTN || !o->qk_norm || o->kv_from >= 0 || o->n_head_kv != c.n_head_kv || o->dk != c.dk || o->dv != c.dv) {
+                    err = lname + ": kv_from names no earlier attention layer with keys and values of its own and the same head sizes";
+                    return false;
+                }
+            }
+        } else if (type->str == "attention_2") {
+            c.mixer = LLM_MIX_ATTN;
+            c.qk_unit = c.sink = c.sink_learned = c.out_gate = c.gate_heads = true;
+            if (!parse_nidudra_rotation(at, c, lname, err)) return false;
+        } else if (parallel) {
+            c.mixer = LLM_MIX_ATTN_LINEAR;
+            c.v_is_k = c.qkv_bias = c.qk_norm = true;
+            c.conv_taps = (int) num(at, "conv", nullptr, 1);
+            c.left_scale = c.right_scale = 0.5f;
+            if (!parse_nidudra_rotation(at, c, lname, err)) return false;
+            c.r_head = c.r_head_kv = (int) num(rt, "heads", nullptr, 0);
+            c.r_dk = (int) num(rt, "dim", nullptr, 0);
+            c.r_dv = (int) num(rt, "vdim", nullptr, c.r_dk);
+            c.r_tau = (float) num(rt, "tau", nullptr, 16.0);
+            c.r_rank = (int) num(rt, "rank", nullptr, 16);  // (a checkpoint's a1 gives it)
+            if (file) {
+                const st_tensor * a1 = file->find("l" + std::to_string(il) + ".mix.right.a1");
+                if (!a1 || a1->shape.size() != 2) { err = lname + ": no right.a1 in the checkpoint"; return false; }
+                c.r_rank = (int) a1->shape[0];
+            }
+            if (c.dv != c.dk) { err = lname + ": values that are the keys have their size"; return false; }
+            if (c.r_head <= 0 || c.r_dk <= 0 || c.r_dk > 256 || c.r_dv <= 0 || c.r_rank <= 0 || !(c.r_tau > 0.0f) || c.conv_taps < 1 || c.conv_taps > 16) {
+                err = lname + ": inconsistent parallel-mixer sizes";
+                return false;
+            }
+            m->has_seq_state = true;
+            m->hist_rows = std::max(m->hist_rows, c.conv_taps - 1);
+        } else { err = lname + ": unknown mixer type"; return false; }
+        c.mask_id = mask_rule_id(m, rule);
+        m->max_embd_k = std::max(m->max_embd_k, c.n_head_kv * c.dk);
+        m->max_embd_v = std::max(m->max_embd_v, c.n_head_kv * c.dv);
+        if (const json_value * ml = sub(&L, "mlp")) {
+            const json_value * kind = ml->get("kind");
+            if (kind && kind->kind == json_value::STR && kind->str == "dense") {
+                c.mlp = LLM_MLP_DENSE;
+                c.ffn_silu_gated = true;
+                c.n_ff = (int) num(ml, "ff", nullptr, 0);
+            } else if (kind && kind->kind == json_value::STR && kind->str == "moe") {
+                c.mlp = LLM_MLP_MOE;
+                c.moe_sigmoid = c.moe_raw = c.moe_scale_in = true;
+                c.n_ff = (int) num(ml, "expert", "ff", 0);
+                c.n_expert = (int) num(ml, "router", "experts", 0);
+                c.n_top = (int) num(ml, "router", "top", 0);
+                if (c.n_expert <= 0 || c.n_top <= 0 || c.n_top > c.n_expert) { err = lname + ": inconsistent experts"; return false; }
+                if (const json_value * sh = sub(ml, "shared")) {
+                    c.n_ff_shared = (int) num(sh, "ff", nullptr, 0);
+                    if (c.n_ff_shared <= 0) { err = lname + ": inconsistent shared expert"; return false; }
+                }
+            } else { err = lname + ": unknown mlp kind"; return false; }
+            if (c.n_ff <= 0) { err = lname + ": ff missing"; return false; }
+        }
+    }
+    hp.n_head = m->lcfg[0].n_head; hp.n_head_kv = m->lcfg[0].n_head_kv; hp.n_embd_head = m->lcfg[0].dk; hp.n_ff = m->lcfg[0].n_ff;
+    hp.rope_freq_base = m->lcfg[0].rot_base;
+    make_runs(m, false);
+    return true;
+}
+
+static std::vector<dir_tensor> nidudra_plan(const llm_model * m) {
+    const llm_hparams & hp = m->hp;
+    const ggml_type wt = m->wtype;
+    const int64_t E = hp.n_embd;
+    std::vector<dir_tensor> plan;
+    auto add = [&](const std::string & name, ggml_type t, int64_t n0, int64_t n1, int64_t n2, std::vector<std::string> src, float gain) -> dir_tensor & {
+        dir_tensor d;
+        d.name = name; d.type = t; d.ne[0] = n0; d.ne[1] = n1; d.ne[2] = n2; d.src = std::move(src); d.synth_gain = gain;
+        plan.push_back(std::move(d));
+        return plan.back();
+    };
+    auto vec = [&](const std::string & name, int64_t n, std::vector<std::string> src, float lo, float hi) {
+        dir_tensor & t = add(name, GGML_TYPE_F32, n, 1, 1, std::move(src), 0.0f);
+        t.synth_lo = lo; t.synth_hi = hi;
+    };
+    add("token_embd.weight", wt, E, hp.n_vocab, 1, {"embed"}, sqrtf((float) E));
+    for (int il = 0; il < hp.n_layer; ++il) {
+        const llm_layer_cfg & c = m->lcfg[(size_t) il];
+        const std::string p = "blk." + std::to_string(il) + ".", q = "l" + std::to_string(il) + ".", x = q + "mix.";
+        const int64_t H = c.n_head, G = c.n_head_kv;
+        const bool linear = c.mixer == LLM_MIX_ATTN_LINEAR;
+        const std::string l = linear ? x + "left." : x;
+        vec(p + "attn_post_norm.weight", E, {q + "norm1"}, 0.7f, 1.4f);
+        if (linear) {
+            const int64_t C = (H + G) * c.dk;
+            add(p + "attn_qkv.weight", wt, E, C, 1, {l + "q", l + "k"}, 1.5f);
+            add(p + "attn_qkv.bias", GGML_TYPE_F32, C, 1, 1, {l + "q.b", l + "k.b"}, 0.3f * sqrtf((float) C));
+            add(p + "ssm_conv1d.weight", GGML_TYPE_F32, c.conv_taps, C, 1, {l + "q.conv", l + "k.conv"}, 1.0f);
+        } else {
+            add(p + "attn_q.weight", wt, E, H * c.dk, 1, {l + "q"}, 1.5f);
+            if (c.kv_from < 0) {
+                add(p + "attn_k.weight", wt, E, G * c.dk, 1, {l + "k"}, 1.5f);
+                add(p + "attn_v.weight", wt, E, G * c.dv, 1, {l + "v"}, 1.0f);
+            }
+            add(p + "attn_gate.weight", wt, E, c.gate_heads ? H : H * c.dv, 1, {l + "g"}, 1.0f);
+        }
+        if (c.qk_norm) {
+            vec(p + "attn_q_norm.weight", c.dk, {l + "q.norm"}, 0.7f, 1.4f);
+            if (c.kv_from < 0) vec(p + "attn_k_norm.weight", c.dk, {l + "k.norm"}, 0.7f, 1.4f);
+        }
+        if (c.sink_learned) add(p + "attn_sink.weight", GGML_TYPE_F32, H, 1, 1, {l + "sink"}, sqrtf((float) H));
+        if (c.rot_dims > 0) add(p + "rope_freq.weight", GGML_TYPE_F32, c.rot_dims / 2, 1, 1, {}, 0.0f).values = rope_frequencies(c);
+        add(p + "attn_output.weight", wt, H * c.dv, E, 1, {l + "o"}, 1.0f);
+        if (linear) {
+            const std::string r = x + "right.";
+            const int64_t RH = c.r_head, KC = RH * c.r_dk, VC = RH * c.r_dv;
+            vec(p + "mix_left_norm.weight", E, {l + "out"}, 0.7f, 1.4f);
+            add(p + "linear_qkv.weight", wt, E, 2 * KC + VC, 1, {r + "q", r + "k", r + "v"}, 1.0f);
+            add(p + "linear_gate.weight", wt, E, VC, 1, {r + "g"}, 1.0f);
+            add(p + "linear_a1.weight", wt, E, c.r_rank, 1, {r + "a1"}, 1.0f);
+            add(p + "linear_a2.weight", wt, c.r_rank, KC, 1, {r + "a2"}, 1.5f);
+            vec(p + "linear_a2.bias", KC, {r + "a2.b"}, -1.0f, 2.0f);
+            vec(p + "attn_sub_norm.weight", c.r_dv, {r + "norm"}, 0.7f, 1.4f);
+            add(p + "linear_output.weight", wt, VC, E, 1, {r + "o"}, 1.0f);
+            vec(p + "mix_right_norm.weight", E, {r + "out"}, 0.7f, 1.4f);
+        }
+        if (c.mlp == LLM_MLP_NONE) continue;
+        const std::string f = q + "mlp.";
+        vec(p + "ffn_post_norm.weight", E, {q + "norm2"}, 0.7f, 1.4f);
+        if (c.mlp == LLM_MLP_DENSE) {
+            add(p + "ffn_gate_up.weight", wt, E, 2 * c.n_ff, 1, {f + "gate", f + "up"}, 1.4f);
+            add(p + "ffn_down.weight", wt, c.n_ff, E, 1, {f + "down"}, 1.0f);
+            continue;
+        }
+        std::vector<std::string> gu, downs;
+        for (int e = 0; e < c.n_expert; ++e) {
+            const std::string pe = f + "e" + std::to_string(e) + ".";
+            gu.push_back(pe + "gate");
+            gu.push_back(pe + "up");
+            downs.push_back(pe + "down");
+        }
+        add(p + "ffn_gate_inp.weight", GGML_TYPE_F32, E, c.n_expert, 1, {f + "router"}, 3.0f);  // router logits are 32-bit in every mode
+        add(p + "ffn_gate_up_exps.weight", wt, E, 2 * c.n_ff, c.n_expert, gu, 1.4f);            // per expert: its gate rows, then its up rows
+        add(p + "ffn_down_exps.weight", wt, c.n_ff, E, c.n_expert, downs, 1.0f);
+        if (c.n_ff_shared > 0) {
+            add(p + "ffn_gate_up_shexp.weight", wt, E, 2 * c.n_ff_shared, 1, {f + "shared.gate", f + "shared.up"}, 1.4f);
+            add(p + "ffn_down_shexp.weight", wt, c.n_ff_shared, E, 1, {f + "shared.down"}, 1.0f);
+            add(p + "ffn_gate_inp_shexp.weight", wt, E, 1, 1, {f + "shared.sg"}, 2.0f);
+        }
+    }
+    vec("output_norm.weight", E, {"final.norm"}, 0.7f, 1.4f);
+    add("output.weight", wt, E, hp.n_vocab, 1, {"head"}, 1.0f);
+    return plan;
+}
+
 // values of one checkpoint tensor (bf16 / f32 / f16 in the file) as `type` (bf16 or f32) into dst
 static bool convert_values(const st_tensor & t, ggml_type type, uint8_t * dst) {
     const int64_t n = t.numel();
@@ -1753,6 +2006,9 @@ static llm_model * model_from_config(const json_value & cfg, const st_file * fil
     } else if (arch->str == "Pisulorn") {
         if (!parse_pisulorn_config(cfg, m, err)) { fprintf(stderr, "llm_model_load_dir: %s\n", err.c_str()); delete m; return nullptr; }
         plan = pisulorn_plan(m);
+    } else if (arch->str == "Nidudra") {
+        if (!parse_nidudra_config(cfg, file, m, err)) { fprintf(stderr, "llm_model_load_dir: %s\n", err.c_str()); delete m; return nullptr; }
+        plan = nidudra_plan(m);
     } else {
         fprintf(stderr, "llm_model_load_dir: unknown architecture \"%s\"\n", arch->str.c_str());
         delete m;
@@ -1936,13 +2192,18 @@ static llm_model * model_from_config(const json_value & cfg, const st_file * fil
             L.hc_in[k] = g((f + "in.weight").c_str()); L.hc_out[k] = g((f + "out.weight").c_str()); L.hc_mix[k] = g((f + "mix.weight").c_str());
         }
         L.attn_slopes = g("attn_slopes.weight"); L.ffn_corr = g("ffn_choice.bias");
+        L.ffn_gate_up = g("ffn_gate_up.weight"); L.ffn_gate_up_shexp = g("ffn_gate_up_shexp.weight"); L.ffn_down_shexp = g("ffn_down_shexp.weight");
+        L.ffn_gate_inp_shexp = g("ffn_gate_inp_shexp.weight"); L.wqkv_r = g("linear_qkv.weight");
+        if (L.wqkv_r) {  // (linear attention: its gate, decay and output projection are where the delta rule beside an attention keeps its own)
+            L.wg1 = g("linear_gate.weight"); L.wa1 = g("linear_a1.weight"); L.wa2 = g("linear_a2.weight"); L.gate_par = g("linear_a2.bias"); L.wo_r = g("linear_output.weight");
+        }
         L.wdkv = g("attn_kv_a.weight"); L.dkv_norm = g("attn_kv_a_norm.weight"); L.wuk_t = g("attn_k_b_t.weight"); L.wuv = g("attn_v_b.weight"); L.rope_freq = g("rope_freq.weight");
         for (ggml_tensor * t : {L.attn_norm, L.attn_post_norm, L.wq, L.wk, L.wv, L.attn_gate, L.wo, L.ffn_norm, L.ffn_post_norm, L.ffn_up, L.ffn_down, L.ffn_gate_inp,
                                 L.attn_sink, L.attn_r12, L.shift, L.ffn_gate, L.ffn_gate_b, L.ffn_up_b, L.ffn_down_b, L.wdkv, L.dkv_norm, L.wuk_t, L.wuv, L.rope_freq,
                                 L.wqkv, L.bqkv, L.conv, L.wgates, L.gate_par, L.sub_norm, L.bo, L.attn_fb, L.tm_taps, L.tm_rkvg, L.tm_w1, L.tm_w2, L.tm_w0, L.tm_u, L.tm_norm, L.tm_out,
                                 L.bq, L.bk, L.bv, L.q_norm, L.k_norm, L.wdq, L.dq_norm, L.wbeta, L.wa1, L.wa2, L.wg1, L.wg2, L.wo_r, L.left_norm, L.right_norm, L.ssm_in_z, L.ssm_in_xbc,
                                 L.ssm_in_dt, L.conv_b, L.side_gate, L.side_proj, L.side_norm, L.hc_in[0], L.hc_in[1], L.hc_out[0], L.hc_out[1], L.hc_mix[0], L.hc_mix[1],
-                                L.attn_slopes, L.ffn_corr})
+                                L.attn_slopes, L.ffn_corr, L.ffn_gate_up, L.ffn_gate_up_shexp, L.ffn_down_shexp, L.ffn_gate_inp_shexp, L.wqkv_r})
             if (t) sbytes += ggml_nbytes(t) * (uint64_t) std::max(1, times_run[(size_t) il]);  // (a layer of a repeated range is streamed once per run)
         if (L.side_embd) sbytes += ggml_row_size(L.side_embd->type, L.side_embd->ne[0]);  // (one row of the layer's part of the side table)
         if (c.mlp == LLM_MLP_MOE) sbytes += (ggml_nbytes(L.ffn_gate_up_exps ? L.ffn_gate_up_exps : L.ffn_up_exps) + ggml_nbytes(L.ffn_down_exps)) / (uint64_t) c.n_expert * (uint64_t) c.n_top *
@@ -2359,6 +2620,17 @@ static ggml_tensor * build_token_shift(llm_context * c, ggml_context * ctx, ggml
     return out;
 }
 
+// the run whose cache rows a layer attends over: its own, or — without keys and values of its own — that of the layer it names, in the same pass
+static int cache_run_of(const llm_context * c, const llm_layer_cfg & lc, int run) {
+    if (lc.kv_from < 0) return run;
+    const llm_model * m = c->model;
+    int at = -1;
+    for (int r = 0; r < run; ++r)
+        if (m->runs[(size_t) r].il == lc.kv_from && m->runs[(size_t) r].pass == m->runs[(size_t) run].pass) at = r;
+    LLM_ASSERT(at >= 0 && c->k_l[(size_t) at]);
+    return at;
+}
+
 // grouped-query attention of one layer run over its cache; returns the heads' outputs [dv * H, T] (gated), before the output projection
 static ggml_tensor * build_mixer_attention(llm_context * c, ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * cur, int il, int run,
                                            int n_tokens, int n_kv, seg_io & io, ggml_tensor ** v_first) {
@@ -2366,47 +2638,77 @@ static ggml_tensor * build_mixer_attention(llm_context * c, ggml_context * ctx, 
     const llm_hparams & hp = m->hp;
     const int64_t H = lc.n_head, G = lc.n_head_kv, DK = lc.dk, DV = lc.dv;
     (void) il;
-    ggml_tensor * Qcur = named(ggml_mul_mat(ctx, L.wq, cur), "Qcur", run);
-    ggml_tensor * Kcur = named(ggml_mul_mat(ctx, L.wk, cur), "Kcur", run);
-    ggml_tensor * Vcur = named(ggml_mul_mat(ctx, L.wv, cur), "Vcur", run);
-    ggml_tensor * gate = lc.out_gate ? named(ggml_mul_mat(ctx, L.attn_gate, cur), "attn_gate", run) : nullptr;
-    if (L.bq) Qcur = named(ggml_add(ctx, Qcur, L.bq), "Qcur_b", run);
-    if (L.bk) Kcur = named(ggml_add(ctx, Kcur, L.bk), "Kcur_b", run);
-    if (L.bv) Vcur = named(ggml_add(ctx, Vcur, L.bv), "Vcur_b", run);
-    if (lc.dist_linear) {  // (the three products of the one input follow one another; the per-head norms and the cache stores then do too, which the backend runs as one launch)
-        ggml_build_forward_expand(gf, Qcur);
+    const bool own_kv = lc.kv_from < 0;
+    ggml_tensor * Qcur = nullptr, * Kcur = nullptr, * Vcur = nullptr;
+    ggml_tensor * gate = nullptr;
+    if (lc.v_is_k) {  // queries and keys as ONE projection (+ bias) through a short convolution; the convolved keys are the values too
+        ggml_tensor * qk_pre = named(ggml_mul_mat(ctx, L.wqkv, cur), "qk_proj", run);
+        ggml_build_forward_expand(gf, qk_pre);
+        if (L.bqkv) qk_pre = named(ggml_add(ctx, qk_pre, L.bqkv), "qk_pre", run);
+        ggml_tensor * qk = named(ggml_seq_conv(ctx, qk_pre, L.conv, c->conv_state[(size_t) run], io.seq_hist, /*act=*/0), "qk_conv", run);
+        ggml_build_forward_expand(gf, qk);  // (the state is read before it is overwritten)
+        if (lc.conv_taps > 1) ggml_build_forward_expand(gf, named(ggml_seq_conv_store(ctx, c->conv_state[(size_t) run], qk_pre, io.seq_upd, io.seq_info, lc.conv_taps), "conv_store", run));
+        qk = ggml_reshape_2d(ctx, qk, qk->ne[0], n_tokens);
+        Qcur = ggml_view_3d(ctx, qk, DK, H, n_tokens, (size_t) DK * sizeof(float), qk->nb[1], 0);
+        Kcur = ggml_view_3d(ctx, qk, DK, G, n_tokens, (size_t) DK * sizeof(float), qk->nb[1], (size_t) (H * DK) * sizeof(float));
+        Vcur = ggml_view_2d(ctx, qk, G * DV, n_tokens, qk->nb[1], (size_t) (H * DK) * sizeof(float));
+    } else {
+        Qcur = named(ggml_mul_mat(ctx, L.wq, cur), "Qcur", run);
+        if (own_kv) {
+            Kcur = named(ggml_mul_mat(ctx, L.wk, cur), "Kcur", run);
+            Vcur = named(ggml_mul_mat(ctx, L.wv, cur), "Vcur", run);
+        }
+        gate = lc.out_gate ? named(ggml_mul_mat(ctx, L.attn_gate, cur), "attn_gate", run) : nullptr;
+        if (L.bq) Qcur = named(ggml_add(ctx, Qcur, L.bq), "Qcur_b", run);
+        if (L.bk) Kcur = named(ggml_add(ctx, Kcur, L.bk), "Kcur_b", run);
+        if (L.bv) Vcur = named(ggml_add(ctx, Vcur, L.bv), "Vcur_b", run);
+        if (lc.qkv_first) {  // (the products of the one input follow one another; the per-head steps and the cache stores then do too, which the backend runs as one launch)
+            ggml_build_forward_expand(gf, Qcur);
+            if (own_kv) {
+                ggml_build_forward_expand(gf, Kcur);
+                ggml_build_forward_expand(gf, Vcur);
+            }
+            if (gate && lc.no_pre_norm) ggml_build_forward_expand(gf, gate);
+        }
+        Qcur = ggml_reshape_3d(ctx, Qcur, DK, H, n_tokens);
+        if (own_kv) Kcur = ggml_reshape_3d(ctx, Kcur, DK, G, n_tokens);
+    }
+    // what a head's query and key go through before the scores
+    auto head_steps = [&](ggml_tensor * x, ggml_tensor * w, bool query, const std::string & n) {
+        if (lc.qk_norm) x = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, x, hp.rms_eps), (n + "_rnorm").c_str(), run), w), (n + "_normed").c_str(), run);  // divided by the root mean square, times a weight row shared by the heads
+        if (query && lc.q_temp_id >= 0) x = named(ggml_mul(ctx, x, io.q_temps[(size_t) lc.q_temp_id]), (n + "_temp").c_str(), run);
+        if (lc.rot_dims > 0) {  // pairs of the leading rot_dims entries, neighbours (2i, 2i + 1) or (i, i + dims / 2); the rest of the head passes through
+            x = named(ggml_rope_ext(ctx, x, io.pos, lc.rot_table ? L.rope_freq : nullptr, lc.rot_dims, lc.rot_half ? GGML_ROPE_TYPE_NEOX : 0, hp.n_ctx_train, lc.rot_base, 1.0f, 0.0f,
+                                    lc.rot_table ? rope_magnitude(lc) : 1.0f, 32.0f, 1.0f), (n + "_rope").c_str(), run);
+            if (lc.rot_table) ggml_rope_set_freq_table(x);
+            else ggml_rope_set_exact_freq(x);  // angle = pos * base^(-2 i / dims) with the frequency itself rounded once (not ggml's running product)
+        }
+        if (lc.qk_unit) x = named(ggml_rms_norm(ctx, x, hp.rms_eps), (n + "_unit").c_str(), run);
+        return x;
+    };
+    Qcur = head_steps(Qcur, L.q_norm, true, "Qcur");
+    if (lc.v_is_k && !lc.qk_norm && lc.rot_dims <= 0 && !lc.qk_unit) Qcur = named(ggml_cont(ctx, Qcur), "Qcur_cont", run);
+    ggml_build_forward_expand(gf, Qcur);
+    const int cache_run = cache_run_of(c, lc, run);
+    ggml_tensor * k_cache = c->k_l[(size_t) cache_run];
+    ggml_tensor * v_cache = c->v_l[(size_t) cache_run];
+    if (own_kv) {
+        Kcur = head_steps(Kcur, L.k_norm, false, "Kcur");
+        if (lc.v_is_k && !lc.qk_norm && lc.rot_dims <= 0 && !lc.qk_unit) Kcur = named(ggml_cont(ctx, Kcur), "Kcur_cont", run);
+        if (lc.v_unit)  // every head's value divided by its root mean square: that is what the cache keeps
+            Vcur = ggml_reshape_2d(ctx, named(ggml_rms_norm(ctx, ggml_reshape_3d(ctx, Vcur, DV, G, n_tokens), hp.rms_eps), "Vcur_unit", run), G * DV, n_tokens);
+        if (lc.v_mix) {
+            if (!*v_first) *v_first = Vcur;
+            else {
+                LLM_ASSERT((*v_first)->ne[0] == Vcur->ne[0]);
+                Vcur = named(ggml_add(ctx, named(ggml_scale(ctx, Vcur, 1.0f - lc.v_lambda), "Vcur_own", run), named(ggml_scale(ctx, *v_first, lc.v_lambda), "Vcur_first", run)), "Vcur_mixed", run);
+            }
+        }
         ggml_build_forward_expand(gf, Kcur);
         ggml_build_forward_expand(gf, Vcur);
+        ggml_build_forward_expand(gf, named(ggml_set_rows(ctx, k_cache, ggml_reshape_2d(ctx, Kcur, G * DK, n_tokens), io.k_idxs), "k_store", run));
+        ggml_build_forward_expand(gf, named(ggml_set_rows(ctx, v_cache, lc.v_is_k ? Vcur : ggml_reshape_2d(ctx, Vcur, G * DV, n_tokens), io.k_idxs), "v_store", run));  // (blended / normed values are what is kept)
     }
-    Qcur = ggml_reshape_3d(ctx, Qcur, DK, H, n_tokens);
-    Kcur = ggml_reshape_3d(ctx, Kcur, DK, G, n_tokens);
-    if (lc.qk_norm) {  // every head's query and key divided by its root mean square, times a weight row shared by the heads
-        Qcur = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, Qcur, hp.rms_eps), "Qcur_rnorm", run), L.q_norm), "Qcur_normed", run);
-        Kcur = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, Kcur, hp.rms_eps), "Kcur_rnorm", run), L.k_norm), "Kcur_normed", run);
-    }
-    if (lc.q_temp_id >= 0) Qcur = named(ggml_mul(ctx, Qcur, io.q_temps[(size_t) lc.q_temp_id]), "Qcur_temp", run);
-    if (lc.rot_dims > 0) {  // neighbouring pairs (2i, 2i + 1) of the leading rot_dims entries; the rest of the head passes through
-        Qcur = named(ggml_rope_ext(ctx, Qcur, io.pos, nullptr, lc.rot_dims, lc.rot_half ? GGML_ROPE_TYPE_NEOX : 0, hp.n_ctx_train, lc.rot_base, 1.0f, 0.0f, 1.0f, 32.0f, 1.0f), "Qcur_rope", run);
-        Kcur = named(ggml_rope_ext(ctx, Kcur, io.pos, nullptr, lc.rot_dims, lc.rot_half ? GGML_ROPE_TYPE_NEOX : 0, hp.n_ctx_train, lc.rot_base, 1.0f, 0.0f, 1.0f, 32.0f, 1.0f), "Kcur_rope", run);
-        ggml_rope_set_exact_freq(Qcur);  // angle = pos * base^(-2 i / dims) with the frequency itself rounded once (not ggml's running product)
-        ggml_rope_set_exact_freq(Kcur);
-    }
-    if (lc.v_unit)  // every head's value divided by its root mean square: that is what the cache keeps
-        Vcur = ggml_reshape_2d(ctx, named(ggml_rms_norm(ctx, ggml_reshape_3d(ctx, Vcur, DV, G, n_tokens), hp.rms_eps), "Vcur_unit", run), G * DV, n_tokens);
-    if (lc.v_mix) {
-        if (!*v_first) *v_first = Vcur;
-        else {
-            LLM_ASSERT((*v_first)->ne[0] == Vcur->ne[0]);
-            Vcur = named(ggml_add(ctx, named(ggml_scale(ctx, Vcur, 1.0f - lc.v_lambda), "Vcur_own", run), named(ggml_scale(ctx, *v_first, lc.v_lambda), "Vcur_first", run)), "Vcur_mixed", run);
-        }
-    }
-    ggml_build_forward_expand(gf, Qcur);
-    ggml_build_forward_expand(gf, Kcur);
-    ggml_build_forward_expand(gf, Vcur);
-    ggml_tensor * k_cache = c->k_l[(size_t) run];
-    ggml_tensor * v_cache = c->v_l[(size_t) run];
-    ggml_build_forward_expand(gf, named(ggml_set_rows(ctx, k_cache, ggml_reshape_2d(ctx, Kcur, G * DK, n_tokens), io.k_idxs), "k_store", run));
-    ggml_build_forward_expand(gf, named(ggml_set_rows(ctx, v_cache, ggml_reshape_2d(ctx, Vcur, G * DV, n_tokens), io.k_idxs), "v_store", run));  // (blended / normed values are what is kept)
     ggml_tensor * q = ggml_permute(ctx, Qcur, 0, 2, 1, 3);
     ggml_tensor * k = ggml_view_3d(ctx, k_cache, DK, n_kv, G, ggml_row_size(k_cache->type, G * DK), ggml_row_size(k_cache->type, DK), 0);
     ggml_tensor * v = ggml_view_3d(ctx, v_cache, DV, n_kv, G, ggml_row_size(v_cache->type, G * DV), ggml_row_size(v_cache->type, DV), 0);
@@ -2452,13 +2754,7 @@ static ggml_tensor * build_mixer_latent(llm_context * c, ggml_context * ctx, ggm
         q_in = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, q_lat_pre, hp.rms_eps), "q_a_rnorm", run), L.dq_norm), "q_latent_normed", run);  // the queries' own normed latent
     }
     ggml_tensor * Qcur = named(ggml_mul_mat(ctx, L.wq, q_in), "Qcur", run);        // [DQ * H, T]: head by head [dk unrotated | dr rotated]
-    int cache_run = run;
-    if (!own_rows) {
-        cache_run = -1;
-        for (int r = 0; r < run; ++r)
-            if (m->runs[(size_t) r].il == lc.kv_from && m->runs[(size_t) r].pass == m->runs[(size_t) run].pass) cache_run = r;
-        LLM_ASSERT(cache_run >= 0 && c->k_l[(size_t) cache_run]);
-    }
+    const int cache_run = cache_run_of(c, lc, run);
     ggml_tensor * k_cache = c->k_l[(size_t) cache_run];
     ggml_tensor * q_rot = nullptr;
     if (DR > 0) {
@@ -2662,20 +2958,55 @@ static ggml_tensor * build_mixer_delta_channel(llm_context * c, ggml_context * c
     return named(ggml_mul_mat(ctx, wo, cur), "delta_out", run);
 }
 
-// grouped-query attention (left) and the delta rule with channel decay (right) over the same input; each output is RMS-normed over the width with a weight of its own,
-// and the mixer is left_scale * left + right_scale * right
+// two branches over one input, each output RMS-normed over the width with a weight of its own: left_scale * left + right_scale * right
+static ggml_tensor * build_two_branches(ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * left, ggml_tensor * right, float eps, int run) {
+    ggml_build_forward_expand(gf, left);
+    ggml_build_forward_expand(gf, right);  // (both branches first: the two norms, the two SCALEs and their ADD then follow one another, which the backend runs as one launch)
+    left = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, left, eps), "mix_left_rnorm", run), L.left_norm), "mix_left_normed", run);
+    right = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, right, eps), "mix_right_rnorm", run), L.right_norm), "mix_right_normed", run);
+    return named(ggml_add(ctx, named(ggml_scale(ctx, left, lc.left_scale), "mix_left", run), named(ggml_scale(ctx, right, lc.right_scale), "mix_right", run)), "mix_sum", run);
+}
+
+// grouped-query attention (left) and the delta rule with channel decay (right)
 static ggml_tensor * build_mixer_attn_delta(llm_context * c, ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * cur, int il, int run,
                                             int n_tokens, int n_kv, seg_io & io) {
-    const float eps = c->model->hp.rms_eps;
     ggml_tensor * v_first = nullptr;
     ggml_tensor * left = build_mixer_attention(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, &v_first);
     left = named(ggml_mul_mat(ctx, L.wo, left), "attn_out", run);
     ggml_build_forward_expand(gf, left);
     ggml_tensor * right = build_mixer_delta_channel(c, ctx, gf, L, L.wo_r, lc.r_head, lc.r_head_kv, lc.r_dk, lc.r_dv, lc.conv_taps, cur, run, n_tokens, io);
-    ggml_build_forward_expand(gf, right);  // (both branches first: the two norms, the two SCALEs and their ADD then follow one another, which the backend runs as one launch)
-    left = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, left, eps), "mix_left_rnorm", run), L.left_norm), "mix_left_normed", run);
-    right = named(ggml_mul(ctx, named(ggml_rms_norm(ctx, right, eps), "mix_right_rnorm", run), L.right_norm), "mix_right_normed", run);
-    return named(ggml_add(ctx, named(ggml_scale(ctx, left, lc.left_scale), "mix_left", run), named(ggml_scale(ctx, right, lc.right_scale), "mix_right", run)), "mix_sum", run);
+    return build_two_branches(ctx, gf, L, lc, left, right, c->model->hp.rms_eps, run);
+}
+
+// gated linear attention: q, k, v as one projection, one decay per (head, key channel) through two small matrices, the recurrence, per-head norm x weight x silu(gate); `wo`.
+// The projections of the input come as operands (the caller places them).  Returns [n_embd, T]
+static ggml_tensor * build_linear_attention(llm_context * c, ggml_context * ctx, const llm_layer & L, ggml_tensor * wo, int H, int DK, int DV, float tau, ggml_tensor * qkv, ggml_tensor * gate,
+                                            ggml_tensor * a_in, int run, int n_tokens, seg_io & io) {
+    ggml_tensor * a_pre = named(ggml_mul_mat(ctx, L.wa2, a_in), "linear_a_pre", run);  // [DK H, T]
+    ggml_tensor * q = ggml_view_2d(ctx, qkv, (int64_t) H * DK, n_tokens, qkv->nb[1], 0);
+    ggml_tensor * k = ggml_view_2d(ctx, qkv, (int64_t) H * DK, n_tokens, qkv->nb[1], (size_t) (H * DK) * sizeof(float));
+    ggml_tensor * v = ggml_view_2d(ctx, qkv, (int64_t) H * DV, n_tokens, qkv->nb[1], (size_t) (2 * H * DK) * sizeof(float));
+    ggml_tensor * o = named(ggml_seq_linear(ctx, q, k, v, a_pre, L.gate_par, c->rec_state[(size_t) run], io.seq_tok, io.seq_info, H, tau), "linear_attn", run);
+    ggml_tensor * cur = build_head_norm_gate(ctx, o, L.sub_norm, gate, GGML_UNARY_OP_SILU, c->model->hp.rms_eps, run);
+    return named(ggml_mul_mat(ctx, wo, cur), "linear_out", run);
+}
+
+// attention (left) and gated linear attention (right)
+static ggml_tensor * build_mixer_attn_linear(llm_context * c, ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * cur, int il, int run,
+                                             int n_tokens, int n_kv, seg_io & io) {
+    ggml_tensor * v_first = nullptr;
+    // (the right branch's products of the input come ahead of the left branch: all products of the one input follow one another)
+    ggml_tensor * qkv = named(ggml_mul_mat(ctx, L.wqkv_r, cur), "linear_qkv", run);
+    ggml_tensor * gate = named(ggml_mul_mat(ctx, L.wg1, cur), "linear_gate", run);
+    ggml_tensor * a_in = named(ggml_mul_mat(ctx, L.wa1, cur), "linear_a_in", run);
+    ggml_build_forward_expand(gf, qkv);
+    ggml_build_forward_expand(gf, gate);
+    ggml_build_forward_expand(gf, a_in);
+    ggml_tensor * left = build_mixer_attention(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, &v_first);
+    left = named(ggml_mul_mat(ctx, L.wo, left), "attn_out", run);
+    ggml_build_forward_expand(gf, left);
+    ggml_tensor * right = build_linear_attention(c, ctx, L, L.wo_r, lc.r_head, lc.r_dk, lc.r_dv, lc.r_tau, qkv, gate, a_in, run, n_tokens, io);
+    return build_two_branches(ctx, gf, L, lc, left, right, c->model->hp.rms_eps, run);
 }
 
 // the per-layer token input: e = the layer's row of the side table for every token; x += rms_norm(W_proj (gelu_tanh(W_gate x) * e)) * w
@@ -2712,7 +3043,15 @@ static ggml_tensor * build_moe_grouped(ggml_context * ctx, ggml_cgraph * gf, con
     return named(out, "ffn_moe_out", il);
 }
 
-// experts chosen by sigmoid scores plus a correction; the weights are the chosen scores themselves divided by their sum; experts with a limited gated activation
+// silu-gated feed-forward over a projection that holds the gate rows, then the up rows
+static ggml_tensor * build_gated_pair(ggml_context * ctx, ggml_tensor * w_gate_up, ggml_tensor * w_down, ggml_tensor * cur, const char * name, int run) {
+    const std::string n = name;
+    ggml_tensor * gu = named(ggml_mul_mat(ctx, w_gate_up, cur), (n + "_gate_up").c_str(), run);
+    return named(ggml_mul_mat(ctx, w_down, named(ggml_swiglu(ctx, gu), (n + "_act").c_str(), run)), (n + "_out").c_str(), run);
+}
+
+// experts chosen by sigmoid scores (plus a correction); the weights are the chosen scores themselves, divided by their sum or as they are, and multiply an expert's output or its
+// input; gated activation, with limits or without; optionally one more expert for every token behind a gate of its own
 static ggml_tensor * build_moe_sigmoid(ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & c, ggml_tensor * cur, int run) {
     const int64_t E = cur->ne[0], T = cur->ne[1], FF = c.n_ff;
     ggml_tensor * logits = named(ggml_mul_mat(ctx, L.ffn_gate_inp, cur), "ffn_moe_logits", run);  // [n_expert, T], f32 weights: 32-bit
@@ -2720,27 +3059,46 @@ static ggml_tensor * build_moe_sigmoid(ggml_context * ctx, ggml_cgraph * gf, con
     ggml_tensor * order = named(ggml_argsort(ctx, L.ffn_corr ? named(ggml_add(ctx, probs, L.ffn_corr), "ffn_moe_choice", run) : probs, 1), "ffn_moe_order", run);
     ggml_tensor * sel = ggml_view_2d(ctx, order, c.n_top, T, order->nb[1], 0);  // [n_top, T] i32
     ggml_tensor * w = named(ggml_get_rows(ctx, ggml_reshape_3d(ctx, probs, 1, c.n_expert, T), sel), "ffn_moe_sel_probs", run);  // [1, n_top, T]
-    w = ggml_reshape_2d(ctx, w, c.n_top, T);
-    w = named(ggml_div(ctx, w, named(ggml_scale_bias(ctx, named(ggml_sum_rows(ctx, w), "ffn_moe_sum", run), 1.0f, 1e-20f), "ffn_moe_sum_eps", run)), "ffn_moe_weights", run);
+    if (!c.moe_raw) {
+        w = ggml_reshape_2d(ctx, w, c.n_top, T);
+        w = named(ggml_div(ctx, w, named(ggml_scale_bias(ctx, named(ggml_sum_rows(ctx, w), "ffn_moe_sum", run), 1.0f, 1e-20f), "ffn_moe_sum_eps", run)), "ffn_moe_weights", run);
+    }
     ggml_set_output(w);                // (its few bytes are not handed to another tensor: the weighted sum over the experts reads them to its last row)
     ggml_build_forward_expand(gf, w);  // (the weights before the experts' products: the router is then one run of nodes, which the backend takes as one launch)
+    w = ggml_reshape_3d(ctx, w, 1, c.n_top, T);
     ggml_tensor * gu = named(ggml_mul_mat_id(ctx, L.ffn_gate_up_exps, ggml_reshape_3d(ctx, cur, E, 1, T), sel), "ffn_moe_gate_up", run);  // [2 ff, n_top, T]: gate rows, then up rows
-    ggml_tensor * act = named(ggml_swiglu_oai(ctx, ggml_reshape_2d(ctx, gu, 2 * FF, c.n_top * T), nullptr, 1.702f, c.moe_limit), "ffn_moe_act", run);
+    if (c.moe_scale_in) gu = named(ggml_mul(ctx, gu, w), "ffn_moe_gate_up_weighted", run);  // (the two products of w h are w times those of h)
+    gu = ggml_reshape_2d(ctx, gu, 2 * FF, c.n_top * T);
+    ggml_tensor * act = named(c.moe_limit > 0.0f ? ggml_swiglu_oai(ctx, gu, nullptr, 1.702f, c.moe_limit) : ggml_swiglu(ctx, gu), "ffn_moe_act", run);
     ggml_tensor * down = named(ggml_mul_mat_id(ctx, L.ffn_down_exps, ggml_reshape_3d(ctx, act, FF, c.n_top, T), sel), "ffn_moe_down", run);  // [E, n_top, T]
-    down = named(ggml_mul(ctx, down, ggml_reshape_3d(ctx, w, 1, c.n_top, T)), "ffn_moe_weighted", run);
+    if (!c.moe_scale_in) down = named(ggml_mul(ctx, down, w), "ffn_moe_weighted", run);
     ggml_build_forward_expand(gf, down);
-    ggml_tensor * out = nullptr;
-    for (int j = 0; j < c.n_top; ++j) {
-        ggml_tensor * v = ggml_view_2d(ctx, down, E, T, down->nb[2], (size_t) j * down->nb[1]);
-        out = out ? ggml_add(ctx, out, v) : v;
+    ggml_tensor * shared = nullptr, * sg = nullptr;
+    if (c.n_ff_shared > 0) {
+        sg = named(ggml_mul_mat(ctx, L.ffn_gate_inp_shexp, cur), "ffn_shared_gate", run);  // [1, T]
+        ggml_build_forward_expand(gf, sg);
+        shared = build_gated_pair(ctx, L.ffn_gate_up_shexp, L.ffn_down_shexp, cur, "ffn_shared", run);
+        ggml_build_forward_expand(gf, shared);  // (the products first: the gate, the sum over the experts and the norm behind it then follow one another, which the backend runs as one launch)
+        shared = named(ggml_mul(ctx, shared, named(ggml_unary(ctx, sg, GGML_UNARY_OP_SIGMOID), "ffn_shared_sigmoid", run)), "ffn_shared_gated", run);
+        ggml_build_forward_expand(gf, shared);
     }
-    if (c.n_top == 1) out = ggml_cont(ctx, out);
+    ggml_tensor * out = nullptr;
+    if (c.n_top == 1 && c.moe_scale_in) out = ggml_reshape_2d(ctx, down, E, T);
+    else {
+        for (int j = 0; j < c.n_top; ++j) {
+            ggml_tensor * v = ggml_view_2d(ctx, down, E, T, down->nb[2], (size_t) j * down->nb[1]);
+            out = out ? ggml_add(ctx, out, v) : v;
+        }
+        if (c.n_top == 1) out = ggml_cont(ctx, out);
+    }
+    if (shared) out = ggml_add(ctx, out, shared);
     return named(out, "ffn_moe_out", run);
 }
 
 static ggml_tensor * build_ffn(ggml_context * ctx, ggml_cgraph * gf, const llm_layer & L, const llm_layer_cfg & lc, ggml_tensor * cur, int il, int run) {
     if (lc.mlp == LLM_MLP_MOE && lc.moe_sigmoid) return build_moe_sigmoid(ctx, gf, L, lc, cur, run);
     if (lc.mlp == LLM_MLP_MOE) return lc.moe_scores_all ? build_moe_grouped(ctx, gf, L, lc, cur, il) : build_moe(ctx, gf, L, lc, cur, il);
+    if (lc.ffn_silu_gated) return build_gated_pair(ctx, L.ffn_gate_up, L.ffn_down, cur, "ffn", run);
     if (lc.ffn_gated_tanh) {
         ggml_tensor * g = named(ggml_add(ctx, named(ggml_mul_mat(ctx, L.ffn_gate, cur), "ffn_gate", run), L.ffn_gate_b), "ffn_gate_b", run);
         ggml_tensor * u = named(ggml_add(ctx, named(ggml_mul_mat(ctx, L.ffn_up, cur), "ffn_up", run), L.ffn_up_b), "ffn_up_b", run);
@@ -2762,6 +3120,7 @@ static ggml_tensor * build_mixer(llm_context * c, ggml_context * ctx, ggml_cgrap
         case LLM_MIX_SIGMOID_WKV: return build_mixer_sigmoid_wkv(c, ctx, gf, L, lc, cur, run, n_tokens, n_kv, io);
         case LLM_MIX_SSD: return build_mixer_ssd(c, ctx, gf, L, lc, cur, run, n_tokens, io);
         case LLM_MIX_ATTN_DELTA: return build_mixer_attn_delta(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io);
+        case LLM_MIX_ATTN_LINEAR: return build_mixer_attn_linear(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io);
         case LLM_MIX_LATENT: cur = build_mixer_latent(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io); break;
         default: cur = build_mixer_attention(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, v_first); break;
     }
@@ -2824,7 +3183,7 @@ static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * g
             inpL = named(ggml_add(ctx, inpL, step), "loop_x", run);
         }
         ggml_tensor * inpSA = inpL;
-        ggml_tensor * h = norm_w(ctx, lc, inpL, L.attn_norm, eps, "attn_norm", run);
+        ggml_tensor * h = lc.no_pre_norm ? inpL : norm_w(ctx, lc, inpL, L.attn_norm, eps, "attn_norm", run);
         ggml_tensor * cur = lc.shift ? build_token_shift(c, ctx, gf, h, L.shift, run, io) : h;
         cur = build_mixer(c, ctx, gf, L, lc, cur, il, run, n_tokens, n_kv, io, &v_first);
         if (lc.parallel) {  // both sublayers read the one normed input (the feed-forward the unshifted one); their sum joins the stream
@@ -2851,7 +3210,7 @@ static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * g
         if (L.attn_post_norm) cur = norm_w(ctx, lc, cur, L.attn_post_norm, eps, "attn_post_norm", run);
         ggml_tensor * ffn_inp = named(ggml_add(ctx, cur, inpSA), lc.mlp == LLM_MLP_NONE ? "l_out" : "ffn_inp", run);
         if (lc.mlp == LLM_MLP_NONE) { inpL = ffn_inp; continue; }
-        cur = norm_w(ctx, lc, ffn_inp, L.ffn_norm, eps, "ffn_norm", run);
+        cur = lc.no_pre_norm ? ffn_inp : norm_w(ctx, lc, ffn_inp, L.ffn_norm, eps, "ffn_norm", run);
         cur = build_ffn(ctx, gf, L, lc, cur, il, run);
         if (L.ffn_post_norm) cur = norm_w(ctx, lc, cur, L.ffn_post_norm, eps, "ffn_post_norm", run);
         inpL = named(ggml_add(ctx, cur, ffn_inp), "l_out", run);
@@ -2860,8 +3219,13 @@ static void build_layerwise(llm_context * c, ggml_context * ctx, ggml_cgraph * g
     ggml_tensor * cur = m->n_streams > 0 ? build_stream_layers(c, ctx, gf, inpL, n_tokens, n_kv, io)
                       : rms_out ? named(ggml_mul(ctx, named(ggml_rms_norm(ctx, inpL, eps), "rnorm", -1), m->output_norm), "result_norm", -1)
                                 : layer_norm_w(ctx, inpL, m->output_norm, eps, "result_norm", -1);
-    cur = named(ggml_mul_mat(ctx, m->output, cur), m->logit_scale != 1.0f ? "result_unscaled" : "result_output", -1);
+    const bool capped = m->logit_softcap > 0.0f;
+    cur = named(ggml_mul_mat(ctx, m->output, cur), m->logit_scale != 1.0f || capped ? "result_unscaled" : "result_output", -1);
     if (m->logit_scale != 1.0f) cur = named(ggml_scale(ctx, cur, m->logit_scale), "result_output", -1);
+    if (capped) {
+        cur = named(ggml_unary(ctx, named(ggml_scale(ctx, cur, 1.0f / m->logit_softcap), "result_by_cap", -1), GGML_UNARY_OP_TANH), "result_tanh", -1);
+        cur = named(ggml_scale(ctx, cur, m->logit_softcap), "result_output", -1);
+    }
     ggml_set_output(cur);
     ggml_build_forward_expand(gf, cur);
     io.out = cur;
@@ -2941,7 +3305,7 @@ extern "C" struct llm_context * llm_context_new(struct llm_model * m, ggml_backe
         // layer keeps ONE row [latent | rotated key part] per token and no values beside it)
         const llm_layer_cfg * lc = layerwise ? &m->lcfg[(size_t) m->runs[(size_t) run].il] : nullptr;
         const bool latent = lc && lc->mixer == LLM_MIX_LATENT;
-        if (lc && (lc->mixer == LLM_MIX_MLSTM || lc->mixer == LLM_MIX_DELTA || lc->mixer == LLM_MIX_SSD || (latent && lc->kv_from >= 0))) {
+        if (lc && (lc->mixer == LLM_MIX_MLSTM || lc->mixer == LLM_MIX_DELTA || lc->mixer == LLM_MIX_SSD || lc->kv_from >= 0)) {
             // (no cells: everything such a layer keeps is its sequence state — or it attends over the rows another layer's cache holds)
             c->k_l.push_back(nullptr);
             c->v_l.push_back(nullptr);
@@ -2972,6 +3336,7 @@ extern "C" struct llm_context * llm_context_new(struct llm_model * m, ggml_backe
             else if (lc.mixer == LLM_MIX_DELTA) { conv_c = 2 * (int64_t) lc.n_head_kv * lc.dk + (int64_t) lc.n_head * lc.dv; rec = ggml_seq_state_size(1, lc.n_head, lc.dk, lc.dv); }
             else if (lc.mixer == LLM_MIX_SSD) { conv_c = (int64_t) lc.n_head * lc.dv + 2 * (int64_t) lc.ssm_groups * lc.ssm_state; rec = ggml_seq_state_size(4, lc.n_head, lc.ssm_state, lc.dv); }
             else if (lc.mixer == LLM_MIX_ATTN_DELTA) { conv_c = 2 * (int64_t) lc.r_head_kv * lc.r_dk + (int64_t) lc.r_head * lc.r_dv; rec = ggml_seq_state_size(3, lc.r_head, lc.r_dk, lc.r_dv); }
+            else if (lc.mixer == LLM_MIX_ATTN_LINEAR) { conv_c = (int64_t) (lc.n_head + lc.n_head_kv) * lc.dk; rec = ggml_seq_state_size(5, lc.r_head, lc.r_dk, lc.r_dv); }
             else if (lc.mixer == LLM_MIX_SIGMOID_WKV) {
                 conv_c = (int64_t) (lc.n_head + lc.n_head_kv) * lc.dk + (int64_t) lc.n_head_kv * lc.dv;
                 rec = ggml_seq_state_size(0, lc.tm_heads, lc.tm_dim, lc.tm_dim);

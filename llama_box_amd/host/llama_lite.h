@@ -65,7 +65,10 @@ struct llm_model * llm_model_load(const char * path, ggml_backend_buffer_type_t 
  * repeated range of layers); "Rarelorn" (mixers with state per sequence: a matrix memory with exponential gates, a gated delta rule behind short
  * convolutions, windowed sigmoid attention beside RWKV-style time mixing; experts chosen from a soft-max over all of them within the best groups);
  * "Nogavik" (latent attention with a query latent, optionally over an earlier layer's cache rows; a state-space mixer; attention beside a delta rule with one decay
- * per key channel; two norms of the same input per layer; a per-layer token input; tied output matrix).  wtype: GGML_TYPE_BF16 keeps the matrices as stored
+ * per key channel; two norms of the same input per layer; a per-layer token input; tied output matrix); "Pisulorn" (several residual streams, a linear distance penalty,
+ * experts chosen by corrected sigmoid scores); "Nidudra" (norms on the sublayers' outputs only; windowed attention with kept first tokens, optionally over an earlier layer's cache;
+ * rotated attention with a learned sink; attention whose values are its convolved keys beside gated linear attention; experts whose weights multiply their input beside a shared
+ * one; soft-capped logits).  wtype: GGML_TYPE_BF16 keeps the matrices as stored
  * (bf16 products, f32 accumulation); GGML_TYPE_F32 widens them at load (everything in 32-bit).  Norm weights and routers are always f32. */
 struct llm_model * llm_model_load_dir(const char * dir, ggml_backend_buffer_type_t buft, int wtype);
 /* the same model classes from the TEXT of a config.json and seeded random weights (benchmarks at sizes no file exists for) */
