@@ -1985,91 +1985,298 @@ static int try_fuse_router_scores(exec_state & st, int i) {
     return 1;
 }
 
-// UNARY(SIGMOID, router logits) [-> ADD(., correction row)] -> ARGSORT (descending) -> VIEW (top k) -> GET_ROWS(scores as [1, n, T], view) -> SUM_ROWS -> SCALE(1, bias) -> DIV: a router
-// that chooses by corrected scores and weights by the normalised scores themselves, one launch (views between the nodes skipped).  Returns the nodes consumed (0: no match)
+// UNARY(SIGMOID, router logits) [-> ADD(., correction row)] -> ARGSORT (descending) -> VIEW (top k) -> GET_ROWS(scores as [1, n, T], view) [-> SUM_ROWS -> SCALE(1, bias) -> DIV]: a router
+// that chooses by (corrected) scores and weights by the scores themselves, as they are or divided by their sum, one launch (views between the nodes skipped).  Returns the nodes consumed
+// (0: no match)
 static int try_fuse_router_sigmoid(exec_state & st, int i) {
     ggml_cgraph * g = st.g;
     const ggml_tensor * sg = g->nodes[i];
     const ggml_tensor * a = sg->src[0];
     if (a->ne[0] > 256 || a->ne[2] != 1 || a->ne[3] != 1 || !is_f32_contig(a) || !is_f32_contig(sg) || (sg->flags & GGML_TENSOR_FLAG_OUTPUT)) return 0;
     const ggml_tensor * at[6] = {};
-    int found = 0, k = i + 1;
+    int found = 0, k = i + 1, k_pick = -1;  // k_pick: one past the GET_ROWS
     for (; k < g->n_nodes && k < i + 16 && found < 6; ++k) {
         const ggml_tensor * t = g->nodes[k];
-        if (st.done[k]) return 0;
+        if (st.done[k]) break;
         if (is_view_op(t)) continue;
         if (found == 0 && t->op != GGML_OP_ADD) at[found++] = nullptr;  // (no correction)
         at[found++] = t;
+        if (found == 3) k_pick = k + 1;
     }
-    if (found < 6) return 0;
+    if (found < 3) return 0;
     const ggml_tensor * ad = at[0], * as = at[1], * gr = at[2], * sm = at[3], * sc = at[4], * dv = at[5];
-    if (as->op != GGML_OP_ARGSORT || gr->op != GGML_OP_GET_ROWS || sm->op != GGML_OP_SUM_ROWS || sc->op != GGML_OP_SCALE || dv->op != GGML_OP_DIV) return 0;
+    if (as->op != GGML_OP_ARGSORT || gr->op != GGML_OP_GET_ROWS) return 0;
+    const bool raw = !(found == 6 && sm->op == GGML_OP_SUM_ROWS && sc->op == GGML_OP_SCALE && dv->op == GGML_OP_DIV);
     if (ad && (ad->src[0] != sg || !is_row_of(ad->src[1], sg) || !same_shape(ad, sg) || !single_use(st, ad))) return 0;
     if (as->src[0] != (ad ? ad : sg) || as->op_params[0] != 1 || as->op_params[1] > 1 || !ggml_abi_is_contiguous(as)) return 0;
     const ggml_tensor * sel = gr->src[1];
     if (!sel || sel->view_src != as || sel->view_offs != 0 || sel->ne[1] != a->ne[1] || sel->ne[0] > 256 || through_views(gr->src[0]) != sg || gr->src[0]->ne[0] != 1) return 0;
     const int64_t top = sel->ne[0], T = a->ne[1];
-    if (through_views(sm->src[0]) != gr || sm->src[0]->ne[0] != top || sc->src[0] != sm || ggml_abi_op_param_f32(sc, 0) != 1.0f || !single_use(st, sm) || !single_use(st, sc)) return 0;
-    if (dv->src[1] != sc || through_views(dv->src[0]) != gr || dv->src[0]->ne[0] != top || !is_f32_contig(dv) || ggml_abi_nelements(dv) != top * T) return 0;
-    if (use_count(st, sg) != 2 || use_count(st, gr) != (dv->src[0] == sm->src[0] ? 1 : 2)) return 0;  // (the sort — or the sum it reads — and the pick; through one view, or one each)
-    if (ranges_overlap(as, a) || ranges_overlap(dv, a) || ranges_overlap(as, dv) || (ad && (ranges_overlap(as, ad->src[1]) || ranges_overlap(dv, ad->src[1])))) return 0;
+    const ggml_tensor * out = raw ? gr : dv;
+    if (!is_f32_contig(out) || ggml_abi_nelements(out) != top * T || use_count(st, sg) != 2) return 0;  // (the scores' readers: the sort — or the sum it reads — and the pick)
+    if (!raw) {
+        if (through_views(sm->src[0]) != gr || sm->src[0]->ne[0] != top || sc->src[0] != sm || ggml_abi_op_param_f32(sc, 0) != 1.0f || !single_use(st, sm) || !single_use(st, sc)) return 0;
+        if (dv->src[1] != sc || through_views(dv->src[0]) != gr || dv->src[0]->ne[0] != top) return 0;
+        if (use_count(st, gr) != (dv->src[0] == sm->src[0] ? 1 : 2)) return 0;  // (through one view, or one each)
+    }
+    if (ranges_overlap(as, a) || ranges_overlap(out, a) || ranges_overlap(as, out) || (ad && (ranges_overlap(as, ad->src[1]) || ranges_overlap(out, ad->src[1])))) return 0;
     timed_scope ts(st.c, "router", (double) ggml_abi_nbytes(a) * 2);
-    launch_router_sigmoid_topk(st.c->stream, TD(a), ad ? (const float *) ad->src[1]->data : nullptr, TD(as), (float *) dv->data, (int) top, ggml_abi_op_param_f32(sc, 1));
+    launch_router_sigmoid_topk(st.c->stream, TD(a), ad ? (const float *) ad->src[1]->data : nullptr, TD(as), (float *) out->data, (int) top, raw ? 0.0f : ggml_abi_op_param_f32(sc, 1), raw);
     st.c->st.kernel_launches++;
-    st.c->st.fused_nodes += ad ? 6 : 5;
-    return k - i;
+    st.c->st.fused_nodes += (ad ? 3 : 2) + (raw ? 0 : 3);
+    return (raw ? k_pick : k) - i;
 }
 
-// RMS_NORM(q per head) -> MUL(w) [-> MUL(., one factor per token)], RMS_NORM(k per head) -> MUL(w), SET_ROWS(k), SET_ROWS(v) (views between the nodes skipped): the queries' and keys' norms
-// and both cache stores in one launch.  Returns the nodes consumed (0: no match)
+// what a head's queries or keys go through between their projection and the scores: [RMS_NORM -> MUL(weight row)] [-> MUL(one factor per token)] [-> ROPE by a table] [-> RMS_NORM]
+struct head_steps {
+    const ggml_tensor *x = nullptr, *norm = nullptr, *mul = nullptr, *temp = nullptr, *rope = nullptr, *unit = nullptr, *out = nullptr;
+    int n = 0;  // nodes that are no views
+};
+// follows the steps from node k (views skipped); returns the node behind them (-1: no such steps).  Every link but the last is read by the next one alone
+static int follow_head_steps(const exec_state & st, int k, head_steps & hs) {
+    const ggml_cgraph * g = st.g;
+    auto at = [&](int j) -> const ggml_tensor * {  // the next node that is no view, from j on (its index in `k`)
+        while (j < g->n_nodes && !st.done[j] && is_view_op(g->nodes[j])) ++j;
+        k = j;
+        return j < g->n_nodes && !st.done[j] ? g->nodes[j] : nullptr;
+    };
+    int end = -1;
+    auto take = [&](const ggml_tensor * t) { hs.out = t; ++hs.n; end = k + 1; };
+    auto linked = [&](const ggml_tensor * t) { return hs.out ? t->src[0] == hs.out && single_use(st, hs.out) : true; };
+    const ggml_tensor * t = at(k);
+    if (t && t->op == GGML_OP_RMS_NORM) {
+        const int k0 = k;
+        const ggml_tensor * m = at(k + 1);
+        if (!m || m->op != GGML_OP_MUL || m->src[0] != t || !is_row_of(m->src[1], t) || !single_use(st, t) || !same_shape(m, t)) return -1;
+        (void) k0;
+        hs.x = t->src[0]; hs.norm = t; hs.mul = m; hs.n = 1;
+        take(m);
+        t = at(end);
+        if (t && t->op == GGML_OP_MUL && t->src[0] == m && single_use(st, m) && is_f32_contig(t->src[1]) && t->src[1]->ne[0] == 1 && t->src[1]->ne[1] == 1 && t->src[1]->ne[2] == m->ne[2] &&
+            t->src[1]->ne[3] == 1) {
+            hs.temp = t;
+            take(t);
+            t = at(end);
+        }
+    }
+    if (t && t->op == GGML_OP_ROPE && linked(t)) {
+        const bool table = t->op_params[3] == 2 && t->src[2] && (t->op_params[2] == GGML_ROPE_TYPE_NEOX || t->op_params[2] == 0) && t->op_params[1] > 0 && (t->op_params[1] % 2) == 0 &&
+                           t->op_params[1] <= t->ne[0] && t->src[1]->type == GGML_TYPE_I32 && ggml_abi_is_contiguous(t->src[1]) && t->src[2]->type == GGML_TYPE_F32 && ggml_abi_is_contiguous(t->src[2]);
+        if (!table) return -1;
+        if (!hs.x) hs.x = t->src[0];
+        hs.rope = t;
+        take(t);
+        t = at(end);
+    }
+    if (t && hs.rope && t->op == GGML_OP_RMS_NORM && linked(t)) {
+        hs.unit = t;
+        take(t);
+    }
+    return end;
+}
+// the steps of the queries, those of the keys, SET_ROWS(k), SET_ROWS(v) (views between the nodes skipped): one launch.  Returns the nodes consumed (0: no match)
 static int try_fuse_qk_norm_store(exec_state & st, int i) {
     ggml_cgraph * g = st.g;
-    const ggml_tensor * nq = g->nodes[i];
-    const ggml_tensor * q = nq->src[0];
-    const ggml_tensor * at[6] = {};
-    int found = 0, k = i + 1;
-    for (; k < g->n_nodes && k < i + 20 && found < 6; ++k) {
-        const ggml_tensor * t = g->nodes[k];
-        if (st.done[k]) return 0;
-        if (is_view_op(t)) continue;
-        if (found == 1 && t->op != GGML_OP_MUL) at[found++] = nullptr;  // (no factor per token)
-        at[found++] = t;
+    head_steps hq, hk;
+    int k = follow_head_steps(st, i, hq);
+    if (k < 0) return 0;
+    k = follow_head_steps(st, k, hk);
+    if (k < 0 || hk.temp || !hq.norm != !hk.norm || !hq.rope != !hk.rope || !hq.unit != !hk.unit) return 0;
+    const ggml_tensor * at[2] = {};
+    for (int found = 0; found < 2; ++k) {
+        if (k >= g->n_nodes || st.done[k]) return 0;
+        if (!is_view_op(g->nodes[k])) at[found++] = g->nodes[k];
     }
-    if (found < 6) return 0;
-    const ggml_tensor * mq = at[0], * tq = at[1], * nk = at[2], * mk = at[3], * sk = at[4], * sv = at[5];
-    if (mq->op != GGML_OP_MUL || nk->op != GGML_OP_RMS_NORM || mk->op != GGML_OP_MUL || sk->op != GGML_OP_SET_ROWS || sv->op != GGML_OP_SET_ROWS) return 0;
-    const int64_t DK = q->ne[0], H = q->ne[1], T = q->ne[2];
-    const ggml_tensor * kx = nk->src[0];
-    if (q->ne[3] != 1 || !is_f32_contig(q) || !is_f32_contig(kx) || kx->ne[0] != DK || kx->ne[2] != T || kx->ne[3] != 1) return 0;
-    const ggml_tensor * qo = tq ? tq : mq;  // the queries as attention reads them
-    if (mq->src[0] != nq || mk->src[0] != nk || !single_use(st, nq) || !single_use(st, nk) || !is_row_of(mq->src[1], nq) || !is_row_of(mk->src[1], nk) || !is_f32_contig(qo) || !same_shape(qo, nq)) return 0;
-    if (tq && (tq->src[0] != mq || !single_use(st, mq) || !is_f32_contig(tq->src[1]) || tq->src[1]->ne[0] != 1 || tq->src[1]->ne[1] != 1 || tq->src[1]->ne[2] != T || tq->src[1]->ne[3] != 1)) return 0;
-    const ggml_tensor * v = through_views(sv->src[0]);
-    const int64_t G = kx->ne[1];
-    if (through_views(sk->src[0]) != mk || use_count(st, mk) != 1 || (mk->flags & GGML_TENSOR_FLAG_OUTPUT) || !is_f32_contig(v) || !is_f32_contig(sv->src[0]) || v == mk) return 0;
-    const ggml_tensor * idx = sk->src[1];
+    const ggml_tensor * sk = at[0], * sv = at[1], * q = hq.x, * kx = hk.x, * qo = hq.out;
+    if (sk->op != GGML_OP_SET_ROWS || sv->op != GGML_OP_SET_ROWS) return 0;
+    const int64_t DK = q->ne[0], H = q->ne[1], T = q->ne[2], G = kx->ne[1];
+    auto heads_ok = [&](const ggml_tensor * t) {  // [DK, heads, T], a token's heads contiguous
+        return t->type == GGML_TYPE_F32 && t->nb[0] == 4 && t->nb[1] == (size_t) DK * 4 && (t->nb[2] % 4) == 0 && t->ne[0] == DK && t->ne[2] == T && t->ne[3] == 1;
+    };
+    if (!heads_ok(q) || !heads_ok(kx) || !is_f32_contig(qo) || !same_shape(qo, q) || !same_shape(hk.out, kx)) return 0;
+    if (hq.rope && (DK > QK_ROT_MAX_DK || memcmp(hq.rope->op_params, hk.rope->op_params, sizeof(hq.rope->op_params)) != 0 || hq.rope->src[1] != hk.rope->src[1] || hq.rope->src[2] != hk.rope->src[2] ||
+                    ggml_abi_nelements(hq.rope->src[1]) != T || ggml_abi_nelements(hq.rope->src[2]) < hq.rope->op_params[1] / 2)) return 0;
+    if (hq.unit && ggml_abi_op_param_f32(hq.unit, 0) != ggml_abi_op_param_f32(hk.unit, 0)) return 0;
+    if (through_views(sk->src[0]) != hk.out || use_count(st, hk.out) != 1 || (hk.out->flags & GGML_TENSOR_FLAG_OUTPUT) || through_views(sv->src[0]) == hk.out) return 0;
+    const ggml_tensor * idx = sk->src[1], * v = sv->src[0];
     if (idx != sv->src[1] || idx->type != GGML_TYPE_I64 || !ggml_abi_is_contiguous(idx) || ggml_abi_nelements(idx) != T) return 0;
     auto cache_ok = [](const ggml_tensor * t) {
         return (t->type == GGML_TYPE_F32 || t->type == GGML_TYPE_BF16 || t->type == GGML_TYPE_F16) && t->nb[0] == ggml_abi_type_size(t->type) && t->ne[2] == 1 && t->ne[3] == 1;
     };
-    const int64_t row_v = sv->src[0]->ne[0];
-    if (!cache_ok(sk) || !cache_ok(sv) || sk->ne[0] != DK * G || sk->src[0]->ne[0] != DK * G || sk->src[0]->ne[1] != T || sv->src[0]->ne[1] != T || sv->ne[0] != row_v || row_v % G != 0 ||
-        ggml_abi_nelements(v) != row_v * T) return 0;
+    const int64_t row_v = v->ne[0];
+    if (!cache_ok(sk) || !cache_ok(sv) || sk->ne[0] != DK * G || sk->src[0]->ne[0] != DK * G || sk->src[0]->ne[1] != T || v->type != GGML_TYPE_F32 || v->nb[0] != 4 || (v->nb[1] % 4) != 0 || v->ne[1] != T ||
+        v->ne[2] != 1 || v->ne[3] != 1 || sv->ne[0] != row_v || row_v % G != 0) return 0;
     // (every wave reads its own row before it writes: the queries' result may be the projection's own block, nothing else)
-    if (!elementwise_safe(qo, q) || ranges_overlap(qo, kx) || ranges_overlap(qo, v) || ranges_overlap(qo, mq->src[1]) || ranges_overlap(qo, mk->src[1]) || (tq && ranges_overlap(qo, tq->src[1]))) return 0;
+    if (!(is_f32_contig(q) ? elementwise_safe(qo, q) : !ranges_overlap(qo, q)) || ranges_overlap(qo, kx) || ranges_overlap(qo, v)) return 0;
+    for (const ggml_tensor * t : {hq.mul ? hq.mul->src[1] : nullptr, hk.mul ? hk.mul->src[1] : nullptr, hq.temp ? hq.temp->src[1] : nullptr, hq.rope ? hq.rope->src[1] : nullptr, hq.rope ? hq.rope->src[2] : nullptr})
+        if (t && ranges_overlap(qo, t)) return 0;
     qk_norm_store_args a{};
     a.q = (const float *) q->data; a.qd = (float *) qo->data; a.k = (const float *) kx->data; a.v = (const float *) v->data;
-    a.qw = (const float *) mq->src[1]->data; a.kw = (const float *) mk->src[1]->data; a.temp = tq ? (const float *) tq->src[1]->data : nullptr;
+    a.q_tok = (int64_t) (q->nb[2] / 4); a.k_tok = (int64_t) (kx->nb[2] / 4); a.v_tok = (int64_t) (v->nb[1] / 4);
+    a.qw = hq.mul ? (const float *) hq.mul->src[1]->data : nullptr; a.kw = hk.mul ? (const float *) hk.mul->src[1]->data : nullptr;
+    a.temp = hq.temp ? (const float *) hq.temp->src[1]->data : nullptr;
+    if (hq.rope) {
+        a.pos = (const int32_t *) hq.rope->src[1]->data; a.freq = (const float *) hq.rope->src[2]->data; a.mag = ggml_abi_op_param_f32(hq.rope, 8);
+        a.n_rot = hq.rope->op_params[1]; a.neox = hq.rope->op_params[2] == GGML_ROPE_TYPE_NEOX;
+    }
+    if (hq.unit) { a.unit = 1; a.eps_unit = ggml_abi_op_param_f32(hq.unit, 0); }
     a.k_cache = (char *) sk->data; a.v_cache = (char *) sv->data;
     a.kc_nb1 = (int64_t) sk->nb[1]; a.vc_nb1 = (int64_t) sv->nb[1];
     a.idx = (const int64_t *) idx->data;
-    a.eps_q = ggml_abi_op_param_f32(nq, 0); a.eps_k = ggml_abi_op_param_f32(nk, 0);
+    if (hq.norm) { a.eps_q = ggml_abi_op_param_f32(hq.norm, 0); a.eps_k = ggml_abi_op_param_f32(hk.norm, 0); }
     a.H = (int) H; a.G = (int) G; a.DK = (int) DK; a.DV = (int) (row_v / G); a.k_type = sk->type; a.v_type = sv->type;
-    timed_scope ts(st.c, "qk_norm_store", (double) (ggml_abi_nbytes(q) * 2 + ggml_abi_nbytes(kx) + ggml_abi_nbytes(v)));
+    timed_scope ts(st.c, "qk_norm_store", (double) (ggml_abi_nbytes(qo) * 2 + ggml_abi_nelements(kx) * 4 + row_v * T * 4));
     launch_qk_norm_store(st.c->stream, a, T);
     st.c->st.kernel_launches++;
-    st.c->st.fused_nodes += tq ? 6 : 5;
+    st.c->st.fused_nodes += hq.n + hk.n + 1;
     return k - i;
+}
+
+// [ADD(x, bias row) ->] SSM_CONV -> SSM_CONV (store) of one input: the bias goes into the loads of both; a batch of one token per sequence is ONE launch (a thread has read its channel's
+// history before it writes it).  Returns the nodes consumed at position i (0: no match)
+static int try_fuse_conv_store(exec_state & st, int i) {
+    ggml_cgraph * g = st.g;
+    const ggml_tensor * n = g->nodes[i], * ad = n->op == GGML_OP_ADD ? n : nullptr;
+    int k = i;
+    auto next_at = [&](int j) -> const ggml_tensor * {
+        while (j < g->n_nodes && !st.done[j] && is_view_op(g->nodes[j])) ++j;
+        k = j;
+        return j < g->n_nodes && !st.done[j] ? g->nodes[j] : nullptr;
+    };
+    const ggml_tensor * cv = ad ? next_at(i + 1) : n;
+    if (!cv || cv->op != GGML_OP_SSM_CONV || cv->op_params[3] != MI_SEQ_OP_TAG || cv->op_params[2] != 0) return 0;
+    const ggml_tensor * x = cv->src[0];
+    if (ad && (x != ad || !is_f32_contig(ad) || !is_f32_contig(ad->src[0]) || !same_shape(ad, ad->src[0]) || !is_row_of(ad->src[1], ad) || (ad->flags & GGML_TENSOR_FLAG_OUTPUT))) return 0;
+    const int taps = cv->op_params[0];
+    const int k_conv = k;
+    const ggml_tensor * so = taps > 1 ? next_at(k_conv + 1) : nullptr;
+    if (so && (so->op != GGML_OP_SSM_CONV || so->op_params[3] != MI_SEQ_OP_TAG || so->op_params[2] != 1 || so->src[0] != x || so->data != cv->src[2]->data || so->op_params[0] != taps)) so = nullptr;
+    if (taps > 1 && !so) return 0;
+    if (ad && use_count(st, ad) != (so ? 2 : 1)) return 0;
+    const int64_t T = x->ne[1], n_seqs = so ? so->src[2]->ne[1] : 0;
+    const bool step = so && n_seqs == T;
+    if (!step && !ad) return 0;
+    const ggml_tensor * in = ad ? ad->src[0] : x;
+    if (ranges_overlap(cv, in) || (ad && ranges_overlap(cv, ad->src[1])) || (so && ranges_overlap(cv, so))) return 0;
+    const float * ib = ad ? (const float *) ad->src[1]->data : nullptr;
+    const float * bias = cv->src[4] ? (const float *) cv->src[4]->data : nullptr;
+    timed_scope ts(st.c, "seq_conv", (double) (ggml_abi_nbytes(x) + ggml_abi_nbytes(cv)));
+    const int32_t * hist = cv->src[3] ? (const int32_t *) cv->src[3]->data : nullptr;
+    const int hs = cv->src[3] ? (int) cv->src[3]->ne[0] : 0;
+    if (step) launch_seq_conv_step(st.c->stream, TD(in), ib, (const float *) cv->src[1]->data, bias, (float *) so->data, hist, hs, (const int32_t *) so->src[1]->data, (int) so->src[1]->ne[0],
+                                   (const int32_t *) so->src[2]->data, (int) n_seqs, TD(cv), taps, cv->op_params[1]);
+    else {
+        launch_seq_conv(st.c->stream, TD(in), ib, (const float *) cv->src[1]->data, bias, cv->src[2] ? (const float *) cv->src[2]->data : nullptr, hist, hs, TD(cv), taps, cv->op_params[1]);
+        if (so) launch_seq_conv_store(st.c->stream, TD(in), ib, (float *) so->data, (const int32_t *) so->src[1]->data, (int) so->src[1]->ne[0], (const int32_t *) so->src[2]->data, (int) n_seqs, taps);
+    }
+    st.c->st.kernel_launches += step || !so ? 1 : 2;
+    st.c->st.fused_nodes += (ad ? 1 : 0) + (step ? 1 : 0);
+    return (so ? k : k_conv) + 1 - i;
+}
+
+// RMS_NORM(.) -> MUL(., w row) -> ADD(x, .) at node k (views skipped): a row `t` that nothing else reads, normed and joining the stream.  Returns the ADD and the node behind it (null: no match)
+struct norm_join {
+    const ggml_tensor *norm = nullptr, *mul = nullptr, *add = nullptr, *w = nullptr, *res = nullptr;
+    int end = -1;
+};
+static norm_join follow_norm_join(const exec_state & st, int k, const ggml_tensor * t) {
+    const ggml_cgraph * g = st.g;
+    const ggml_tensor * at[3] = {};
+    for (int found = 0; found < 3; ++k) {
+        if (k >= g->n_nodes || st.done[k]) return {};
+        if (!is_view_op(g->nodes[k])) at[found++] = g->nodes[k];
+    }
+    norm_join j;
+    j.norm = at[0]; j.mul = at[1]; j.add = at[2];
+    if (j.norm->op != GGML_OP_RMS_NORM || j.norm->src[0] != t || j.mul->op != GGML_OP_MUL || j.mul->src[0] != j.norm || j.add->op != GGML_OP_ADD || j.add->src[0] == j.add->src[1]) return {};
+    if (j.add->src[0] != j.mul && j.add->src[1] != j.mul) return {};
+    j.res = j.add->src[0] == j.mul ? j.add->src[1] : j.add->src[0];
+    j.w = j.mul->src[1];
+    if (!single_use(st, t) || !single_use(st, j.norm) || !single_use(st, j.mul) || !is_f32_contig(t) || !is_f32_contig(j.add) || !is_f32_contig(j.res) || !same_shape(j.add, t) || !same_shape(j.res, t) ||
+        !same_shape(j.mul, t) || !is_row_of(j.w, t) || !elementwise_safe(j.add, j.res) || ranges_overlap(j.add, j.w)) return {};
+    j.end = k;
+    return j;
+}
+
+// UNARY(SIGMOID, one gate per token) -> MUL(shared expert's row, .) ... the sum of the token's expert rows as a chain of ADDs over slices of one MUL_MAT_ID ... ADD(., gated row)
+// [-> RMS_NORM -> MUL(w) -> ADD(x)]: one launch.  Without a shared expert the pattern begins at the first ADD of the chain.  Returns the nodes consumed (0: no match)
+static int try_fuse_expert_join(exec_state & st, int i) {
+    ggml_cgraph * g = st.g;
+    const ggml_tensor * first = g->nodes[i];
+    int k = i;
+    auto next_at = [&](int j) -> const ggml_tensor * {
+        while (j < g->n_nodes && !st.done[j] && is_view_op(g->nodes[j])) ++j;
+        k = j;
+        return j < g->n_nodes && !st.done[j] ? g->nodes[j] : nullptr;
+    };
+    auto base_of = [](const ggml_tensor * t) -> const ggml_tensor * {
+        const ggml_tensor * b = t && (t->op == GGML_OP_VIEW || t->op == GGML_OP_RESHAPE) ? t->view_src : nullptr;
+        return b && b->op == GGML_OP_MUL_MAT_ID && is_f32_contig(b) && b->ne[3] == 1 ? b : nullptr;
+    };
+    const ggml_tensor * gated = nullptr, * sh = nullptr, * sg = nullptr, * t = first;
+    int n_ops = 0;
+    if (first->op == GGML_OP_UNARY) {
+        sg = first->src[0];
+        if (first->op_params[0] != GGML_UNARY_OP_SIGMOID || !is_f32_contig(sg) || sg->ne[0] != 1 || !single_use(st, first)) return 0;
+        gated = next_at(i + 1);
+        if (!gated || gated->op != GGML_OP_MUL || gated->src[1] != first || !single_use(st, gated) || !is_f32_contig(gated)) return 0;
+        sh = gated->src[0];
+        if (!is_f32_contig(sh) || !same_shape(gated, sh) || sh->ne[2] != 1 || sh->ne[3] != 1 || ggml_abi_nelements(sg) != sh->ne[1]) return 0;
+        n_ops = 2;
+        t = next_at(k + 1);
+    }
+    if (!t || t->op != GGML_OP_ADD) return 0;
+    const ggml_tensor * D = base_of(t->src[0]);
+    if (!D) return 0;
+    const int64_t E = D->ne[0], top = D->ne[1], T = D->ne[2];
+    if (top > 64 || (sh && (sh->ne[0] != E || sh->ne[1] != T)) || (!sh && top < 2)) return 0;
+    auto slice = [&](const ggml_tensor * v, int64_t u) {
+        return base_of(v) == D && v->ne[0] == E && v->ne[1] == T && v->ne[2] == 1 && v->ne[3] == 1 && v->nb[0] == 4 && v->nb[1] == (size_t) D->nb[2] && (const char *) v->data == (const char *) D->data + u * D->nb[1];
+    };
+    if (!slice(t->src[0], 0)) return 0;
+    int64_t u = 1;
+    const ggml_tensor * acc = nullptr;  // the last ADD taken
+    int end = -1;
+    for (;;) {
+        if (!t || t->op != GGML_OP_ADD || (acc && (t->src[0] != acc || !single_use(st, acc))) || !is_f32_contig(t) || t->ne[0] != E || t->ne[1] != T || t->ne[2] != 1 || t->ne[3] != 1) return 0;
+        const bool last = sh ? t->src[1] == gated : u == top - 1;
+        if (sh && last ? u != top : !slice(t->src[1], u)) return 0;
+        ++n_ops;
+        acc = t;
+        end = k + 1;
+        if (last) break;
+        ++u;
+        t = next_at(k + 1);
+    }
+    const norm_join j = follow_norm_join(st, end, acc);
+    const ggml_tensor * out = j.add ? j.add : acc;
+    if (!(top == 1 ? elementwise_safe(out, D) : !ranges_overlap(out, D)) || (sh && (!elementwise_safe(out, sh) || ranges_overlap(out, sg)))) return 0;
+    timed_scope ts(st.c, "expert_join", (double) (E * T) * 4.0 * (double) (top + (sh ? 1 : 0) + (j.add ? 2 : 1)));
+    launch_expert_join(st.c->stream, (const float *) D->data, (int) top, sh ? (const float *) sh->data : nullptr, sh ? (const float *) sg->data : nullptr, (float *) out->data, E, T,
+                       j.add ? (const float *) j.w->data : nullptr, j.add ? (const float *) j.res->data : nullptr, j.add ? ggml_abi_op_param_f32(j.norm, 0) : 0.0f);
+    st.c->st.kernel_launches++;
+    st.c->st.fused_nodes += n_ops - 1 + (j.add ? 3 : 0);
+    return (j.add ? j.end : end) - i;
+}
+
+// MUL(rows of MUL_MAT_ID [2 nc, n_used, T], one factor per row) -> SwiGLU of the halves: one launch.  Returns the nodes consumed (0: no match)
+static int try_fuse_swiglu_scaled(exec_state & st, int i) {
+    ggml_cgraph * g = st.g;
+    const ggml_tensor * m = g->nodes[i], * gu = m->src[0], * w = m->src[1];
+    int k = i + 1;
+    while (k < g->n_nodes && !st.done[k] && is_view_op(g->nodes[k])) ++k;
+    if (k >= g->n_nodes || st.done[k]) return 0;
+    const ggml_tensor * gl = g->nodes[k];
+    if (gl->op != GGML_OP_GLU || gl->op_params[0] != GGML_GLU_OP_SWIGLU || gl->op_params[1] != 0 || gl->src[1] || through_views(gl->src[0]) != m || use_count(st, m) != 1 || (m->flags & GGML_TENSOR_FLAG_OUTPUT)) return 0;
+    const int64_t nc = gl->ne[0], rows = ggml_abi_nrows(gl);
+    if (!is_f32_contig(gu) || !is_f32_contig(m) || !is_f32_contig(gl) || !is_f32_contig(w) || !same_shape(m, gu) || gu->ne[0] != 2 * nc || gl->src[0]->ne[0] != 2 * nc || ggml_abi_nrows(gu) != rows ||
+        w->ne[0] != 1 || w->ne[1] != gu->ne[1] || w->ne[2] != gu->ne[2] || w->ne[3] != gu->ne[3]) return 0;
+    if (ranges_overlap(gl, gu) || ranges_overlap(gl, w)) return 0;
+    timed_scope ts(st.c, "swiglu", (double) ggml_abi_nbytes(gl) * 3);
+    launch_swiglu_scaled(st.c->stream, (const float *) gu->data, (const float *) w->data, (float *) gl->data, nc, rows);
+    st.c->st.kernel_launches++;
+    st.c->st.fused_nodes++;
+    return k + 1 - i;
 }
 
 // ADD(x, y) -> RMS_NORM(.) -> MUL(., w row): a residual update and the norm of the sublayer that follows in one launch (pre-norm models whose norms are RMS norms).
@@ -2178,7 +2385,19 @@ static int try_fuse_norm2_blend(exec_state & st, int i) {
     const ggml_tensor * l = n1->src[0], * r = n2->src[0], * wl = m1->src[1], * wr = m2->src[1];
     for (const ggml_tensor * t : {n1, m1, n2, m2, s1, s2}) if (!single_use(st, t) || !is_f32_contig(t) || !same_shape(t, ad)) return 0;
     if (!is_f32_contig(l) || !is_f32_contig(r) || !is_f32_contig(ad) || !same_shape(l, ad) || !same_shape(r, ad) || !is_row_of(wl, ad) || !is_row_of(wr, ad)) return 0;
+    // ... -> RMS_NORM -> MUL(w) -> ADD(x): the blend normed once more and joining the stream
+    const norm_join nj = follow_norm_join(st, i + 7, ad);
+    if (nj.add && elementwise_safe(nj.add, l) && elementwise_safe(nj.add, r) && !ranges_overlap(nj.add, wl) && !ranges_overlap(nj.add, wr)) {
+        timed_scope ts(st.c, "norm2_blend", (double) ggml_abi_nbytes(ad) * 4);
+        launch_rms_norm2_blend_join(st.c->stream, (const float *) l->data, (const float *) r->data, (const float *) wl->data, (const float *) wr->data, ggml_abi_op_param_f32(s1, 0),
+                                    ggml_abi_op_param_f32(s2, 0), (const float *) nj.w->data, (const float *) nj.res->data, (float *) nj.add->data, ad->ne[0], ggml_abi_nrows(ad),
+                                    ggml_abi_op_param_f32(n1, 0), ggml_abi_op_param_f32(nj.norm, 0));
+        st.c->st.kernel_launches++;
+        st.c->st.fused_nodes += 9;
+        return nj.end - i;
+    }
     if (!elementwise_safe(ad, l) || !elementwise_safe(ad, r) || ranges_overlap(ad, wl) || ranges_overlap(ad, wr)) return 0;
+    timed_scope ts(st.c, "norm2_blend", (double) ggml_abi_nbytes(ad) * 3);
     launch_rms_norm2_blend(st.c->stream, (const float *) l->data, (const float *) r->data, (const float *) wl->data, (const float *) wr->data, ggml_abi_op_param_f32(s1, 0),
                            ggml_abi_op_param_f32(s2, 0), (float *) ad->data, ad->ne[0], ggml_abi_nrows(ad), ggml_abi_op_param_f32(n1, 0));
     st.c->st.kernel_launches++;
@@ -2529,11 +2748,14 @@ static int run_node(exec_state & st, int i) {
 
         case GGML_OP_ADD: case GGML_OP_SUB: case GGML_OP_MUL: case GGML_OP_DIV: {
             if (fuse && n->op == GGML_OP_ADD) {
-                const int used = try_fuse_add_rms_norm(st, i);
+                int used = try_fuse_expert_join(st, i);
+                if (used == 0) used = try_fuse_conv_store(st, i);
+                if (used == 0) used = try_fuse_add_rms_norm(st, i);
                 if (used) return used;
             }
             if (fuse && n->op == GGML_OP_MUL) {
-                const int used = try_fuse_expert_sum(st, i);
+                int used = try_fuse_expert_sum(st, i);
+                if (used == 0) used = try_fuse_swiglu_scaled(st, i);
                 if (used > 0) return used;
             }
             static const bool row_fusions = !getenv("GGML_MI355X_ROW_FUSIONS") || atoi(getenv("GGML_MI355X_ROW_FUSIONS")) != 0;
@@ -2583,12 +2805,25 @@ static int run_node(exec_state & st, int i) {
                 c->st.fused_nodes += 2;
                 return 3;
             }
+            // SCALE(x, a) -> TANH -> SCALE(., b): a soft cap, one pass
+            if (fuse && s2 && ad && !st.done[i + 1] && !st.done[i + 2] && s2->op == GGML_OP_UNARY && s2->op_params[0] == GGML_UNARY_OP_TANH && s2->src[0] == n && ad->op == GGML_OP_SCALE && ad->src[0] == s2 &&
+                ggml_abi_op_param_f32(n, 1) == 0.0f && ggml_abi_op_param_f32(ad, 1) == 0.0f && single_use(st, n) && single_use(st, s2) && elementwise_safe(ad, a)) {
+                timed_scope ts(c, "softcap", (double) ggml_abi_nbytes(ad) * 2);
+                launch_softcap(s, (const float *) a->data, (float *) ad->data, ggml_abi_nelements(ad), ggml_abi_op_param_f32(n, 0), ggml_abi_op_param_f32(ad, 0));
+                c->st.kernel_launches++;
+                c->st.fused_nodes += 2;
+                return 3;
+            }
             launch_scale(s, TD(a), TD(n), ggml_abi_op_param_f32(n, 0), ggml_abi_op_param_f32(n, 1));
             c->st.kernel_launches++;
             return 1;
         }
         case GGML_OP_UNARY: {
-            if (fuse && n->op_params[0] == GGML_UNARY_OP_SIGMOID) { const int r = try_fuse_router_sigmoid(st, i); if (r) return r; }
+            if (fuse && n->op_params[0] == GGML_UNARY_OP_SIGMOID) {
+                int r = try_fuse_router_sigmoid(st, i);
+                if (r == 0) r = try_fuse_expert_join(st, i);
+                if (r) return r;
+            }
             // SIGMOID(g) -> RESHAPE -> MUL(x, .) with ONE gate per row of x (a number per head): one pass
             if (fuse && n->op_params[0] == GGML_UNARY_OP_SIGMOID && next(1) && next(2) && !st.done[i + 1] && !st.done[i + 2]) {
                 const ggml_tensor * rs = next(1), * gm2 = next(2);
@@ -2715,13 +2950,14 @@ static int run_node(exec_state & st, int i) {
             return 1;
         }
         case GGML_OP_SSM_CONV: {
+            if (fuse) { const int r = try_fuse_conv_store(st, i); if (r) return r; }
             const int taps = n->op_params[0];
             if (n->op_params[2] == 1) {
                 timed_scope ts(c, "seq_conv", (double) ggml_abi_nbytes(n));
-                launch_seq_conv_store(s, TD(a), (float *) n->data, (const int32_t *) n->src[1]->data, (int) n->src[1]->ne[0], (const int32_t *) n->src[2]->data, (int) n->src[2]->ne[1], taps);
+                launch_seq_conv_store(s, TD(a), nullptr, (float *) n->data, (const int32_t *) n->src[1]->data, (int) n->src[1]->ne[0], (const int32_t *) n->src[2]->data, (int) n->src[2]->ne[1], taps);
             } else {
                 timed_scope ts(c, "seq_conv", (double) ggml_abi_nbytes(a) + (double) ggml_abi_nbytes(n));
-                launch_seq_conv(s, TD(a), (const float *) n->src[1]->data, n->src[4] ? (const float *) n->src[4]->data : nullptr, n->src[2] ? (const float *) n->src[2]->data : nullptr,
+                launch_seq_conv(s, TD(a), nullptr, (const float *) n->src[1]->data, n->src[4] ? (const float *) n->src[4]->data : nullptr, n->src[2] ? (const float *) n->src[2]->data : nullptr,
                                 n->src[3] ? (const int32_t *) n->src[3]->data : nullptr,
                                 n->src[3] ? (int) n->src[3]->ne[0] : 0, TD(n), taps, n->op_params[1]);
             }
@@ -2801,7 +3037,7 @@ static int run_node(exec_state & st, int i) {
             // the down projection of a mixture-of-experts block reads the same ids as its up projection: the per-expert column lists are made once
             // (valid only while nothing but element-wise nodes ran in between: they do not touch the scratch area)
             bool valid = st.moe_ids == ids && st.moe_node >= 0 && i - st.moe_node <= 6 && g->nodes[st.moe_node]->src[0]->ne[2] == a->ne[2];
-            for (int k = st.moe_node + 1; valid && k < i; ++k) valid = is_view_op(g->nodes[k]) || g->nodes[k]->op == GGML_OP_UNARY || g->nodes[k]->op == GGML_OP_SQR || (g->nodes[k]->op == GGML_OP_GLU && !is_quant(a->type));
+            for (int k = st.moe_node + 1; valid && k < i; ++k) valid = is_view_op(g->nodes[k]) || g->nodes[k]->op == GGML_OP_UNARY || g->nodes[k]->op == GGML_OP_SQR || g->nodes[k]->op == GGML_OP_MUL || (g->nodes[k]->op == GGML_OP_GLU && !is_quant(a->type));
             const size_t need = mul_mat_id_workspace_bytes(TD(a), TD(ids));
             void * ws = (c->ws && st.aux_off + need <= c->ws_size) ? (char *) c->ws + st.aux_off : nullptr;
             timed_scope ts(c, "mul_mat_id", (double) ggml_abi_nbytes(a) / (double) std::max<int64_t>(1, a->ne[2]) * (double) std::min<int64_t>(a->ne[2], ggml_abi_nelements(ids)));
@@ -3020,6 +3256,8 @@ static int run_node(exec_state & st, int i) {
         }
         case GGML_OP_ROPE: {
             if (fuse && n->op_params[3] == 2) {
+                const int r = try_fuse_qk_norm_store(st, i);
+                if (r > 0) return r;
                 timed_scope ts(c, "rope_rows", (double) ggml_abi_nbytes(n) * 2);
                 int used = try_fuse_latent_row_store(st, i);
                 if (used == 0) used = try_fuse_concat_rope(st, i);

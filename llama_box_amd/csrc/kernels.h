@@ -385,8 +385,12 @@ bool repack_q80_supported(int type, int64_t K, int64_t N, int64_t nb1);  // Q8_0
 void launch_repack_q80_panels(hipStream_t s, const void * src, void * dst, int64_t K, int64_t N, int64_t nb1);
 
 // ---- layers with state per sequence (seq.hip): short convolutions over a sequence's history and three recurrences over a matrix state per head
-void launch_seq_conv(hipStream_t s, const tdesc & x, const float * w, const float * bias, const float * state, const int32_t * hist, int hs, const tdesc & dst, int taps, int act);
-void launch_seq_conv_store(hipStream_t s, const tdesc & x, float * state, const int32_t * upd, int hs, const int32_t * info, int n_seqs, int taps);
+// in_bias (may be null): a row added to the batch's inputs (the state already holds such sums)
+void launch_seq_conv(hipStream_t s, const tdesc & x, const float * in_bias, const float * w, const float * bias, const float * state, const int32_t * hist, int hs, const tdesc & dst, int taps, int act);
+void launch_seq_conv_store(hipStream_t s, const tdesc & x, const float * in_bias, float * state, const int32_t * upd, int hs, const int32_t * info, int n_seqs, int taps);
+// both for a batch that holds ONE token of every sequence in it
+void launch_seq_conv_step(hipStream_t s, const tdesc & x, const float * in_bias, const float * w, const float * bias, float * state, const int32_t * hist, int hs, const int32_t * upd, int hs_upd,
+                          const int32_t * info, int n_seqs, const tdesc & dst, int taps, int act);
 struct seq_rec_args {
     tdesc q, k, v;             // [rows, T] f32 (rows contiguous): q / r, k and v of all heads
     tdesc g;                   // wkv6: w_pre [D H, T]; delta: (b_pre, a_pre) [2 H, T]; mlstm: (i_pre, f_pre) [2 H, T]; channel decay, linear: a_pre [DK H, T]; state space: dt_pre [H, T]
@@ -414,19 +418,32 @@ void launch_seq_recurrence(hipStream_t s, int kind, const seq_rec_args & a, int 
 void launch_router_softmax_topk(hipStream_t s, const tdesc & logits, const tdesc & probs, const tdesc & ids, const tdesc & wts /* [1, k, T] */, int k, int groups, int keep, float wscale);
 // UNARY(SIGMOID) over a router's logits, ADD of a correction, the descending ARGSORT of the sums, GET_ROWS of the k first SCORES, their SUM_ROWS, SCALE(1, bias) and DIV in one launch
 // (n <= 256 experts): ids gets the whole permutation, wts [1, k, T] the normalised scores
-void launch_router_sigmoid_topk(hipStream_t s, const tdesc & logits, const float * corr, const tdesc & ids, float * wts, int k, float sum_bias);
-// queries and keys behind their projections: RMS_NORM per head -> MUL(weight row) [-> MUL(one factor per token)] of q in place or to qd, RMS_NORM -> MUL of k and v as it is straight into
-// their cache rows (f32 / bf16 / f16) at idx[token]
+// (raw: the weights are the chosen scores as they are)
+void launch_router_sigmoid_topk(hipStream_t s, const tdesc & logits, const float * corr, const tdesc & ids, float * wts, int k, float sum_bias, bool raw);
+// queries and keys behind their projections: [RMS_NORM per head -> MUL(weight row)] [-> MUL(one factor per token)] [-> ROPE by a table of frequencies] [-> RMS_NORM] of q in place or to qd,
+// the same (without the factor) of k and v as it is straight into their cache rows (f32 / bf16 / f16) at idx[token]
 struct qk_norm_store_args {
-    const float * q; float * qd; const float * k; const float * v;  // q, qd [DK, H, T]; k [DK, G, T]; v [DV G, T], contiguous
-    const float * qw; const float * kw; const float * temp;          // temp: [T] or null
+    const float * q; float * qd; const float * k; const float * v;  // qd [DK, H, T] contiguous; q [DK, H, T], k [DK, G, T], v [DV G, T]: a token's heads contiguous
+    int64_t q_tok, k_tok, v_tok;                                     // floats from a token to the next
+    const float * qw; const float * kw; const float * temp;          // qw, kw null: no norm in front; temp: [T] or null
+    const int32_t * pos; const float * freq; float mag;              // rotation of the leading n_rot entries (0: none), pairs (i, i + n_rot / 2) or (neox 0) neighbours
+    int n_rot, neox, unit; float eps_unit;                           // unit: divided by the root mean square behind the rotation
     char * k_cache; char * v_cache;
     int64_t kc_nb1, vc_nb1;
     const int64_t * idx;
     float eps_q, eps_k;
     int H, G, DK, DV, k_type, v_type;
 };
+constexpr int QK_ROT_MAX_DK = 640;  // (head entries a wave parks in LDS between the steps)
 void launch_qk_norm_store(hipStream_t s, const qk_norm_store_args & a, int64_t n_tok);
+// MUL(rows [2 nc, R], one factor per row) -> SwiGLU of the two halves
+void launch_swiglu_scaled(hipStream_t s, const float * gu, const float * w, float * dst, int64_t nc, int64_t rows);
+// the end of an expert feed-forward: sum over the `top` rows of a token, + shared row x sigmoid(gate) (shared may be null); with w: -> RMS_NORM -> MUL(w) -> ADD(residual)
+void launch_expert_join(hipStream_t s, const float * rows, int top, const float * shared, const float * gate, float * d, int64_t n, int64_t n_tok, const float * w, const float * residual, float eps);
+// two normed branches blended (launch_rms_norm2_blend), the blend normed, weighted and added to a residual
+void launch_rms_norm2_blend_join(hipStream_t s, const float * l, const float * r, const float * wl, const float * wr, float a, float b, const float * w, const float * residual, float * d, int64_t n,
+                                 int64_t rows, float eps, float eps_join);
+void launch_softcap(hipStream_t s, const float * x, float * d, int64_t n, float by, float cap);  // cap * tanh(x * by)
 void launch_sum_rows(hipStream_t s, const tdesc & src, const tdesc & dst);
 void launch_swiglu_limited(hipStream_t s, const tdesc & a, const tdesc * b, const tdesc & dst, int swapped, float alpha, float limit);  // min(g, l) sigmoid(alpha min(g, l)) (clamp(u, -l, l) + 1)
 

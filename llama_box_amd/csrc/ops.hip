@@ -338,8 +338,9 @@ void launch_router_softmax_topk(hipStream_t s, const tdesc & logits, const tdesc
 
 // ------------------------------------------------------------------------------------------------ router: sigmoid scores, corrected choice, normalised weights
 // one workgroup per token, a thread per expert (n <= 256): UNARY(SIGMOID), ADD(correction), the descending ARGSORT of the sums (ranks by counting: the stable order of
-// k_argsort), GET_ROWS of the k first scores, SUM_ROWS (f64, as k_sum_rows), SCALE(1, bias) and DIV — the nodes' own results
-__global__ void __launch_bounds__(256) k_router_sigmoid_topk(const tdesc a, const float * __restrict__ corr, const tdesc ids, float * __restrict__ wts, const int k, const float sum_bias) {
+// k_argsort), GET_ROWS of the k first scores, SUM_ROWS (f64, as k_sum_rows), SCALE(1, bias) and DIV — the nodes' own results (raw: the scores themselves are the weights)
+__global__ void __launch_bounds__(256) k_router_sigmoid_topk(const tdesc a, const float * __restrict__ corr, const tdesc ids, float * __restrict__ wts, const int k, const float sum_bias,
+                                                             const int raw) {
     __shared__ float c[256], top[256];
     __shared__ float sum_sh;
     const int64_t t = blockIdx.x;
@@ -358,8 +359,12 @@ __global__ void __launch_bounds__(256) k_router_sigmoid_topk(const tdesc a, cons
             before += (u > v || (u == v && j < i)) ? 1 : 0;
         }
         ((int32_t *) (ids.data + t * ids.nb[1]))[before] = i;
-        if (before < k) top[before] = sc;
+        if (before < k) {
+            top[before] = sc;
+            if (raw) wts[t * k + before] = sc;
+        }
     }
+    if (raw) return;
     __syncthreads();
     if (i < 64) {
         double s = 0.0;
@@ -370,9 +375,9 @@ __global__ void __launch_bounds__(256) k_router_sigmoid_topk(const tdesc a, cons
     __syncthreads();
     if (i < k) wts[t * k + i] = top[i] / sum_sh;
 }
-void launch_router_sigmoid_topk(hipStream_t s, const tdesc & logits, const float * corr, const tdesc & ids, float * wts, int k, float sum_bias) {
+void launch_router_sigmoid_topk(hipStream_t s, const tdesc & logits, const float * corr, const tdesc & ids, float * wts, int k, float sum_bias, bool raw) {
     if (logits.ne[1] == 0) return;
-    hipLaunchKernelGGL(k_router_sigmoid_topk, dim3((unsigned) logits.ne[1]), dim3(256), 0, s, logits, corr, ids, wts, k, sum_bias);
+    hipLaunchKernelGGL(k_router_sigmoid_topk, dim3((unsigned) logits.ne[1]), dim3(256), 0, s, logits, corr, ids, wts, k, sum_bias, raw ? 1 : 0);
 }
 
 // ------------------------------------------------------------------------------------------------ SUM_ROWS
@@ -410,13 +415,13 @@ __global__ void __launch_bounds__(256) k_qk_norm_store(const qk_norm_store_args 
     const int j = (int) (row % per), DK = A.DK;
     if (j >= A.H + A.G) {
         const int g = j - A.H - A.G, DV = A.DV;
-        const float * x = A.v + (t * A.G + g) * DV;
+        const float * x = A.v + t * A.v_tok + (int64_t) g * DV;
         char * vrow = A.v_cache + A.idx[t] * A.vc_nb1;
         for (int i = lane; i < DV; i += 64) cache_put(vrow, A.v_type, (int64_t) g * DV + i, x[i]);
         return;
     }
     const bool is_q = j < A.H;
-    const float * x = is_q ? A.q + (t * A.H + j) * DK : A.k + (t * A.G + (j - A.H)) * DK;
+    const float * x = is_q ? A.q + t * A.q_tok + (int64_t) j * DK : A.k + t * A.k_tok + (int64_t) (j - A.H) * DK;
     double s = 0.0;
     for (int i = lane; i < DK; i += 64) s += (double) (x[i] * x[i]);
     for (int off = 32; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
@@ -439,10 +444,78 @@ __global__ void __launch_bounds__(256) k_qk_norm_store(const qk_norm_store_args 
         }
     }
 }
+// the same with a rotation among the steps: [norm, weight] [factor] -> rotation of the leading entries -> [norm without a weight].  The wave parks its row in LDS between the steps (a
+// rotation pair crosses lanes); the query's result may lie over the projection (the row is in LDS before any of it is written)
+__global__ void __launch_bounds__(256) k_qk_rot_store(const qk_norm_store_args A, const int64_t rows) {
+    __shared__ float park[4][QK_ROT_MAX_DK];
+    const int lane = threadIdx.x & 63, per = A.H + 2 * A.G;
+    const int64_t row = (int64_t) blockIdx.x * 4 + (threadIdx.x >> 6);
+    const bool live = row < rows;
+    const int64_t t = live ? row / per : 0;
+    const int j = live ? (int) (row % per) : 0, DK = A.DK, half = A.n_rot / 2;
+    const bool is_v = live && j >= A.H + A.G, is_q = j < A.H, head = live && !is_v;
+    float * buf = park[threadIdx.x >> 6];
+    if (is_v) {
+        const int g = j - A.H - A.G, DV = A.DV;
+        const float * x = A.v + t * A.v_tok + (int64_t) g * DV;
+        char * vrow = A.v_cache + A.idx[t] * A.vc_nb1;
+        for (int i = lane; i < DV; i += 64) cache_put(vrow, A.v_type, (int64_t) g * DV + i, x[i]);
+    }
+    if (head) {
+        const float * x = is_q ? A.q + t * A.q_tok + (int64_t) j * DK : A.k + t * A.k_tok + (int64_t) (j - A.H) * DK;
+        const float * w = is_q ? A.qw : A.kw;
+        float scale = 1.0f;
+        if (w) {
+            double s = 0.0;
+            for (int i = lane; i < DK; i += 64) s += (double) (x[i] * x[i]);
+            for (int off = 32; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
+            scale = 1.0f / sqrtf((float) (s / (double) DK) + (is_q ? A.eps_q : A.eps_k));
+        }
+        const bool tmp = is_q && A.temp;
+        const float f = tmp ? A.temp[t] : 1.0f;
+        for (int i = lane; i < DK; i += 64) {
+            float v = x[i];
+            if (w) {
+                v = v * scale;
+                v = v * w[i];
+            }
+            buf[i] = tmp ? v * f : v;
+        }
+    }
+    __syncthreads();
+    if (head) {
+        const float pos_f = (float) A.pos[t];
+        for (int ip = lane; ip < half; ip += 64) {
+            const int ia = A.neox ? ip : 2 * ip, ib = A.neox ? ip + half : 2 * ip + 1;
+            const float x0 = buf[ia], x1 = buf[ib];
+            float cs, sn;
+            rope_cos_sin_table(ip, pos_f, A.freq, A.mag, cs, sn);
+            buf[ia] = x0 * cs - x1 * sn;
+            buf[ib] = x0 * sn + x1 * cs;
+        }
+    }
+    __syncthreads();
+    if (!head) return;
+    float scale = 1.0f;
+    if (A.unit) {
+        double s = 0.0;
+        for (int i = lane; i < DK; i += 64) s += (double) (buf[i] * buf[i]);
+        for (int off = 32; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
+        scale = 1.0f / sqrtf((float) (s / (double) DK) + A.eps_unit);
+    }
+    float * y = A.qd + (t * A.H + j) * DK;
+    char * krow = A.k_cache + A.idx[t] * A.kc_nb1;
+    for (int i = lane; i < DK; i += 64) {
+        const float v = A.unit ? buf[i] * scale : buf[i];
+        if (is_q) y[i] = v;
+        else cache_put(krow, A.k_type, (int64_t) (j - A.H) * DK + i, v);
+    }
+}
 void launch_qk_norm_store(hipStream_t s, const qk_norm_store_args & a, int64_t n_tok) {
     const int64_t rows = n_tok * (a.H + 2 * a.G);
     if (rows == 0) return;
-    hipLaunchKernelGGL(k_qk_norm_store, dim3((unsigned) ((rows + 3) / 4)), dim3(256), 0, s, a, rows);
+    if (a.n_rot > 0 || a.unit) hipLaunchKernelGGL(k_qk_rot_store, dim3((unsigned) ((rows + 3) / 4)), dim3(256), 0, s, a, rows);
+    else hipLaunchKernelGGL(k_qk_norm_store, dim3((unsigned) ((rows + 3) / 4)), dim3(256), 0, s, a, rows);
 }
 
 // ------------------------------------------------------------------------------------------------ residual sum and the RMS norm of the next sublayer
@@ -669,6 +742,161 @@ void launch_rms_norm2_blend(hipStream_t s, const float * l, const float * r, con
     if (rows == 0 || n == 0) return;
     hipLaunchKernelGGL(k_rms_norm2_blend, dim3((unsigned) rows), dim3(256), 0, s, l, r, wl, wr, a, b, d, n, eps);
 }
+
+// ------------------------------------------------------------------------------------------------ a normed row joining the stream, the row made on the way
+// d = rms_norm(row) * w + residual for a row that no earlier launch has written: `F` gives its entries (four neighbours at `v4(i)`, one at `v1(i)`).  A workgroup of 256 per row.
+// VEC (16-byte aligned rows of up to 8192 entries, whole groups of four): the row is made once and kept in registers; else it is made again for the second pass.  The sum of squares is
+// f64 as in k_rms_norm.  A thread has made (read) every entry it writes before it writes it, and reads nothing that another thread writes.
+constexpr int ROW_JOIN_MAX_VEC = 8192;
+template <bool VEC, typename F>
+__device__ __forceinline__ void row_norm_join(const F & f, const int64_t n, const float * __restrict__ w, const float * res, float * out, const float eps, double * sh) {
+    double s = 0.0;
+    if constexpr (VEC) {
+        const int n4 = (int) (n >> 2);
+        float4 r[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int i = threadIdx.x + 256 * u;
+            r[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (i < n4) r[u] = f.v4(i);
+            s += (double) (r[u].x * r[u].x) + (double) (r[u].y * r[u].y) + (double) (r[u].z * r[u].z) + (double) (r[u].w * r[u].w);
+        }
+        s = block_sum_d(s, sh);
+        const float scale = 1.0f / sqrtf((float) (s / (double) n) + eps);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int i = threadIdx.x + 256 * u;
+            if (i >= n4) continue;
+            const float4 g = ((const float4 *) w)[i], e = ((const float4 *) res)[i];
+            float4 v = make_float4(r[u].x * scale, r[u].y * scale, r[u].z * scale, r[u].w * scale);
+            v = make_float4(v.x * g.x, v.y * g.y, v.z * g.z, v.w * g.w);
+            ((float4 *) out)[i] = make_float4(v.x + e.x, v.y + e.y, v.z + e.z, v.w + e.w);
+        }
+    } else {
+        for (int64_t i = threadIdx.x; i < n; i += 256) {
+            const float v = f.v1(i);
+            s += (double) (v * v);
+        }
+        s = block_sum_d(s, sh);
+        const float scale = 1.0f / sqrtf((float) (s / (double) n) + eps);
+        for (int64_t i = threadIdx.x; i < n; i += 256) {
+            float v = f.v1(i) * scale;
+            v = v * w[i];
+            out[i] = v + res[i];
+        }
+    }
+}
+__device__ __forceinline__ float4 f4_add(const float4 a, const float4 b) { return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w); }
+// the sum over a token's expert rows, in their order, plus the shared expert's row times its gate
+struct expert_row {
+    const float * rows;
+    const float * shared;
+    int64_t n;
+    int top;
+    float gate;
+    __device__ __forceinline__ float4 v4(const int i) const {
+        float4 a = ((const float4 *) rows)[i];
+        for (int u = 1; u < top; ++u) a = f4_add(a, ((const float4 *) (rows + u * n))[i]);
+        if (shared) {
+            const float4 s = ((const float4 *) shared)[i];
+            a = f4_add(a, make_float4(s.x * gate, s.y * gate, s.z * gate, s.w * gate));
+        }
+        return a;
+    }
+    __device__ __forceinline__ float v1(const int64_t i) const {
+        float a = rows[i];
+        for (int u = 1; u < top; ++u) a = a + rows[u * n + i];
+        if (shared) {
+            const float p = shared[i] * gate;
+            a = a + p;
+        }
+        return a;
+    }
+};
+template <bool VEC>
+__global__ void __launch_bounds__(256) k_expert_join(const float * rows, const int top, const float * shared, const float * __restrict__ gate, float * d, const int64_t n, const float * __restrict__ w,
+                                                     const float * res, const float eps) {
+    __shared__ double sh[4];
+    const int64_t t = blockIdx.x;
+    const expert_row f{rows + t * top * n, shared ? shared + t * n : nullptr, n, top, shared ? 1.f / (1.f + expf(-gate[t])) : 0.0f};
+    if (w) {
+        row_norm_join<VEC>(f, n, w, res + t * n, d + t * n, eps, sh);
+        return;
+    }
+    for (int64_t i = threadIdx.x; i < n; i += 256) d[t * n + i] = f.v1(i);
+}
+static bool join_vec_ok(int64_t n, std::initializer_list<const void *> ps) {
+    uintptr_t a = 0;
+    for (const void * p : ps) a |= (uintptr_t) p;
+    return (n % 4) == 0 && n <= ROW_JOIN_MAX_VEC && (a & 15) == 0;
+}
+void launch_expert_join(hipStream_t s, const float * rows, int top, const float * shared, const float * gate, float * d, int64_t n, int64_t n_tok, const float * w, const float * residual, float eps) {
+    if (n_tok == 0 || n == 0) return;
+    if (join_vec_ok(n, {rows, shared, d, w, residual})) hipLaunchKernelGGL(k_expert_join<true>, dim3((unsigned) n_tok), dim3(256), 0, s, rows, top, shared, gate, d, n, w, residual, eps);
+    else hipLaunchKernelGGL(k_expert_join<false>, dim3((unsigned) n_tok), dim3(256), 0, s, rows, top, shared, gate, d, n, w, residual, eps);
+}
+// a * (l * sl) * wl + b * (r * sr) * wr: two normed branches blended (k_rms_norm2_blend's entries)
+struct blend_row {
+    const float * l; const float * r; const float * wl; const float * wr;
+    float sl, sr, a, b;
+    __device__ __forceinline__ float one(const float x, const float y, const float gl, const float gr) const {
+        float v = x * sl, q = y * sr;
+        v = v * gl;
+        q = q * gr;
+        const float pa = v * a, pb = q * b;
+        return pa + pb;
+    }
+    __device__ __forceinline__ float4 v4(const int i) const {
+        const float4 x = ((const float4 *) l)[i], y = ((const float4 *) r)[i], gl = ((const float4 *) wl)[i], gr = ((const float4 *) wr)[i];
+        return make_float4(one(x.x, y.x, gl.x, gr.x), one(x.y, y.y, gl.y, gr.y), one(x.z, y.z, gl.z, gr.z), one(x.w, y.w, gl.w, gr.w));
+    }
+    __device__ __forceinline__ float v1(const int64_t i) const { return one(l[i], r[i], wl[i], wr[i]); }
+};
+template <bool VEC>
+__global__ void __launch_bounds__(256) k_rms_norm2_blend_join(const float * l, const float * r, const float * __restrict__ wl, const float * __restrict__ wr, const float a, const float b,
+                                                              const float * __restrict__ w, const float * res, float * d, const int64_t n, const float eps, const float eps_join) {
+    __shared__ double sh[4];
+    const int64_t row = blockIdx.x;
+    const float * x = l + row * n, * y = r + row * n;
+    double s = 0.0, u = 0.0;
+    if constexpr (VEC) {
+        for (int i = threadIdx.x; i < (int) (n >> 2); i += 256) {
+            const float4 v = ((const float4 *) x)[i], q = ((const float4 *) y)[i];
+            s += (double) (v.x * v.x) + (double) (v.y * v.y) + (double) (v.z * v.z) + (double) (v.w * v.w);
+            u += (double) (q.x * q.x) + (double) (q.y * q.y) + (double) (q.z * q.z) + (double) (q.w * q.w);
+        }
+    } else {
+        for (int64_t i = threadIdx.x; i < n; i += 256) {
+            const float v = x[i], q = y[i];
+            s += (double) (v * v);
+            u += (double) (q * q);
+        }
+    }
+    s = block_sum_d(s, sh);
+    __syncthreads();
+    u = block_sum_d(u, sh);
+    __syncthreads();
+    const blend_row f{x, y, wl, wr, 1.0f / sqrtf((float) (s / (double) n) + eps), 1.0f / sqrtf((float) (u / (double) n) + eps), a, b};
+    row_norm_join<VEC>(f, n, w, res + row * n, d + row * n, eps_join, sh);
+}
+void launch_rms_norm2_blend_join(hipStream_t s, const float * l, const float * r, const float * wl, const float * wr, float a, float b, const float * w, const float * residual, float * d, int64_t n,
+                                 int64_t rows, float eps, float eps_join) {
+    if (rows == 0 || n == 0) return;
+    if (join_vec_ok(n, {l, r, wl, wr, w, residual, d})) hipLaunchKernelGGL(k_rms_norm2_blend_join<true>, dim3((unsigned) rows), dim3(256), 0, s, l, r, wl, wr, a, b, w, residual, d, n, eps, eps_join);
+    else hipLaunchKernelGGL(k_rms_norm2_blend_join<false>, dim3((unsigned) rows), dim3(256), 0, s, l, r, wl, wr, a, b, w, residual, d, n, eps, eps_join);
+}
+// SCALE(by) -> TANH -> SCALE(cap)
+__global__ void __launch_bounds__(256) k_softcap(const float * x, float * d, const int64_t n, const float by, const float cap) {
+    for (int64_t i = (int64_t) blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t) gridDim.x * 256) {
+        const float z = x[i] * by;
+        d[i] = tanhf(z) * cap;
+    }
+}
+void launch_softcap(hipStream_t s, const float * x, float * d, int64_t n, float by, float cap) {
+    if (n == 0) return;
+    hipLaunchKernelGGL(k_softcap, dim3((unsigned) std::min<int64_t>((n + 255) / 256, 4096)), dim3(256), 0, s, x, d, n, by, cap);
+}
+
 __global__ void __launch_bounds__(256) k_weighted_rows_sum(const tdesc rows, const tdesc w, const tdesc d) {
     const int64_t t = blockIdx.x, n_used = rows.ne[1];
     const float * __restrict__ wt = (const float *) (w.data + t * w.nb[2]);
@@ -817,6 +1045,32 @@ void launch_swiglu(hipStream_t s, const tdesc & a, const tdesc * b, const tdesc 
     const dim3 grid((unsigned) rows, (unsigned) ((nc + 1023) / 1024));
     if (vec) hipLaunchKernelGGL(k_swiglu<true>, grid, dim3(256), 0, s, pa, pb, d.data, nc, a.nb[1], nbb1, d.nb[1]);
     else hipLaunchKernelGGL(k_swiglu<false>, grid, dim3(256), 0, s, pa, pb, d.data, nc, a.nb[1], nbb1, d.nb[1]);
+}
+
+// SwiGLU of the two halves of rows that carry one factor each (the factor multiplies both halves first: experts whose weight multiplies their input)
+template <bool VEC>
+__global__ void __launch_bounds__(256) k_swiglu_scaled(const float * __restrict__ gu, const float * __restrict__ w, float * __restrict__ d, const int64_t nc) {
+    const int64_t row = blockIdx.x, i0 = ((int64_t) blockIdx.y * 256 + threadIdx.x) * 4;
+    const float * a = gu + row * 2 * nc;
+    const float f = w[row];
+    auto one = [&](const float g, const float u) {
+        const float gs = g * f, us = u * f;
+        return silu_f(gs) * us;
+    };
+    if constexpr (VEC) {
+        if (i0 < nc) {
+            const float4 g = *(const float4 *) (a + i0), u = *(const float4 *) (a + nc + i0);
+            *(float4 *) (d + row * nc + i0) = make_float4(one(g.x, u.x), one(g.y, u.y), one(g.z, u.z), one(g.w, u.w));
+        }
+    } else {
+        for (int64_t i = i0; i < i0 + 4 && i < nc; ++i) d[row * nc + i] = one(a[i], a[nc + i]);
+    }
+}
+void launch_swiglu_scaled(hipStream_t s, const float * gu, const float * w, float * dst, int64_t nc, int64_t rows) {
+    if (rows == 0 || nc == 0) return;
+    const dim3 grid((unsigned) rows, (unsigned) ((nc + 1023) / 1024));
+    if ((nc % 4) == 0 && (((uintptr_t) gu | (uintptr_t) dst) & 15) == 0) hipLaunchKernelGGL(k_swiglu_scaled<true>, grid, dim3(256), 0, s, gu, w, dst, nc);
+    else hipLaunchKernelGGL(k_swiglu_scaled<false>, grid, dim3(256), 0, s, gu, w, dst, nc);
 }
 
 // a gated activation with limits (ggml_swiglu_oai): g = min(a, limit), u = clamp(b, -limit, limit); y = g / (1 + exp(-alpha g)) * (u + 1)

@@ -10,6 +10,7 @@
 // Kernels:
 //   k_seq_conv        short causal convolution per channel over a sequence's history (taps inputs, the last one the token's own), optionally followed by SiLU;
 //                     several weight sets over the same input give several outputs (a token shift h + (h_prev - h) mu is the 2-tap case with weights (mu, 1 - mu))
+//   k_seq_conv_step   both at once for a batch of one token per sequence
 //   k_seq_conv_store  the last taps - 1 inputs of every sequence of the batch become its state
 //   k_seq_recurrence<SEQ_WKV6>   o_t = (S + diag(u) k v^T)^T r;  S <- diag(w) S + k v^T, w = exp(-exp(w_pre + w0)) per key channel
 //   k_seq_recurrence<SEQ_DELTA>  gated delta rule: S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q — unit-length q, k, sigmoid beta and the decay
@@ -37,8 +38,8 @@ constexpr int SEQ_MAX_TAPS = 16;
 constexpr int SEQ_MAX_DK = 256;  // key rows of a head (16 lanes x up to 16 rows each)
 
 __device__ __forceinline__ float seq_hist_value(const int code, const int c, const int64_t C, const int taps, const char * __restrict__ xdata, const int64_t x_nb1,
-                                                const float * __restrict__ state) {
-    if (code >= 0) return ((const float *) (xdata + (int64_t) code * x_nb1))[c];
+                                                const float * __restrict__ state, const float in_bias) {
+    if (code >= 0) return ((const float *) (xdata + (int64_t) code * x_nb1))[c] + in_bias;
     if (code == -1) return 0.0f;
     const int cd = -2 - code, slot = cd >> 6, age = cd & 63;
     return state[((int64_t) slot * (taps - 1) + age) * C + c];
@@ -46,16 +47,8 @@ __device__ __forceinline__ float seq_hist_value(const int code, const int c, con
 
 __device__ __forceinline__ float seq_silu(const float z) { return z / (1.0f + expf(-z)); }
 
-// y[c, t, m] = act(sum_j w[j, c, m] * x_(t - (taps - 1 - j))[c] + bias[c, m])   (bias may be null)
-__global__ void __launch_bounds__(256) k_seq_conv(const tdesc x, const float * __restrict__ w, const float * __restrict__ bias, const float * __restrict__ state,
-                                                  const int32_t * __restrict__ hist, const int hs, const tdesc dst, const int taps, const int act) {
-    const int64_t C = x.ne[0], t = blockIdx.y;
-    const int c = blockIdx.x * 256 + threadIdx.x;
-    if (c >= C) return;
-    float xv[SEQ_MAX_TAPS];  // xv[d]: the input d tokens back
-    xv[0] = ((const float *) (x.data + t * x.nb[1]))[c];
-#pragma unroll
-    for (int d = 1; d < SEQ_MAX_TAPS; ++d) xv[d] = d < taps ? seq_hist_value(hist[t * hs + d - 1], c, C, taps, x.data, x.nb[1], state) : 0.0f;
+__device__ __forceinline__ void seq_conv_outputs(const float (&xv)[SEQ_MAX_TAPS], const float * __restrict__ w, const float * __restrict__ bias, const tdesc & dst, const int64_t t, const int c,
+                                                 const int64_t C, const int taps, const int act) {
     for (int64_t m = 0; m < dst.ne[2]; ++m) {
         const float * __restrict__ wc = w + (m * C + c) * taps;
         float y = 0.0f;
@@ -67,27 +60,67 @@ __global__ void __launch_bounds__(256) k_seq_conv(const tdesc x, const float * _
     }
 }
 
-__global__ void __launch_bounds__(256) k_seq_conv_store(const tdesc x, float * __restrict__ state, const int32_t * __restrict__ upd, const int hs, const int32_t * __restrict__ info,
-                                                        const int taps) {
+// y[c, t, m] = act(sum_j w[j, c, m] * x_(t - (taps - 1 - j))[c] + bias[c, m])   (bias may be null)
+__global__ void __launch_bounds__(256) k_seq_conv(const tdesc x, const float * __restrict__ in_bias, const float * __restrict__ w, const float * __restrict__ bias, const float * __restrict__ state,
+                                                  const int32_t * __restrict__ hist, const int hs, const tdesc dst, const int taps, const int act) {
+    const int64_t C = x.ne[0], t = blockIdx.y;
+    const int c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= C) return;
+    const float ib = in_bias ? in_bias[c] : 0.0f;
+    float xv[SEQ_MAX_TAPS];  // xv[d]: the input d tokens back
+    xv[0] = ((const float *) (x.data + t * x.nb[1]))[c] + ib;
+#pragma unroll
+    for (int d = 1; d < SEQ_MAX_TAPS; ++d) xv[d] = d < taps ? seq_hist_value(hist[t * hs + d - 1], c, C, taps, x.data, x.nb[1], state, ib) : 0.0f;
+    seq_conv_outputs(xv, w, bias, dst, t, c, C, taps, act);
+}
+
+// a batch of ONE token per sequence: the convolution and the state's update in one pass — a thread has read its channel's whole history of the sequence before it writes any of it, and
+// no other thread touches that history
+__global__ void __launch_bounds__(256) k_seq_conv_step(const tdesc x, const float * __restrict__ in_bias, const float * __restrict__ w, const float * __restrict__ bias, float * state,
+                                                       const int32_t * __restrict__ hist, const int hs, const int32_t * __restrict__ upd, const int hs_upd, const int32_t * __restrict__ info,
+                                                       const tdesc dst, const int taps, const int act) {
+    const int64_t C = x.ne[0], s = blockIdx.y, t = upd[s * hs_upd];  // (the newest input of the sequence after the batch: its token's row)
+    const int c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= C || t < 0 || t >= x.ne[1]) return;
+    const int slot = info[4 * s + 2];
+    const float ib = in_bias ? in_bias[c] : 0.0f;
+    float xv[SEQ_MAX_TAPS];
+    xv[0] = ((const float *) (x.data + t * x.nb[1]))[c] + ib;
+#pragma unroll
+    for (int d = 1; d < SEQ_MAX_TAPS; ++d) xv[d] = d < taps ? seq_hist_value(hist[t * hs + d - 1], c, C, taps, x.data, x.nb[1], state, ib) : 0.0f;
+    seq_conv_outputs(xv, w, bias, dst, t, c, C, taps, act);
+#pragma unroll
+    for (int a = 0; a < SEQ_MAX_TAPS - 1; ++a)
+        if (a < taps - 1) state[((int64_t) slot * (taps - 1) + a) * C + c] = xv[a];
+}
+
+__global__ void __launch_bounds__(256) k_seq_conv_store(const tdesc x, const float * __restrict__ in_bias, float * __restrict__ state, const int32_t * __restrict__ upd, const int hs,
+                                                        const int32_t * __restrict__ info, const int taps) {
     const int64_t C = x.ne[0], s = blockIdx.y;
     const int c = blockIdx.x * 256 + threadIdx.x;
     if (c >= C) return;
     const int slot = info[4 * s + 2];
+    const float ib = in_bias ? in_bias[c] : 0.0f;
     float nv[SEQ_MAX_TAPS - 1];
 #pragma unroll
-    for (int a = 0; a < SEQ_MAX_TAPS - 1; ++a) nv[a] = a < taps - 1 ? seq_hist_value(upd[s * hs + a], c, C, taps, x.data, x.nb[1], state) : 0.0f;
+    for (int a = 0; a < SEQ_MAX_TAPS - 1; ++a) nv[a] = a < taps - 1 ? seq_hist_value(upd[s * hs + a], c, C, taps, x.data, x.nb[1], state, ib) : 0.0f;
 #pragma unroll
     for (int a = 0; a < SEQ_MAX_TAPS - 1; ++a)
         if (a < taps - 1) state[((int64_t) slot * (taps - 1) + a) * C + c] = nv[a];  // (every value was read before the first is written: the rows shift in place)
 }
 
-void launch_seq_conv(hipStream_t s, const tdesc & x, const float * w, const float * bias, const float * state, const int32_t * hist, int hs, const tdesc & dst, int taps, int act) {
+void launch_seq_conv(hipStream_t s, const tdesc & x, const float * in_bias, const float * w, const float * bias, const float * state, const int32_t * hist, int hs, const tdesc & dst, int taps, int act) {
     if (x.ne[1] == 0 || x.ne[0] == 0) return;
-    hipLaunchKernelGGL(k_seq_conv, dim3((unsigned) ((x.ne[0] + 255) / 256), (unsigned) x.ne[1]), dim3(256), 0, s, x, w, bias, state, hist, hs, dst, taps, act);
+    hipLaunchKernelGGL(k_seq_conv, dim3((unsigned) ((x.ne[0] + 255) / 256), (unsigned) x.ne[1]), dim3(256), 0, s, x, in_bias, w, bias, state, hist, hs, dst, taps, act);
 }
-void launch_seq_conv_store(hipStream_t s, const tdesc & x, float * state, const int32_t * upd, int hs, const int32_t * info, int n_seqs, int taps) {
+void launch_seq_conv_store(hipStream_t s, const tdesc & x, const float * in_bias, float * state, const int32_t * upd, int hs, const int32_t * info, int n_seqs, int taps) {
     if (n_seqs == 0 || x.ne[0] == 0 || taps < 2) return;
-    hipLaunchKernelGGL(k_seq_conv_store, dim3((unsigned) ((x.ne[0] + 255) / 256), (unsigned) n_seqs), dim3(256), 0, s, x, state, upd, hs, info, taps);
+    hipLaunchKernelGGL(k_seq_conv_store, dim3((unsigned) ((x.ne[0] + 255) / 256), (unsigned) n_seqs), dim3(256), 0, s, x, in_bias, state, upd, hs, info, taps);
+}
+void launch_seq_conv_step(hipStream_t s, const tdesc & x, const float * in_bias, const float * w, const float * bias, float * state, const int32_t * hist, int hs, const int32_t * upd, int hs_upd,
+                          const int32_t * info, int n_seqs, const tdesc & dst, int taps, int act) {
+    if (n_seqs == 0 || x.ne[0] == 0 || taps < 2) return;
+    hipLaunchKernelGGL(k_seq_conv_step, dim3((unsigned) ((x.ne[0] + 255) / 256), (unsigned) n_seqs), dim3(256), 0, s, x, in_bias, w, bias, state, hist, hs, upd, hs_upd, info, dst, taps, act);
 }
 
 // ------------------------------------------------------------------------------------------------ the recurrences
