@@ -250,6 +250,42 @@ def pisulorn_config(z):
             "residual_mult": 0.5, "streams": z["streams"], "vocab": z["vocab"], "width": z["width"]}
 
 
+# ------------------------------------------------------------------------------------------------ --nidudra: norms on the sublayers' outputs; rotated attention with a sink, windowed attention
+# over its own or an earlier layer's cache, attention over convolved keys beside gated linear attention; dense and expert feed-forwards; beside Pisulorn (experts, windowed attention, a recurrence)
+# and Nogavik (attention beside a recurrence with one decay per key channel) at equal size
+NIDUDRA_SIZES = {
+    # width, heads, kv heads, head size, window, kept first tokens, taps, inner size of the decay's matrices, dense ff (gated: three matrices), experts, top, expert ff (gated), ff of the shared
+    # expert, vocab.  Six layers (rotated + dense, parallel + experts, windowed + dense, windowed over the third layer's cache + experts, rotated + experts, parallel + experts), as many as the
+    # models beside it have layer runs; a token's experts and the shared one together stream what Pisulorn's two experts do
+    "s": dict(width=1024, heads=8, kv=2, hd=64, window=512, keep=4, taps=4, low=64, ff=2752, experts=8, top=2, eff=704, shared=640, vocab=32000),
+    "m": dict(width=2048, heads=16, kv=4, hd=128, window=1024, keep=4, taps=4, low=128, ff=5504, experts=8, top=2, eff=1376, shared=1344, vocab=32000),
+    "l": dict(width=4096, heads=32, kv=8, hd=128, window=2048, keep=4, taps=4, low=128, ff=9600, experts=8, top=2, eff=2752, shared=2688, vocab=32000),
+}
+
+
+def nidudra_config(z):
+    H, G, D = z["heads"], z["kv"], z["hd"]
+    dense = {"kind": "dense", "ff": z["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": z["eff"]}, "router": {"experts": z["experts"], "top": z["top"]}, "shared": {"ff": z["shared"]}}
+    head = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5}
+
+    def rotated(mlp):
+        return {"type": "attention_2", "mlp": mlp, "mixer": dict(head, rot={"base": 5e5, "dims": D, "scaling": {"factor": 8.0, "high": 4.0, "low": 1.0, "original": 8192}})}
+
+    def windowed(mlp, kv_from=None):
+        mx = dict(head, mask={"size": z["window"], "keep_first": z["keep"]})
+        if kv_from is not None:
+            mx["kv_from"] = kv_from
+        return {"type": "attention", "mlp": mlp, "mixer": mx}
+
+    def parallel(mlp):
+        left = dict(head, conv=z["taps"], rot={"base": 1e6, "dims": D, "scaling": {"factor": 4.0, "fast": 32.0, "slow": 1.0, "original": 8192}})
+        return {"type": "parallel", "mlp": mlp, "mixer": {"left": left, "right": {"heads": H, "dim": D, "vdim": D, "tau": 16.0, "rank": z["low"]}}}
+
+    return {"architecture": "Nidudra", "layers": [rotated(dense), parallel(moe), windowed(dense), windowed(moe, 2), rotated(moe), parallel(moe)], "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "vocab": z["vocab"], "width": z["width"]}
+
+
 def bench_nigozen(args):
     """Prefill and decode throughput of Nigozen models (bf16 matrices, bf16 cache, random weights) at sizes that resemble real layers, beside the
     closest existing class at equal size: llama with f16 matrices and an f16 cache (same width, layers, heads, head size, dense ff and vocabulary;
@@ -265,7 +301,7 @@ def bench_nigozen(args):
 
     be = L.Backend(0)
     n_prompt, n_dec, ub = args.prefill, max(8, min(args.steps, 64)), args.ubatch
-    many_sided = bool(args.zigipel or args.rarelorn or args.nogavik or args.pisulorn)
+    many_sided = bool(args.zigipel or args.rarelorn or args.nogavik or args.pisulorn or args.nidudra)
     if many_sided and n_prompt == 2048:
         # decoded positions 1984 .. 2047: a model confined to chunks of 512 / 1024 / 2048 positions then sees 449 .. 512 / 961 .. 1024 / 1985 .. 2048 cells, about as many as a
         # sliding window of the same length does (right behind a chunk's start it would see next to nothing, and the two decode steps would not compare)
@@ -315,6 +351,26 @@ def bench_nigozen(args):
         ctx.free()
         return res
 
+    if args.nidudra:  # Nidudra beside Pisulorn (experts, windowed attention) and Nogavik (attention beside a recurrence with channel decay): as many layer runs, equal width, heads, head size, vocabulary
+        out["metric"] = "nidudra_vs_pisulorn_tokens_per_s"
+        out["dtype"] = "bf16 (all)"
+        be.close()
+        for name in args.nidudra.split(","):
+            res = {}
+            for side, cfg in (("nidudra", nidudra_config(NIDUDRA_SIZES[name])), ("pisulorn", pisulorn_config(PISULORN_SIZES[name])), ("nogavik", nogavik_config(NOGAVIK_SIZES[name]))):
+                be = L.Backend(0)
+                mdl = Model(config_json=_json.dumps(cfg), seed=7, buft=be.buft, wtype=L.BF16)
+                res[side] = run(mdl, NIDUDRA_SIZES[name]["vocab"])
+                res[side]["weight_bytes"] = int(L.host().llm_model_total_bytes(mdl.m))
+                res[side]["stream_bytes_per_token"] = mdl.stream_bytes()
+                mdl.free()
+                be.close()
+            out["sizes"][name] = {"config": NIDUDRA_SIZES[name], **res}
+            for other in ("pisulorn", "nogavik"):
+                out["sizes"][name]["prefill_ratio_" + other] = round(res["nidudra"]["prefill_tok_s"] / res[other]["prefill_tok_s"], 3)
+                out["sizes"][name]["decode_ratio_" + other] = round(res["nidudra"]["decode_tok_s"] / res[other]["decode_tok_s"], 3)
+        print(_json.dumps(out))
+        return
     if args.pisulorn:  # Pisulorn beside Rarelorn (its delta rule and experts) and Zigipel (its windowed attention): as many layer runs, equal width, heads, head size, vocabulary and parameters
         out["metric"] = "pisulorn_vs_rarelorn_tokens_per_s"
         out["dtype"] = "bf16 (all)"
@@ -430,6 +486,8 @@ def main():
     ap.add_argument("--nogavik", default="", help="comma-separated sizes (s, m, l): time prefill and decode of Nogavik models (latent attention with shared cache rows, a state-space "
                     "mixer, attention beside a delta rule with channel decay, a per-layer token input) beside Zigipel and Rarelorn models of equal size, print one JSON line and exit; "
                     "the default workload is not run")
+    ap.add_argument("--nidudra", default="", help="comma-separated sizes (s, m, l): time prefill and decode of Nidudra models (norms behind the sublayers, rotated attention with a sink, windowed "
+                    "attention over an own or an earlier layer's cache, attention beside gated linear attention, experts with a shared one) beside Pisulorn and Nogavik models of equal size instead of the default workload")
     ap.add_argument("--pisulorn", default="", help="comma-separated sizes (s, m, l): time prefill and decode of Pisulorn models (several residual streams, windowed attention with a linear "
                     "distance penalty, a gated delta rule, dense and expert feed-forwards, a repeated range) beside Rarelorn and Zigipel models of equal size, print one JSON line and exit; "
                     "the default workload is not run")
@@ -461,7 +519,7 @@ def main():
     ap.add_argument("--pmc-traffic", type=int, default=1, help="1: re-run a short decode under rocprofv3 --pmc FETCH_SIZE (own pass) for roofline.traffic")
     args = ap.parse_args()
 
-    if args.nigozen or args.zigipel or args.rarelorn or args.nogavik or args.pisulorn:
+    if args.nigozen or args.zigipel or args.rarelorn or args.nogavik or args.pisulorn or args.nidudra:
         bench_nigozen(args)
         return
 
