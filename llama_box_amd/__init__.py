@@ -172,6 +172,7 @@ _SIGS = {
     "ggml_seq_wkv6": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, TP, TP, _I]), "ggml_seq_gated_delta": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, TP, _I, _I]),
     "ggml_seq_mlstm": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, TP, _I, _F]), "ggml_seq_state_size": (C.c_int64, [_I, _I, _I, _I]),
     "ggml_seq_delta_channel": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, TP, TP, _I, _I]), "ggml_seq_ssd": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, TP, _I, _I]),
+    "ggml_seq_linear": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, TP, _I, C.c_float]),
     "ggml_seq_conv_set_bias": (None, [TP, TP]),
     "ggml_flash_attn_ext_add_linear_distance": (None, [TP, TP]), "ggml_swiglu_oai": (TP, [_P, TP, TP, _F, _F]), "ggml_sum_rows": (TP, [_P, TP]),
     "ggml_stream_step": (TP, [_P, TP, TP, TP, TP, TP, TP, TP, _I, _I, _F, _F]), "ggml_stream_step_rows": (TP, [_P, TP]), "ggml_stream_step_streams": (TP, [_P, TP]),

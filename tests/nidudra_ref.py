@@ -18,8 +18,9 @@ def over_rms(x, eps):
 
 
 def squash(z):
-    """the logistic function"""
-    return 0.5 * (1.0 + np.tanh(0.5 * z))
+    """the logistic function, exact in relative terms on both sides (a decay is a root of it)"""
+    e = np.exp(-np.abs(z))
+    return np.where(z >= 0, 1.0, e) / (1.0 + e)
 
 
 def silu(z):
