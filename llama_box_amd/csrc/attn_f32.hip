@@ -7,7 +7,9 @@
 //   k_attn_f32_rows  — one workgroup per (query token, head), its four waves take the cache in interleaved blocks of 64 cells and merge
 //                      their (max, sum, accumulator) through LDS; a block none of whose cells the mask lets through is skipped after
 //                      one 128-byte mask read (attention confined to a window or a chunk touches few blocks).  Decode steps and
-//                      small batches.
+//                      small batches.  With few (token, head) pairs over a long cache the cells are split over several workgroups
+//                      whose partial (max, sum, accumulator) records k_attn_f32_combine merges — and, where the graph gates the
+//                      heads behind the attention, multiplies by the gate's sigmoid on the way out.
 //   k_attn_f32_tile  — prompt batches: a workgroup owns 64 query tokens of one head; K and V blocks of 64 cells are staged through LDS as
 //                      f32 once per workgroup and every wave runs 16 of the queries against them (a lane owns one cell for the scores
 //                      and one or more value columns for the sum); blocks the mask hides from all 64 queries are skipped.
@@ -35,6 +37,7 @@ __device__ __forceinline__ float wave_sum_f(float v) {
 }
 
 constexpr int ATTN_F32_MAX_D = 640;   // largest head size (query/key or value): a latent cache row (latent + rotated part) serves as the key of every head
+constexpr int ATTN_F32_MAX_SPLITS = 32;  // workgroups over the cells of one (token, head) at most
 constexpr float ATTN_F32_LOW = -1e30f;  // "no score yet": finite, so that differences of maxima never give NaN
 
 // mask element -> additive term (f16 or f32 mask rows; -inf hides the cell)
@@ -118,7 +121,8 @@ __device__ __forceinline__ void attn_f32_pv8(const float p, const uint64_t live,
 
 template <int KT, int VT>
 __global__ void __launch_bounds__(256) k_attn_f32_rows(const tdesc q, const tdesc k, const tdesc v, const tdesc mask, const int has_mask, const float * __restrict__ sinks,
-                                                       const float * __restrict__ r12, const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap, const int pen_kind) {
+                                                       const float * __restrict__ r12, const tdesc dst, const float scale, const float * __restrict__ sig, const float softcap, const int pen_kind,
+                                                       float * __restrict__ parts) {
     __shared__ float qs[ATTN_F32_MAX_D];
     __shared__ float part_acc[4][ATTN_F32_MAX_D];
     __shared__ float part_m[4], part_l[4];
@@ -141,11 +145,11 @@ __global__ void __launch_bounds__(256) k_attn_f32_rows(const tdesc q, const tdes
     const bool sgm = sig != nullptr;
     const float s_temp = sgm ? sig[h] : 1.0f, s_bias = sgm ? sig[q.ne[2] + h] : 0.0f;
     float m = sgm ? 0.0f : ATTN_F32_LOW, l = 0.0f;
-    if (sinks && wave == 0 && !sgm) { m = sinks[h]; l = 1.0f; }  // the sink: exp(sink - m) = 1 in the denominator, nothing in the numerator
+    if (sinks && wave == 0 && blockIdx.z == 0 && !sgm) { m = sinks[h]; l = 1.0f; }  // the sink: exp(sink - m) = 1 in the denominator, nothing in the numerator
     float acc[ATTN_F32_MAX_D / 64];
 #pragma unroll
     for (int r = 0; r < ATTN_F32_MAX_D / 64; ++r) acc[r] = 0.0f;
-    for (int64_t j0 = (int64_t) wave * 64; j0 < n_kv; j0 += 256) {
+    for (int64_t j0 = (int64_t) (blockIdx.z * 4 + wave) * 64; j0 < n_kv; j0 += 256 * (int64_t) gridDim.z) {
         const int64_t j = j0 + lane;
         float mv = -INFINITY;
         if (j < n_kv) mv = has_mask ? mask_ld(mrow, mask.type, j) : 0.0f;
@@ -215,12 +219,48 @@ __global__ void __launch_bounds__(256) k_attn_f32_rows(const tdesc q, const tdes
     for (int w = 1; w < 4; ++w) M = fmaxf(M, part_m[w]);
     float L = 0.0f, cw[4];
     for (int w = 0; w < 4; ++w) { cw[w] = expf(part_m[w] - M); L += part_l[w] * cw[w]; }
+    if (gridDim.z > 1) {  // one of several workgroups over the cells of this (token, head): its record for the merge
+        float * rec = parts + ((t * q.ne[2] + h) * gridDim.z + blockIdx.z) * (int64_t) (DV + 2);
+        if (lane == 0) { rec[0] = M; rec[1] = L; }
+        for (int dcol = lane; dcol < DV; dcol += 64) {
+            float o = 0.0f;
+            for (int w = 0; w < 4; ++w) o += part_acc[w][dcol] * cw[w];
+            rec[2 + dcol] = o;
+        }
+        return;
+    }
     const float inv = sgm ? 1.0f : (L > 0.0f ? 1.0f / L : 0.0f);
     float * out = (float *) (dst.data + h * dst.nb[1] + t * dst.nb[2]);
     for (int dcol = lane; dcol < DV; dcol += 64) {
         float o = 0.0f;
         for (int w = 0; w < 4; ++w) o += part_acc[w][dcol] * cw[w];
         out[dcol] = o * inv;
+    }
+}
+
+// the merge of k_attn_f32_rows' partial records: one workgroup per (token, head).  gate (may be null): the output is multiplied by sigmoid(gate), one number per head or per entry
+__global__ void __launch_bounds__(128) k_attn_f32_combine(const float * __restrict__ parts, const int S, const int H, const int DV, const tdesc dst, const int sgm, const float * __restrict__ gate,
+                                                          const int gate_heads) {
+    __shared__ float cw[ATTN_F32_MAX_SPLITS];
+    const int64_t t = blockIdx.x, h = blockIdx.y;
+    const float * rec = parts + (t * H + h) * S * (int64_t) (DV + 2);
+    float M = rec[0];
+    for (int s = 1; s < S; ++s) M = fmaxf(M, rec[s * (int64_t) (DV + 2)]);
+    float L = 0.0f;
+    for (int s = 0; s < S; ++s) {
+        const float c = expf(rec[s * (int64_t) (DV + 2)] - M);
+        if (threadIdx.x == 0) cw[s] = c;
+        L += rec[s * (int64_t) (DV + 2) + 1] * c;
+    }
+    __syncthreads();
+    const float inv = sgm ? 1.0f : (L > 0.0f ? 1.0f / L : 0.0f);
+    float * out = (float *) (dst.data + h * dst.nb[1] + t * dst.nb[2]);
+    for (int d = threadIdx.x; d < DV; d += 128) {
+        float o = 0.0f;
+        for (int s = 0; s < S; ++s) o += rec[s * (int64_t) (DV + 2) + 2 + d] * cw[s];
+        o = o * inv;
+        if (gate) o = o * (1.f / (1.f + expf(-gate[gate_heads ? t * H + h : (t * H + h) * DV + d])));
+        out[d] = o;
     }
 }
 
@@ -705,6 +745,22 @@ static bool attn_mma_bf16_ok(const tdesc & q, const tdesc & k, const tdesc & v, 
     return true;
 }
 
+// how many workgroups share the cells of one (token, head) — 1 unless the row kernel serves the op with few pairs over a cache of several blocks.  Every split walks whole groups of
+// 256 cells (a block of 64 per wave)
+int attn_f32_row_splits(const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const tdesc & dst) {
+    static const bool on = !getenv("GGML_MI355X_ATTN_SPLIT") || atoi(getenv("GGML_MI355X_ATTN_SPLIT")) != 0;
+    static const bool mma_on = !getenv("GGML_MI355X_ATTN_MMA") || atoi(getenv("GGML_MI355X_ATTN_MMA")) != 0;
+    const int64_t pairs = q.ne[1] * q.ne[2], groups = (k.ne[1] + 255) / 256;
+    if (!on || groups < 2 || pairs >= 512) return 1;
+    if (mask && q.ne[1] >= 32 && q.ne[0] <= 128 && v.ne[0] <= 128) return 1;  // (the tile or the matrix-core kernel)
+    if (mma_on && (attn_mma_bf16_wide_ok(q, k, v, mask, dst) || attn_mma_bf16_ok(q, k, v, mask, dst))) return 1;
+    return (int) std::max<int64_t>(1, std::min<int64_t>({groups, (int64_t) ATTN_F32_MAX_SPLITS, 1024 / std::max<int64_t>(1, pairs)}));
+}
+size_t attn_f32_workspace_bytes(const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const tdesc & dst) {
+    const int S = attn_f32_row_splits(q, k, v, mask, dst);
+    return S > 1 ? (size_t) q.ne[1] * (size_t) q.ne[2] * (size_t) S * (size_t) (v.ne[0] + 2) * sizeof(float) : 0;
+}
+
 static bool attn_f32_type_ok(int t) { return t == GGML_TYPE_F32 || t == GGML_TYPE_BF16 || t == GGML_TYPE_F16; }
 
 // may launch_attn_f32 serve this op?  q f32 [DK, n_q, H], k [DK, n_kv, G], v [DV, n_kv, G] of one type each, rows contiguous, one batch
@@ -721,7 +777,7 @@ bool attn_f32_applies(const tdesc & q, const tdesc & k, const tdesc & v, const t
 
 template <int KT, int VT>
 static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const float * sinks, const float * r12, const tdesc & dst, float scale,
-                              const float * sig, float softcap, int pen_kind) {
+                              const float * sig, float softcap, int pen_kind, const attn_f32_extra & x) {
     const int64_t n_q = q.ne[1], H = q.ne[2];
     const int DK = (int) q.ne[0], DV = (int) v.ne[0];
     if constexpr (KT == GGML_TYPE_BF16 && VT == GGML_TYPE_BF16) {
@@ -748,8 +804,13 @@ static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, c
             const dim3 block((unsigned) (64 * nw));
             const int dk16 = (DK + 15) / 16, dvt = (DV + 31) / 32;
 #define MI_ATT_MMA(A, B) hipLaunchKernelGGL((k_attn_mma_bf16<A, B>), grid, block, 0, s, q, k, v, *mask, sinks, r12, dst, scale, sig, softcap, pen_kind)
-            const int a = dk16 <= 2 ? 2 : (dk16 <= 4 ? 4 : 8), b = dvt <= 1 ? 1 : (dvt <= 2 ? 2 : 4);
+            const int a = dk16 <= 2 ? 2 : (dk16 <= 4 ? 4 : (dk16 <= 6 ? 6 : 8)), b = dvt <= 1 ? 1 : (dvt <= 2 ? 2 : (dvt <= 3 ? 3 : 4));
             if (a == 2 && b == 1) MI_ATT_MMA(2, 1); else if (a == 2 && b == 2) MI_ATT_MMA(2, 2); else if (a == 2) MI_ATT_MMA(2, 4);
+            else if (a == 6 && b == 3) MI_ATT_MMA(6, 3);
+            else if (b == 3) MI_ATT_MMA(8, 4);  // (between the tilings: the next larger one)
+            else if (a == 6 && b == 4) MI_ATT_MMA(8, 4);
+            else if (a == 6 && b == 2) MI_ATT_MMA(8, 2);
+            else if (a == 6) MI_ATT_MMA(8, 1);
             else if (a == 4 && b == 1) MI_ATT_MMA(4, 1); else if (a == 4 && b == 2) MI_ATT_MMA(4, 2); else if (a == 4) MI_ATT_MMA(4, 4);
             else if (b == 1) MI_ATT_MMA(8, 1); else if (b == 2) MI_ATT_MMA(8, 2); else MI_ATT_MMA(8, 4);
 #undef MI_ATT_MMA
@@ -772,13 +833,20 @@ static void attn_f32_launch_t(hipStream_t s, const tdesc & q, const tdesc & k, c
         else go(k_attn_f32_tile<KT, VT, 128, 128>, 128, 128);
         return;
     }
-    hipLaunchKernelGGL((k_attn_f32_rows<KT, VT>), dim3((unsigned) n_q, (unsigned) H), dim3(256), 0, s, q, k, v, mask ? *mask : q, mask ? 1 : 0, sinks, r12, dst, scale, sig, softcap, pen_kind);
+    const int S = attn_f32_row_splits(q, k, v, mask, dst);
+    const bool split = S > 1 && x.ws && attn_f32_workspace_bytes(q, k, v, mask, dst) <= x.ws_bytes;
+    hipLaunchKernelGGL((k_attn_f32_rows<KT, VT>), dim3((unsigned) n_q, (unsigned) H, split ? (unsigned) S : 1u), dim3(256), 0, s, q, k, v, mask ? *mask : q, mask ? 1 : 0, sinks, r12, dst, scale, sig,
+                       softcap, pen_kind, (float *) x.ws);
+    if (!split) return;
+    tdesc o = dst;
+    if (x.gate) o.data = (char *) x.gated;
+    hipLaunchKernelGGL(k_attn_f32_combine, dim3((unsigned) n_q, (unsigned) H), dim3(128), 0, s, (const float *) x.ws, S, (int) H, DV, o, sig ? 1 : 0, x.gate, x.gate_heads);
 }
 
 void launch_attn_f32(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const float * sinks, const float * r12, const tdesc & dst, float scale,
-                     const float * sig, float softcap, int pen_kind) {
+                     const float * sig, float softcap, int pen_kind, const attn_f32_extra & x) {
     if (q.ne[1] == 0 || q.ne[2] == 0) return;
-#define MI_ATTN_F32_CASE(KT, VT) if (k.type == KT && v.type == VT) { attn_f32_launch_t<KT, VT>(s, q, k, v, mask, sinks, r12, dst, scale, sig, softcap, pen_kind); return; }
+#define MI_ATTN_F32_CASE(KT, VT) if (k.type == KT && v.type == VT) { attn_f32_launch_t<KT, VT>(s, q, k, v, mask, sinks, r12, dst, scale, sig, softcap, pen_kind, x); return; }
     MI_ATTN_F32_CASE(GGML_TYPE_F32, GGML_TYPE_F32)
     MI_ATTN_F32_CASE(GGML_TYPE_BF16, GGML_TYPE_BF16)
     MI_ATTN_F32_CASE(GGML_TYPE_F16, GGML_TYPE_F16)

@@ -361,7 +361,10 @@ static ws_plan plan_ws(backend_ctx * c, const ggml_cgraph * g) {
         } else if (n->op == GGML_OP_GATED_LINEAR_ATTN && n->op_params[3] == MI_SEQ_OP_TAG && (n->op_params[0] == SEQ_DELTA_CH || n->op_params[0] == SEQ_LINEAR) && n->src[0] && n->src[3]) {
             p.aux_bytes = std::max(p.aux_bytes, seq_recurrence_scratch_bytes(n->op_params[0], n->op_params[1], (int) (n->src[0]->ne[0] / std::max(1, n->op_params[2])), n->src[3]->ne[1]));
         } else if (n->op == GGML_OP_FLASH_ATTN_EXT && fa_route(n) == 4) {
-            continue;  // the 32-bit kernels keep their running sums on chip
+            // the 32-bit kernels keep their running sums on chip, but for few (token, head) pairs over a long cache: partial records of the splits
+            const tdesc md = n->src[3] ? TD(n->src[3]) : TD(n->src[0]);
+            p.aux_bytes = std::max(p.aux_bytes, attn_f32_workspace_bytes(TD(n->src[0]), TD(n->src[1]), TD(n->src[2]), n->src[3] ? &md : nullptr, TD(n)));
+            continue;
         } else if (n->op == GGML_OP_FLASH_ATTN_EXT) {
             const tdesc q = TD(n->src[0]), k = TD(n->src[1]), v = TD(n->src[2]);
             // (both forms a 33+-token batch may take — matrix-core tiles or, for a mask known to be sparse, position lists — fit this)
@@ -2521,6 +2524,38 @@ static int try_fuse_concat_rope(exec_state & st, int i) {
     return 2;
 }
 
+// FLASH_ATTN_EXT -> UNARY(SIGMOID, gate) -> MUL of the two (views skipped; one gate per head or per entry): fills the gate's part of `x` for an attention whose cells are split over
+// workgroups — the merge applies the gate.  Returns the nodes consumed at position i (1: no gate)
+static int attn_gate_behind(exec_state & st, int i, attn_f32_extra & x) {
+    ggml_cgraph * g = st.g;
+    const ggml_tensor * n = g->nodes[i];
+    if (!is_f32_contig(n) || n->ne[3] != 1 || !single_use(st, n)) return 1;
+    const ggml_tensor * at[2] = {};
+    int k = i + 1;
+    for (int found = 0; found < 2; ++k) {
+        if (k >= g->n_nodes || st.done[k]) return 1;
+        if (!is_view_op(g->nodes[k])) at[found++] = g->nodes[k];
+    }
+    const ggml_tensor * un = at[0], * ml = at[1];
+    if (un->op != GGML_OP_UNARY || un->op_params[0] != GGML_UNARY_OP_SIGMOID || ml->op != GGML_OP_MUL || !single_use(st, un) || through_views(ml->src[0]) != n || through_views(ml->src[1]) != un) return 1;
+    for (const ggml_tensor * t : {ml->src[0], ml->src[1]})
+        if (t != n && t != un && !single_use(st, t)) return 1;
+    const ggml_tensor * gate = un->src[0];
+    const int64_t H = n->ne[1], T = n->ne[2], total = ggml_abi_nelements(n);
+    if (!is_f32_contig(gate) || !is_f32_contig(ml) || !is_f32_contig(ml->src[0]) || !is_f32_contig(ml->src[1]) || ggml_abi_nelements(ml) != total) return 1;
+    if (ggml_abi_nelements(gate) == total && same_shape(ml->src[0], ml->src[1])) {
+        if (!elementwise_safe(ml, gate)) return 1;
+        x.gate_heads = 0;
+    } else if (ggml_abi_nelements(gate) == H * T && ml->src[1]->ne[0] == 1 && ml->src[1]->ne[1] == H && ml->src[1]->ne[2] == T && same_shape(ml->src[0], n)) {
+        if (ranges_overlap(ml, gate)) return 1;
+        x.gate_heads = 1;
+    } else return 1;
+    x.gate = (const float *) gate->data;
+    x.gated = (float *) ml->data;
+    st.c->st.fused_nodes += 2;
+    return k - i;
+}
+
 static int run_node(exec_state & st, int i) {
     backend_ctx * c = st.c;
     ggml_cgraph * g = st.g;
@@ -3314,11 +3349,16 @@ static int run_node(exec_state & st, int i) {
             if (fa_route(n) == 4) {
                 const tdesc md4 = m ? TD(m) : qd;
                 timed_scope ts(c, "attn_f32", (double) ggml_abi_nbytes(k) + (double) ggml_abi_nbytes(v));
+                attn_f32_extra x;
+                int used = 1;
+                if (c->ws && c->ws_size > st.aux_off) { x.ws = (char *) c->ws + st.aux_off; x.ws_bytes = c->ws_size - st.aux_off; }
+                const size_t need = attn_f32_workspace_bytes(qd, kd, vd, m ? &md4 : nullptr, TD(n));
+                if (fuse && need > 0 && x.ws && need <= x.ws_bytes) used = attn_gate_behind(st, i, x);
                 launch_attn_f32(s, qd, kd, vd, m ? &md4 : nullptr, n->src[4] ? (const float *) n->src[4]->data : nullptr, n->src[5] ? (const float *) n->src[5]->data : nullptr, TD(n), p.scale,
-                                n->src[6] ? (const float *) n->src[6]->data : nullptr, p.logit_softcap, n->src[5] && ggml_abi_nelements(n->src[5]) == a->ne[2] ? ATTN_PEN_LINEAR : ATTN_PEN_LOG);
+                                n->src[6] ? (const float *) n->src[6]->data : nullptr, p.logit_softcap, n->src[5] && ggml_abi_nelements(n->src[5]) == a->ne[2] ? ATTN_PEN_LINEAR : ATTN_PEN_LOG, x);
                 c->st.kernel_launches++;
                 c->st.attn_f32_nodes++;
-                return 1;
+                return used;
             }
             bool imaged = fa_route(n) == 3;
             bool native_kv = false;

@@ -174,8 +174,13 @@ bool attn_f32_applies(const tdesc & q, const tdesc & k, const tdesc & v, const t
 // q.k * scale - r1 ln(1 + r2 distance); with pen_kind ATTN_PEN_LINEAR r12 holds r1 alone and the score is q.k * scale - r1 distance
 enum { ATTN_PEN_LOG = 1, ATTN_PEN_LINEAR = 2 };
 // sig: per head a factor on the score, then per head a bias ([heads, 2]) — the weights are then sigmoid(score + bias), not a soft-max; softcap > 0: score <- cap tanh(score / cap)
+// scratch for the row kernel's partial records (attn_f32_workspace_bytes(): a batch of few (token, head) pairs over a long cache splits the cells over several workgroups; without it the
+// cells stay together); gate (only where the cells are split): the heads times sigmoid(gate), one number per head or per entry, go to `gated` (laid out as dst) instead of dst
+struct attn_f32_extra { void * ws = nullptr; size_t ws_bytes = 0; const float * gate = nullptr; int gate_heads = 0; float * gated = nullptr; };
+int attn_f32_row_splits(const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const tdesc & dst);
+size_t attn_f32_workspace_bytes(const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const tdesc & dst);
 void launch_attn_f32(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const float * sinks, const float * r12, const tdesc & dst, float scale,
-                     const float * sig = nullptr, float softcap = 0.0f, int pen_kind = ATTN_PEN_LOG);
+                     const float * sig = nullptr, float softcap = 0.0f, int pen_kind = ATTN_PEN_LOG, const attn_f32_extra & x = {});
 // ---- non-flash attention chain of a small batch over position lists (attn_nf.hip)
 size_t attn_nf_list_scratch_bytes(const tdesc & q, const tdesc & k, int * dq_out);
 bool launch_attn_nf_list(hipStream_t s, const tdesc & q, const tdesc & k, const tdesc & v, const tdesc & mask, const tdesc & dst, const int * lists, int list_stride,

@@ -19,6 +19,7 @@
 //                     raw a [DK H, T] being a projection of its own; beta = sigmoid(b_pre) from a [H, T] projection; the rest as SEQ_DELTA
 //   k_seq_recurrence<SEQ_SSD>    state-space duality (Mamba-2): dt = softplus(dt_pre + dt_bias); S <- exp(-exp(A_log) dt) S + dt B x^T; y = S^T C + D x, with B as the keys,
 //                     C as the queries (grouped: head h reads group h / (H / G)) and x as the values
+//   k_seq_linear_block  the same recurrence over prompt portions: several waves share each staged block of tokens
 //   k_seq_recurrence<SEQ_LINEAR>  gated linear attention: S <- diag(w) S + k v^T, w = sigmoid(a + offset)^(1 / tau) per key channel; o = S^T q dk^-1/2
 //   k_seq_recurrence<SEQ_MLSTM>  matrix memory with exponential gates under a running maximum m: m' = max(f + m, i); S <- e^(f + m - m') S + e^(i - m') k v^T; n likewise with k;
 //                     o = S^T q / (max(|n . q|, e^(-m')) + 1e-6); log gates capped by cap tanh(. / cap), f through log-sigmoid
@@ -488,6 +489,126 @@ __global__ void __launch_bounds__(256) k_seq_linear_decay(const tdesc a, const f
     if (c >= C) return;
     out[t * C + c] = seq_linear_decay(((const float *) (a.data + t * a.nb[1]))[c] + p0[c], tau);
 }
+// gated linear attention over a prompt portion.  A token's update of the state waits for nothing but the state, so what the walk costs is bringing the tokens' vectors to the lanes: here NW
+// waves (4 NW value columns of a head) share ONE staged copy of each block of TB tokens, double-buffered in LDS and fetched sixteen bytes at a time, with the decays already computed by the
+// pass above.  Thread layout, state and arithmetic are k_seq_recurrence's, operation by operation: a sequence may pass from one kernel to the other between its portions.  A key-sized
+// vector lies in LDS in the order the lanes read it — lane ks's m-th group of four entries at 4 (16 m + ks) — so sixteen lanes read 256 neighbouring bytes.
+// Needs key and value rows of whole groups of four, 16-byte aligned (seq_linear_block_ok); R = key rows per lane exactly.
+template <int R, int NW, int TB>
+__global__ void __launch_bounds__(64 * NW) k_seq_linear_block(const seq_rec_args A) {
+    constexpr int KP = SEQ_LPC * R, COLS = SEQ_COLS * NW, PER = 3 * KP + COLS, NT = 64 * NW;
+    constexpr int K4 = TB * 3 * (KP / 4), NK = (K4 + NT - 1) / NT, V4 = TB * (COLS / 4);  // float4 items of a block: key-sized ones, values (V4 <= NT)
+    static_assert(V4 <= NT, "a thread stages at most one group of values");
+    __shared__ __attribute__((aligned(16))) float blk[2][TB * PER];
+    __shared__ int rows_of[3][TB];
+    const int s = blockIdx.x, h = blockIdx.y, j0 = blockIdx.z * COLS, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int begin = A.info[4 * s], count = A.info[4 * s + 1], slot = A.info[4 * s + 2], reset = A.info[4 * s + 3];
+    const int DK = A.DK, DV = A.DV;
+    const int ks = lane & (SEQ_LPC - 1), jl = wave * SEQ_COLS + (lane >> 4), j = j0 + jl;
+    const bool col = j < DV;
+    float * __restrict__ Sm = A.state + (int64_t) slot * A.state_stride + (int64_t) h * R * DV * SEQ_LPC;
+    float S[R];
+#pragma unroll
+    for (int ii = 0; ii < R; ++ii) {
+        const bool ok = ks * R + ii < DK && col;
+        const float sv = Sm[ok ? ((int64_t) ii * DV + j) * SEQ_LPC + ks : 0];
+        S[ii] = (ok && !reset) ? sv : 0.0f;
+    }
+    float4 pk[NK], pv;
+    auto fetch = [&](const int * rows, const int n_tok) {
+#pragma unroll
+        for (int i = 0; i < NK; ++i) {
+            const int item = tid + NT * i, u = item / (3 * (KP / 4)), f = item - u * (3 * (KP / 4)), which = f / (KP / 4), e = 4 * (f - which * (KP / 4));
+            const bool ok = item < K4 && u < n_tok && e < DK;
+            const tdesc & t = which == 0 ? A.k : which == 1 ? A.q : A.g;
+            const float4 v = *(const float4 *) (t.data + (int64_t) rows[ok ? u : 0] * t.nb[1] + (int64_t) (h * DK + (ok ? e : 0)) * 4);
+            pk[i] = ok ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+        if (tid < V4) {
+            const int u = tid / (COLS / 4), e = 4 * (tid - u * (COLS / 4));
+            const bool ok = u < n_tok && j0 + e < DV;
+            const float4 v = *(const float4 *) (A.v.data + (int64_t) rows[ok ? u : 0] * A.v.nb[1] + (int64_t) (h * DV + (ok ? j0 + e : 0)) * 4);
+            pv = ok ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+    };
+    auto park = [&](float * d) {
+#pragma unroll
+        for (int i = 0; i < NK; ++i) {
+            const int item = tid + NT * i, u = item / (3 * (KP / 4)), f = item - u * (3 * (KP / 4)), which = f / (KP / 4), e4 = f - which * (KP / 4);
+            if (item < K4) *(float4 *) (d + u * PER + which * KP + 4 * ((e4 % (R / 4)) * SEQ_LPC + e4 / (R / 4))) = pk[i];
+        }
+        if (tid < V4) *(float4 *) (d + (tid / (COLS / 4)) * PER + 3 * KP + 4 * (tid % (COLS / 4))) = pv;
+    };
+    if (tid < TB)
+        for (int b = 0; b < 2; ++b) rows_of[b][tid] = b * TB + tid < count ? A.tok[begin + b * TB + tid] : 0;
+    __syncthreads();
+    fetch(rows_of[0], min(TB, count));
+    park(blk[0]);
+    __syncthreads();
+    auto token = [&](const float * lt, const int row) {
+        const float4 * k4 = (const float4 *) lt + ks, * q4 = (const float4 *) (lt + KP) + ks, * w4 = (const float4 *) (lt + 2 * KP) + ks;
+        const float vj = lt[3 * KP + jl];
+        float p0 = 0.0f, p1 = 0.0f, p2 = 0.0f, p3 = 0.0f;
+#pragma unroll
+        for (int m = 0; m < R / 4; ++m) {
+            const float4 kk = k4[SEQ_LPC * m], qq = q4[SEQ_LPC * m], ww = w4[SEQ_LPC * m];
+            S[4 * m] = fmaf(ww.x, S[4 * m], kk.x * vj);
+            S[4 * m + 1] = fmaf(ww.y, S[4 * m + 1], kk.y * vj);
+            S[4 * m + 2] = fmaf(ww.z, S[4 * m + 2], kk.z * vj);
+            S[4 * m + 3] = fmaf(ww.w, S[4 * m + 3], kk.w * vj);
+            p0 = fmaf(S[4 * m], qq.x, p0);
+            p1 = fmaf(S[4 * m + 1], qq.y, p1);
+            p2 = fmaf(S[4 * m + 2], qq.z, p2);
+            p3 = fmaf(S[4 * m + 3], qq.w, p3);
+        }
+        const float o = quad_sum((p0 + p1) + (p2 + p3)) * A.qscale;
+        if (col && ks == 0) ((float *) (A.dst.data + (int64_t) h * A.dst.nb[1] + (int64_t) row * A.dst.nb[2]))[j] = o;
+    };
+    for (int b0 = 0, b = 0; b0 < count; b0 += TB, ++b) {
+        const int n_here = min(TB, count - b0), n_next = min(TB, count - b0 - TB);
+        const float * cur = blk[b & 1];
+        const int * trow = rows_of[b % 3];
+        int row_after = 0;
+        if (n_next > 0) {
+            fetch(rows_of[(b + 1) % 3], n_next);
+            if (tid < TB && b0 + 2 * TB + tid < count) row_after = A.tok[begin + b0 + 2 * TB + tid];
+        }
+        if (n_here == TB) {
+#pragma unroll
+            for (int u = 0; u < TB; ++u) token(cur + u * PER, trow[u]);
+        } else
+            for (int u = 0; u < n_here; ++u) token(cur + u * PER, trow[u]);
+        if (n_next > 0) {
+            park(blk[(b + 1) & 1]);  // (last read in the block before this one: every thread has passed the barrier behind it)
+            if (tid < TB) rows_of[(b + 2) % 3][tid] = row_after;
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int ii = 0; ii < R; ++ii)
+        if (col && ks * R + ii < DK) Sm[((int64_t) ii * DV + j) * SEQ_LPC + ks] = S[ii];
+}
+static bool seq_linear_block_ok(const seq_rec_args & a) {
+    auto rows16 = [](const tdesc & t) { return t.nb[0] == 4 && (t.nb[1] % 16) == 0 && (((uintptr_t) t.data) & 15) == 0; };
+    return a.w_ready && (a.DK % 4) == 0 && (a.DV % 4) == 0 && rows16(a.q) && rows16(a.k) && rows16(a.v) && rows16(a.g);
+}
+static bool launch_seq_linear_block(hipStream_t s, const seq_rec_args & a, int n_seqs) {
+    static const bool on = !getenv("GGML_MI355X_SEQ_BLOCK") || atoi(getenv("GGML_MI355X_SEQ_BLOCK")) != 0;
+    if (!on || !seq_linear_block_ok(a)) return false;
+    const int R = seq_rows_per_lane(a.DK);
+    // two waves per workgroup while four would leave CUs without one
+    const bool two = (int64_t) n_seqs * a.H * ((a.DV + 15) / 16) < 256;
+#define MI_SEQ_LIN(RR, TB) do { if (two) hipLaunchKernelGGL((k_seq_linear_block<RR, 2, TB>), dim3((unsigned) n_seqs, (unsigned) a.H, (unsigned) ((a.DV + 7) / 8)), dim3(128), 0, s, a); \
+                                else hipLaunchKernelGGL((k_seq_linear_block<RR, 4, TB>), dim3((unsigned) n_seqs, (unsigned) a.H, (unsigned) ((a.DV + 15) / 16)), dim3(256), 0, s, a); } while (0)
+    if (R == 4) MI_SEQ_LIN(4, 16);
+    else if (R == 8) MI_SEQ_LIN(8, 16);
+    else if (R == 12) MI_SEQ_LIN(12, 8);
+    else if (R == 16) MI_SEQ_LIN(16, 8);
+    else return false;
+#undef MI_SEQ_LIN
+    return true;
+}
+
 size_t seq_recurrence_scratch_bytes(int kind, int H, int DK, int64_t T) { return ((kind == SEQ_DELTA_CH || kind == SEQ_LINEAR) && T >= SEQ_DECAY_PREPASS_MIN) ? (size_t) T * H * DK * sizeof(float) : 0; }
 
 // floats of state one slot needs
@@ -531,7 +652,7 @@ void launch_seq_recurrence(hipStream_t s, int kind, const seq_rec_args & a_in, i
     else if (kind == SEQ_DELTA) seq_recurrence_launch<SEQ_DELTA>(s, a, n_seqs);
     else if (kind == SEQ_DELTA_CH) seq_recurrence_launch<SEQ_DELTA_CH>(s, a, n_seqs);
     else if (kind == SEQ_SSD) seq_recurrence_launch<SEQ_SSD>(s, a, n_seqs);
-    else if (kind == SEQ_LINEAR) seq_recurrence_launch<SEQ_LINEAR>(s, a, n_seqs);
+    else if (kind == SEQ_LINEAR) { if (!launch_seq_linear_block(s, a, n_seqs)) seq_recurrence_launch<SEQ_LINEAR>(s, a, n_seqs); }
     else seq_recurrence_launch<SEQ_MLSTM>(s, a, n_seqs);
 }
 
