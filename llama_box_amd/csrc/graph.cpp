@@ -2262,7 +2262,29 @@ static int try_fuse_expert_join(exec_state & st, int i) {
     return (j.add ? j.end : end) - i;
 }
 
-// MUL(rows of MUL_MAT_ID [2 nc, n_used, T], one factor per row) -> SwiGLU of the halves: one launch.  Returns the nodes consumed (0: no match)
+// the product that follows a gated activation `gl` (node k - 1) of rows `gu` and reads nothing else: a decode step's down projection takes the activation as its prologue.  Returns the node
+// behind the product (-1: no such product)
+static int try_glu_into_product(exec_state & st, int k, const ggml_tensor * gl, const ggml_tensor * gu, const ggml_tensor * w) {
+    backend_ctx * c = st.c;
+    ggml_cgraph * g = st.g;
+    static const bool on = !getenv("GGML_MI355X_GLU_MATVEC") || atoi(getenv("GGML_MI355X_GLU_MATVEC")) != 0;
+    while (k < g->n_nodes && !st.done[k] && is_view_op(g->nodes[k])) ++k;
+    if (!on || k >= g->n_nodes || st.done[k] || !single_use(st, gl)) return -1;
+    const ggml_tensor * mm = g->nodes[k], * a = mm->src[0], * x = mm->src[1];
+    if ((mm->op != GGML_OP_MUL_MAT && mm->op != GGML_OP_MUL_MAT_ID) || through_views(x) != gl || (x != gl && !single_use(st, x)) || buffer_is_split(a->buffer) || tp_active(c) || !is_f32_contig(mm) ||
+        !is_f32_contig(x) || a->ne[0] != gl->ne[0] || ranges_overlap(mm, gu) || (w && ranges_overlap(mm, w))) return -1;
+    const ggml_tensor * ids = mm->op == GGML_OP_MUL_MAT_ID ? mm->src[2] : nullptr;
+    const int64_t cols = ggml_abi_nrows(gl);
+    if (ids ? (x->ne[1] != ids->ne[0] || x->ne[2] != ids->ne[1] || cols != ggml_abi_nelements(ids) || ranges_overlap(mm, ids)) : cols != 1 || mm_cache_image_ok(mm)) return -1;
+    const tdesc id = ids ? TD(ids) : TD(a);
+    if (!matvec_glu_ok(TD(a), gu->data, ids ? &id : nullptr)) return -1;
+    timed_scope ts(c, ids ? "mul_mat_id" : "mul_mat_f", (double) ggml_abi_nbytes(a) / (double) std::max<int64_t>(1, a->ne[2]) * (double) (ids ? std::min<int64_t>(a->ne[2], cols) : 1));
+    launch_matvec_glu(c->stream, TD(a), (const float *) gu->data, w ? (const float *) w->data : nullptr, ids ? &id : nullptr, TD(mm));
+    c->st.kernel_launches++;
+    c->st.fused_nodes++;
+    return k + 1;
+}
+// MUL(rows of MUL_MAT_ID [2 nc, n_used, T], one factor per row) -> SwiGLU of the halves [-> the product that reads it]: one launch.  Returns the nodes consumed (0: no match)
 static int try_fuse_swiglu_scaled(exec_state & st, int i) {
     ggml_cgraph * g = st.g;
     const ggml_tensor * m = g->nodes[i], * gu = m->src[0], * w = m->src[1];
@@ -2274,6 +2296,11 @@ static int try_fuse_swiglu_scaled(exec_state & st, int i) {
     const int64_t nc = gl->ne[0], rows = ggml_abi_nrows(gl);
     if (!is_f32_contig(gu) || !is_f32_contig(m) || !is_f32_contig(gl) || !is_f32_contig(w) || !same_shape(m, gu) || gu->ne[0] != 2 * nc || gl->src[0]->ne[0] != 2 * nc || ggml_abi_nrows(gu) != rows ||
         w->ne[0] != 1 || w->ne[1] != gu->ne[1] || w->ne[2] != gu->ne[2] || w->ne[3] != gu->ne[3]) return 0;
+    const int behind = try_glu_into_product(st, k + 1, gl, gu, w);
+    if (behind > 0) {
+        st.c->st.fused_nodes++;
+        return behind - i;
+    }
     if (ranges_overlap(gl, gu) || ranges_overlap(gl, w)) return 0;
     timed_scope ts(st.c, "swiglu", (double) ggml_abi_nbytes(gl) * 3);
     launch_swiglu_scaled(st.c->stream, (const float *) gu->data, (const float *) w->data, (float *) gl->data, nc, rows);
@@ -3107,6 +3134,10 @@ static int run_node(exec_state & st, int i) {
                 c->st.kernel_launches++;
                 c->st.fused_nodes++;
                 return 1;
+            }
+            if (fuse && !b && n->op_params[1] == 0 && is_f32_contig(a) && is_f32_contig(n) && a->ne[0] == 2 * n->ne[0]) {
+                const int behind = try_glu_into_product(st, i + 1, n, a, nullptr);
+                if (behind > 0) return behind - i;
             }
             timed_scope ts(c, "swiglu", (double) ggml_abi_nbytes(n) * 3);
             launch_swiglu(s, TD(a), b ? &bd : nullptr, TD(n), n->op_params[1]);

@@ -168,6 +168,9 @@ void launch_matvec_bf16_multi(hipStream_t s, matvec_multi mm, const float * x, i
 // per-expert column lists of the batched form; lists_valid: an earlier call left the lists of these same ids there
 size_t mul_mat_id_workspace_bytes(const tdesc & as, const tdesc & ids);
 bool launch_mul_mat_id(hipStream_t s, const tdesc & as, const tdesc & b, const tdesc & ids, const tdesc & d, void * ws, size_t ws_bytes, bool lists_valid);  // true: the batched form ran and left the lists in ws
+// MUL_MAT of ONE column / MUL_MAT_ID of few columns by a bf16 matrix whose operand is silu(g f) (u f) of rows gu [2 K, n_used, T] (f: one factor per row, or null)
+bool matvec_glu_ok(const tdesc & a, const void * gu, const tdesc * ids);
+void launch_matvec_glu(hipStream_t s, const tdesc & a, const float * gu, const float * f, const tdesc * ids, const tdesc & d);
 // FLASH_ATTN_EXT in 32-bit arithmetic over f32 / bf16 / f16 K and V read in place, any head sizes up to 256, K and V sizes independent (attn_f32.hip)
 bool attn_f32_applies(const tdesc & q, const tdesc & k, const tdesc & v, const tdesc * mask, const tdesc & dst);
 // r12 (optional: r1 of every head, then r2 of every head): the mask then holds the DISTANCE between query and cell for visible pairs (-inf for hidden ones) and the score is

@@ -976,6 +976,65 @@ __global__ void __launch_bounds__(256) k_mul_mat_id_vec(const tdesc a, const tde
     }
 }
 
+// ... and the same rows against a column that is a gated activation, made on the way in: x = silu(g f) (u f) from rows [g (K) | u (K)] with one factor f per row (w null: 1) — the down projection
+// of a decode step's feed-forward without the launch in front of it.  ids null: one matrix.  Every workgroup makes the whole column (K activations over 256 threads); the products and their
+// order are those of k_mul_mat_id_vec / k_mul_mat_f16_gqa_long
+__global__ void __launch_bounds__(256) k_matvec_glu_bf16(const tdesc a, const float * __restrict__ gu, const float * __restrict__ f, const tdesc ids, const int has_ids, const tdesc d) {
+    __shared__ float part[4][4];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int64_t u = blockIdx.y, t = blockIdx.z, K = a.ne[0], row0 = (int64_t) blockIdx.x * 4, col = u + t * gridDim.y;
+    int32_t e = 0;
+    if (has_ids) {
+        e = *(const int32_t *) (ids.data + u * ids.nb[0] + t * ids.nb[1]);
+        if (e < 0 || e >= a.ne[2]) return;
+    }
+    const char * wr[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) wr[r] = a.data + std::min<int64_t>(row0 + r, a.ne[1] - 1) * a.nb[1] + (int64_t) e * a.nb[2];
+    const float * gr = gu + col * 2 * K;
+    const float fac = f ? f[col] : 1.0f;
+    float acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int64_t k = (int64_t) wave * 512 + lane * 8; k < K; k += 2048) {
+        float w[4][8], x[8];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mmf_w8<true>(wr[r] + k * 2, w[r]);
+        const float4 g0 = *(const float4 *) (gr + k), g1 = *(const float4 *) (gr + k + 4), u0 = *(const float4 *) (gr + K + k), u1 = *(const float4 *) (gr + K + k + 4);
+        const float gg[8] = {g0.x, g0.y, g0.z, g0.w, g1.x, g1.y, g1.z, g1.w}, uu[8] = {u0.x, u0.y, u0.z, u0.w, u1.x, u1.y, u1.z, u1.w};
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const float gs = f ? gg[i] * fac : gg[i], us = f ? uu[i] * fac : uu[i];
+            x[i] = mmf_bf16_round(silu_f(gs) * us);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) acc[r] = fmaf(w[r][i], x[i], acc[r]);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const float v = wave_sum(acc[r]);
+        if (lane == 0) part[wave][r] = v;
+    }
+    __syncthreads();
+    if (threadIdx.x < 4) {
+        const int r = threadIdx.x;
+        const float v = ((part[0][r] + part[1][r]) + part[2][r]) + part[3][r];
+        if (row0 + r < a.ne[1]) *(float *) (d.data + (row0 + r) * d.nb[0] + u * d.nb[1] + t * d.nb[2]) = v;
+    }
+}
+// may launch_matvec_glu serve MUL_MAT (ids null: one column) / MUL_MAT_ID (few columns) over the activation of rows gu [2 K, n_used, T]?  Only where the plain launch runs the kernels whose
+// sums it repeats
+bool matvec_glu_ok(const tdesc & a, const void * gu, const tdesc * ids) {
+    const int64_t K = a.ne[0];
+    if (a.type != GGML_TYPE_BF16 || a.nb[0] != 2 || (a.nb[1] % 16) || (a.nb[2] % 16) || (K % 8) || ((((uintptr_t) a.data) | ((uintptr_t) gu)) & 15) || a.ne[3] != 1) return false;
+    return ids ? K >= 256 && ids->ne[0] * ids->ne[1] < 64 : K > 512 && a.ne[1] >= 64 && a.ne[2] == 1;
+}
+void launch_matvec_glu(hipStream_t s, const tdesc & a, const float * gu, const float * f, const tdesc * ids, const tdesc & d) {
+    if (a.ne[1] == 0) return;
+    const dim3 grid((unsigned) ((a.ne[1] + 3) / 4), ids ? (unsigned) ids->ne[0] : 1u, ids ? (unsigned) ids->ne[1] : 1u);
+    hipLaunchKernelGGL(k_matvec_glu_bf16, grid, dim3(256), 0, s, a, gu, f, ids ? *ids : a, ids ? 1 : 0, d);
+}
+
 // up to four bf16 matrices against the same single column (a decode step's q / k / v / gate projections) in one launch: the workgroups are dealt over
 // the matrices' rows, four rows each, the waves taking slices of K (k_mul_mat_f16_gqa_long's form and arithmetic)
 __global__ void __launch_bounds__(256) k_matvec_bf16_multi(const matvec_multi mm, const char * __restrict__ x, const int64_t K) {

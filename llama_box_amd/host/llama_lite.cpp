@@ -3043,10 +3043,17 @@ static ggml_tensor * build_moe_grouped(ggml_context * ctx, ggml_cgraph * gf, con
     return named(out, "ffn_moe_out", il);
 }
 
+// a decode step's gate and up rows keep their few bytes to the graph's end: the down projection that takes the activation as its prologue reads them while it writes its own result (left to
+// itself, the allocator would hand their block to that result)
+static ggml_tensor * keep_small(ggml_tensor * gu) {
+    if (ggml_nrows(gu) <= 8) ggml_set_output(gu);
+    return gu;
+}
+
 // silu-gated feed-forward over a projection that holds the gate rows, then the up rows
 static ggml_tensor * build_gated_pair(ggml_context * ctx, ggml_tensor * w_gate_up, ggml_tensor * w_down, ggml_tensor * cur, const char * name, int run) {
     const std::string n = name;
-    ggml_tensor * gu = named(ggml_mul_mat(ctx, w_gate_up, cur), (n + "_gate_up").c_str(), run);
+    ggml_tensor * gu = keep_small(named(ggml_mul_mat(ctx, w_gate_up, cur), (n + "_gate_up").c_str(), run));
     return named(ggml_mul_mat(ctx, w_down, named(ggml_swiglu(ctx, gu), (n + "_act").c_str(), run)), (n + "_out").c_str(), run);
 }
 
@@ -3067,7 +3074,7 @@ static ggml_tensor * build_moe_sigmoid(ggml_context * ctx, ggml_cgraph * gf, con
     ggml_build_forward_expand(gf, w);  // (the weights before the experts' products: the router is then one run of nodes, which the backend takes as one launch)
     w = ggml_reshape_3d(ctx, w, 1, c.n_top, T);
     ggml_tensor * gu = named(ggml_mul_mat_id(ctx, L.ffn_gate_up_exps, ggml_reshape_3d(ctx, cur, E, 1, T), sel), "ffn_moe_gate_up", run);  // [2 ff, n_top, T]: gate rows, then up rows
-    if (c.moe_scale_in) gu = named(ggml_mul(ctx, gu, w), "ffn_moe_gate_up_weighted", run);  // (the two products of w h are w times those of h)
+    if (c.moe_scale_in) gu = named(ggml_mul(ctx, keep_small(gu), w), "ffn_moe_gate_up_weighted", run);  // (the two products of w h are w times those of h)
     gu = ggml_reshape_2d(ctx, gu, 2 * FF, c.n_top * T);
     ggml_tensor * act = named(c.moe_limit > 0.0f ? ggml_swiglu_oai(ctx, gu, nullptr, 1.702f, c.moe_limit) : ggml_swiglu(ctx, gu), "ffn_moe_act", run);
     ggml_tensor * down = named(ggml_mul_mat_id(ctx, L.ffn_down_exps, ggml_reshape_3d(ctx, act, FF, c.n_top, T), sel), "ffn_moe_down", run);  // [E, n_top, T]

@@ -708,6 +708,42 @@ def test_attention_with_sinks_over_windows_with_kept_tokens(backend, H, n_q, n_k
     assert np.abs(got - ref).max() <= (2e-5 if kv_type == L.F32 else 2e-3) * max(1.0, np.abs(ref).max())
 
 
+@pytest.mark.parametrize("ff,width,used,experts,T_", [(1024, 96, 1, 1, 1), (2752, 70, 1, 1, 1), (1000, 50, 1, 1, 1), (520, 33, 2, 5, 1), (704, 64, 3, 4, 3), (256, 40, 1, 3, 2), (264, 12, 4, 4, 1), (1376, 24, 2, 3, 9)])
+def test_gated_activation_inside_the_down_projection(backend, H, ff, width, used, experts, T_):
+    """a decode step's feed-forward: SwiGLU (of rows that carry a factor each) -> bf16 product, as one launch and as the graph's own nodes: the same bits, and the reference's numbers"""
+    rng = np.random.default_rng(ff + width)
+    gu = rng.standard_normal((T_, used, 2 * ff)).astype(np.float32)
+    w = rng.uniform(0.1, 1.0, (T_, used, 1)).astype(np.float32)
+    W = R.bf16_round(rng.standard_normal((experts, width, ff)) / np.sqrt(ff))
+    ids = np.stack([rng.permutation(experts)[:used] for _ in range(T_)]).astype(np.int32)
+    one = experts == 1
+    bits = (W.astype(np.float32).view(np.uint32) >> 16).astype(np.uint16)
+    got, fused = {}, {}
+    for fusion in (1, 0):
+        backend.set_option("fusion", fusion)
+
+        def build(g):
+            tw = g.new(L.BF16, [ff, width] if one else [ff, width, experts], bits)
+            x = H.ggml_scale(g.ctx, g.new(L.F32, [2 * ff, used, T_], gu), 1.0)
+            if one:
+                return H.ggml_mul_mat(g.ctx, tw, H.ggml_swiglu(g.ctx, H.ggml_reshape_2d(g.ctx, x, 2 * ff, 1)))
+            sel = g.new(L.I32, [used, T_], ids)
+            y = H.ggml_mul(g.ctx, x, g.new(L.F32, [1, used, T_], w))
+            act = H.ggml_swiglu(g.ctx, H.ggml_reshape_2d(g.ctx, y, 2 * ff, used * T_))
+            return H.ggml_mul_mat_id(g.ctx, tw, H.ggml_reshape_3d(g.ctx, act, ff, used, T_), sel)
+
+        before = backend.stat("fused_nodes")
+        got[fusion] = run(backend, build)[0].reshape(T_, used, width)
+        fused[fusion] = backend.stat("fused_nodes") - before
+    backend.set_option("fusion", 1)
+    assert np.array_equal(got[0], got[1])
+    x = gu.astype(np.float64) * (1.0 if one else w.astype(np.float64))
+    act = R.bf16_round(R.silu(x[..., :ff]) * x[..., ff:])
+    ref = np.stack([[W[0 if one else ids[t, u]] @ act[t, u] for u in range(used)] for t in range(T_)])
+    assert np.abs(got[1] - ref).max() <= 4e-3 * np.abs(ref).max()
+    assert fused[0] == 0 and (fused[1] > 0) == (not one or width >= 64)
+
+
 # ------------------------------------------------------------------------------------------------ the program, and random configurations
 def test_trace_run_command_line(tmp_path):
     cfg = cfg_b()
